@@ -333,3 +333,89 @@ def load_moe_checkpoint(model_dir: str, capacity: int = 1024):
         f.close()
     native.sync()
     return cfg, w
+
+
+# ---------------------------------------------------------------- layer-list decoders (architecture "Pusavik")
+#
+# config.json lists the layers (`layers`: type, mixer, mlp), the looped range (`loop`), `embedding.scale`, `norm.eps`,
+# `vocab` and `width`; tensors are bf16, [out, in].  The low-rank width of the queries may be left to the tensor's shape.
+
+def layer_config_from_json(c: dict, shapes: Dict[str, Tuple[int, ...]], act: int = 16):
+    """LayerConfig of a parsed config.json; `shapes` are the checkpoint's tensor shapes."""
+    from .layer_decoder import Experts, Layer, LatentAttention, LayerConfig, Mamba2
+    layers = []
+    for i, l in enumerate(c["layers"]):
+        m, f = l["mixer"], l.get("mlp")
+        if l["type"] == "latent_attention":
+            rot = m["rot"]
+            mixer = LatentAttention(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                                    kv_rank=int(m["kv_rank"]), q_rank=int(m.get("q_rank") or shapes[f"l{i}.mix.dq"][0]),
+                                    window=int(m["mask"]["size"]), scale=float(m["scale"]), rot_base=float(rot["base"]),
+                                    rot_dims=int(rot.get("dims", m["rot_dim"])))
+        elif l["type"] == "mamba2":
+            mixer = Mamba2(heads=int(m["heads"]), vdim=int(m["vdim"]), state=int(m["state"]), groups=int(m["groups"]),
+                           conv=int(m["conv"]), norm_groups=int(m["norm_groups"]))
+        else:
+            raise ValueError(f"layer {i}: unknown mixer type {l['type']!r}")
+        mlp = None
+        if f is not None:
+            if f.get("kind", "moe") != "moe":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+            r = f["router"]
+            mlp = Experts(experts=int(r["experts"]), identity=int(r.get("identity") or 0), top=int(r["top"]), ff=int(f["expert"]["ff"]))
+        layers.append(Layer(mixer, mlp))
+    loop = c.get("loop") or {}
+    return LayerConfig(width=int(c["width"]), vocab=int(c["vocab"]), layers=layers, eps=float(c["norm"]["eps"]),
+                       embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)), loop_start=int(loop.get("start", 0)),
+                       loop_stop=int(loop.get("stop", 0)), loop_times=int(loop.get("times", 1)), act=act)
+
+
+def layer_config_to_json(cfg) -> dict:
+    layers = []
+    for l in cfg.layers:
+        m, f = l.mixer, l.mlp
+        if m.kind == "latent_attention":
+            mixer = dict(heads=m.heads, dim=m.dim, rot_dim=m.rot_dim, vdim=m.vdim, kv_rank=m.kv_rank, q_rank=m.q_rank,
+                         mask=dict(size=m.window), scale=m.scale, rot=dict(base=m.rot_base, dims=m.rot_dims))
+        else:
+            mixer = dict(heads=m.heads, vdim=m.vdim, state=m.state, groups=m.groups, conv=m.conv, norm_groups=m.norm_groups)
+        mlp = None if f is None else dict(kind="moe", expert=dict(ff=f.ff), router=dict(experts=f.experts, identity=f.identity, top=f.top))
+        layers.append(dict(type=m.kind, mixer=mixer, mlp=mlp))
+    out = dict(architecture="Pusavik", vocab=cfg.vocab, width=cfg.width, norm=dict(eps=cfg.eps),
+               embedding=dict(scale=cfg.embed_scale), layers=layers)
+    if cfg.looped:
+        out["loop"] = dict(start=cfg.loop_start, stop=cfg.loop_stop, times=cfg.loop_times)
+    return out
+
+
+def save_layer_checkpoint(model_dir: str, cfg, tensors: Dict[str, np.ndarray]) -> None:
+    """config.json + model.safetensors from bf16 bit patterns (layer_decoder.random_tensors)."""
+    os.makedirs(model_dir, exist_ok=True)
+    write_safetensors(os.path.join(model_dir, "model.safetensors"), [(n, "BF16", a.shape, a) for n, a in tensors.items()])
+    json.dump(layer_config_to_json(cfg), open(os.path.join(model_dir, "config.json"), "w"), indent=1)
+
+
+def load_layer_checkpoint(model_dir: str, act: int = 16):
+    """(LayerConfig, LayerWeights) of a layer-list model; every tensor's dtype and shape is checked against the config."""
+    from .layer_decoder import LayerWeights, tensor_shapes
+    files = [SafetensorsFile(os.path.join(model_dir, f)) for f in sorted(os.listdir(model_dir)) if f.endswith(".safetensors")]
+    if not files:
+        raise FileNotFoundError(f"no .safetensors file in {model_dir}")
+    where = {name: f for f in files for name in f.tensors}
+    cfg = layer_config_from_json(json.load(open(os.path.join(model_dir, "config.json"))),
+                                 {n: tuple(f.tensors[n]["shape"]) for n, f in where.items()}, act)
+    for name, shape in tensor_shapes(cfg).items():
+        if name not in where:
+            raise KeyError(f"checkpoint has no tensor {name}")
+        t = where[name].tensors[name]
+        if t["dtype"] != "BF16" or tuple(t["shape"]) != shape:
+            raise ValueError(f"{name}: {t['dtype']} {tuple(t['shape'])}, expected BF16 {shape}")
+
+    def get(name: str) -> np.ndarray:
+        data, _, shape = where[name].raw(name)
+        return np.frombuffer(data.tobytes(), np.uint16).reshape(shape)
+
+    w = LayerWeights.from_tensors(cfg, get)
+    for f in files:
+        f.close()
+    return cfg, w

@@ -1,4 +1,4 @@
-// Greedy argmax over bf16 logits as packed 64-bit candidates, shared by the stand-alone argmax launch and by the
+// Greedy argmax over bf16 or fp32 logits as packed 64-bit candidates, shared by the stand-alone argmax launch and by the
 // LM-head GEMV that selects the token itself.
 //
 // A candidate is (order-preserving key of the logit << 32) | ~index: the maximum of the packed values is the largest
@@ -29,8 +29,11 @@ __device__ __forceinline__ uint32_t order_key(float v) {
     return (u & 0x80000000u) ? ~u : (u | 0x80000000u);
 }
 
+__device__ __forceinline__ uint64_t argmax_candidate_f32(float logit, uint32_t index) {
+    return ((uint64_t)order_key(logit) << 32) | (uint32_t)(~index);
+}
 __device__ __forceinline__ uint64_t argmax_candidate(uint32_t bf16_bits, uint32_t index) {
-    return ((uint64_t)order_key(bf16_bits_to_f32((uint16_t)bf16_bits)) << 32) | (uint32_t)(~index);
+    return argmax_candidate_f32(bf16_bits_to_f32((uint16_t)bf16_bits), index);
 }
 
 // Called by all BLOCK threads of every block of the launch, each with the best candidate it has seen (0: none).

@@ -215,6 +215,7 @@ struct EmbedArgs {
     uint32_t vocab, hidden, bits, group;
     float out_scale;
     uint16_t* x;
+    uint32_t x_stride, x32;  // x32: x holds fp32 rows
 };
 
 // x = T(embed[token] * scale); quantised rows unpack (word >> ((d % lanes) * bits)) & mask
@@ -234,11 +235,13 @@ __global__ __launch_bounds__(256) void embed_lookup_kernel(const EmbedArgs a) {
         const size_t g = (size_t)token * (a.hidden / a.group) + d / a.group;
         val = (float)qv * bf16_bits_to_f32(a.scales[g]) + bf16_bits_to_f32(a.biases[g]);
     }
-    a.x[(size_t)tr * a.hidden + d] = (uint16_t)f32_to_bf16_bits(val * a.out_scale);
+    const size_t at = (size_t)tr * a.x_stride + d;
+    if (a.x32) reinterpret_cast<float*>(a.x)[at] = val * a.out_scale;
+    else a.x[at] = (uint16_t)f32_to_bf16_bits(val * a.out_scale);
 }
 
 fk_status plan_embed(const fk_weight* E, const uint32_t* token_ptr, uint32_t token_imm, float out_scale,
-                     uint16_t* x, Launch* out, uint32_t rows) {
+                     uint16_t* x, Launch* out, uint32_t rows, uint32_t x_stride, bool x32) {
     const DeviceFacts* dev;
     FK_TRY(device_facts(&dev));
     if (!E || !E->w || !x) return set_error(FK_ERR_INVALID, "embed: null pointer");
@@ -253,6 +256,8 @@ fk_status plan_embed(const fk_weight* E, const uint32_t* token_ptr, uint32_t tok
     a.vocab = E->n; a.hidden = E->k; a.bits = E->bits; a.group = E->group;
     a.out_scale = out_scale;
     a.x = x;
+    a.x_stride = x_stride ? x_stride : E->k;
+    a.x32 = x32 ? 1u : 0u;
     if (rows == 0 || rows > 65535 || (rows > 1 && !token_ptr))
         return set_error(FK_ERR_INVALID, "embed: rows need a device token array");
     out->func = reinterpret_cast<const void*>(&embed_lookup_kernel);
@@ -266,7 +271,7 @@ fk_status plan_embed(const fk_weight* E, const uint32_t* token_ptr, uint32_t tok
 // ---------------------------------------------------------------- argmax
 struct ArgmaxArgs {
     const uint16_t* logits;
-    uint32_t n;
+    uint32_t n, logits32;  // logits32: fp32 values
     ArgmaxTail tail;
 };
 
@@ -277,14 +282,14 @@ __global__ __launch_bounds__(256) void argmax_kernel(const ArgmaxArgs a) {
     __shared__ uint32_t is_last;
     uint64_t best = 0;
     for (uint32_t i = blockIdx.x * 256 + threadIdx.x; i < a.n; i += gridDim.x * 256) {
-        const uint64_t cand = argmax_candidate(a.logits[i], i);
+        const uint64_t cand = a.logits32 ? argmax_candidate_f32(reinterpret_cast<const float*>(a.logits)[i], i) : argmax_candidate(a.logits[i], i);
         best = cand > best ? cand : best;
     }
     argmax_block_finish<256>(a.tail, best, sm, &is_last);
 }
 
 fk_status plan_argmax(const uint16_t* logits, uint32_t n, uint32_t* next_token, uint32_t* history,
-                      uint32_t* hist_counter, uint32_t hist_capacity, void* workspace, Launch* out) {
+                      uint32_t* hist_counter, uint32_t hist_capacity, void* workspace, Launch* out, bool logits32) {
     const DeviceFacts* dev;
     FK_TRY(device_facts(&dev));
     if (!logits || !next_token || !workspace) return set_error(FK_ERR_INVALID, "argmax: null pointer");
@@ -293,7 +298,7 @@ fk_status plan_argmax(const uint16_t* logits, uint32_t n, uint32_t* next_token, 
     if (grid > 160) grid = 160;
     ArgmaxArgs a;
     memset(&a, 0, sizeof(a));
-    a.logits = logits; a.n = n; a.tail.next_token = next_token;
+    a.logits = logits; a.n = n; a.logits32 = logits32 ? 1u : 0u; a.tail.next_token = next_token;
     a.tail.history = history; a.tail.hist_counter = hist_counter; a.tail.hist_capacity = hist_capacity;
     a.tail.counter = reinterpret_cast<uint32_t*>(workspace);
     a.tail.partial = reinterpret_cast<uint64_t*>(reinterpret_cast<char*>(workspace) + 8);

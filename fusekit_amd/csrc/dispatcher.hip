@@ -26,6 +26,7 @@
 #include "decode_token.hpp"
 #include "fk_host.hpp"
 #include "fk_json.hpp"
+#include "layered.hpp"
 #include "xcd_layer.hpp"
 
 namespace fk {
@@ -134,10 +135,12 @@ fk_status plan_embed_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     const uint32_t rows = d.u("rows", 1);  // active_m > 1: one token id and one output row per active row
     if (rows == 0) return set_error(FK_ERR_INVALID, d.kernel + ": rows must be at least 1");
     FK_TRY(need_bytes(d, 0, (size_t)rows * 4));
-    FK_TRY(need_bytes(d, n - 1, (size_t)rows * hidden * 2));
+    const uint32_t out_bits = d.u("out_bits", 16), stride = d.u("x_row_stride", hidden);   // 32: an fp32 residual stream
+    if ((out_bits != 16 && out_bits != 32) || stride < hidden) return set_error(FK_ERR_INVALID, d.kernel + ": bad out_bits / x_row_stride");
+    FK_TRY(need_bytes(d, n - 1, ((size_t)(rows - 1) * stride + hidden) * (out_bits / 8)));
     all_but_last(n, 1, rw);
     return plan_embed(&E, arg_ptr<const uint32_t>(d, 0), 0, (float)d.param("output_scale", 1.0),
-                      arg_ptr<uint16_t>(d, n - 1), l, rows);
+                      arg_ptr<uint16_t>(d, n - 1), l, rows, stride, out_bits == 32);
 }
 
 // x, [norm_w], W_q, W_k, W_v, [s_q, s_k, s_v, b_q, b_k, b_v], [bias_q, bias_k, bias_v], q, k, v
@@ -1468,8 +1471,9 @@ fk_status plan_qgemm_swiglu_d(const Dispatch& d, Launch* l, SlotRW* rw) {
 fk_status plan_argmax_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     const bool hist = d.args.size() == 5;
     FK_TRY(need_args(d, hist ? 5 : 3));
-    const uint32_t vocab = d.u("vocab");
-    FK_TRY(need_bytes(d, 0, (size_t)vocab * 2));
+    const uint32_t vocab = d.u("vocab"), logits_bits = d.u("logits_bits", 16);   // 32: fp32 logits
+    if (logits_bits != 16 && logits_bits != 32) return set_error(FK_ERR_UNSUPPORTED, d.kernel + ": logits_bits must be 16 or 32");
+    FK_TRY(need_bytes(d, 0, (size_t)vocab * (logits_bits / 8)));
     FK_TRY(need_bytes(d, 1, 4));
     FK_TRY(need_bytes(d, 2, kArgmaxWorkspaceBytes));
     uint32_t cap = 0;
@@ -1484,8 +1488,10 @@ fk_status plan_argmax_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     }
     return plan_argmax(arg_ptr<const uint16_t>(d, 0), vocab, arg_ptr<uint32_t>(d, 1),
                        hist ? arg_ptr<uint32_t>(d, 3) : nullptr, hist ? arg_ptr<uint32_t>(d, 4) : nullptr, cap,
-                       d.args[2].ptr, l);
+                       d.args[2].ptr, l, logits_bits == 32);
 }
+
+#include "families_layered.hpp"
 
 struct Family {
     const char* prefix;
@@ -1544,6 +1550,16 @@ const Family kFamilies[] = {
     {"fusekit_xcd_mla_block", plan_xcd_mla_d},
     {"fusekit_read_reduce", plan_read_reduce_d},
     {"fusekit_route_order", plan_route_order_d},
+    {"fusekit_residual_norm", plan_residual_norm_d},
+    {"fusekit_group_norm", plan_group_norm_d},
+    {"fusekit_dense", plan_dense_d},
+    {"fusekit_route_rows", plan_route_rows_d},
+    {"fusekit_route_group", plan_route_group_d},
+    {"fusekit_experts", plan_experts_d},
+    {"fusekit_latent_store", plan_latent_store_d},
+    {"fusekit_latent_attn", plan_latent_attn_d},
+    {"fusekit_ssm_conv", plan_ssm_conv_d},
+    {"fusekit_ssm_scan", plan_ssm_scan_d},
 };
 
 const Family* find_family(const std::string& kernel) {

@@ -1,0 +1,252 @@
+// Dispatch families of the layer-list decoder (layered.hpp).  Included by dispatcher.hip inside its anonymous
+// namespace, where Dispatch, SlotRW and the slot checks live.  Slots are listed in order, optional ones in brackets
+// with the parameter that announces them; `act` (16 or 32) is the width of an activation element.  Row strides are
+// elements of padded rows (multiples of 64).
+
+// Walks the slots of a dispatch: checks sizes, records the access, remembers the first error.
+struct SlotCursor {
+    const Dispatch& d;
+    SlotRW* rw;
+    size_t at = 0;
+    fk_status status = FK_OK;
+
+    void* take(uint64_t bytes, bool read, bool write) {
+        const size_t s = at++;
+        if (status != FK_OK) return nullptr;
+        if (s >= d.args.size()) {
+            status = set_error(FK_ERR_INVALID, d.kernel + ": expected more than " + std::to_string(d.args.size()) + " buffers");
+            return nullptr;
+        }
+        if (!d.args[s].ptr || d.args[s].nbytes == 0) {
+            status = set_error(FK_ERR_INVALID, d.kernel + ": buffer slot " + std::to_string(s) + " is null or empty");
+            return nullptr;
+        }
+        status = need_bytes(d, s, (size_t)bytes);
+        if (read) rw->reads.push_back((uint32_t)s);
+        if (write) rw->writes.push_back((uint32_t)s);
+        return d.args[s].ptr;
+    }
+    template <typename T = void>
+    const T* in(uint64_t bytes) { return (const T*)take(bytes, true, false); }
+    template <typename T = void>
+    T* out(uint64_t bytes) { return (T*)take(bytes, false, true); }
+    template <typename T = void>
+    T* inout(uint64_t bytes) { return (T*)take(bytes, true, true); }
+    fk_status end() {
+        if (status == FK_OK && at != d.args.size())
+            return set_error(FK_ERR_INVALID, d.kernel + ": expected " + std::to_string(at) + " buffers, got " + std::to_string(d.args.size()));
+        return status;
+    }
+};
+
+uint64_t act_bytes(uint32_t act) { return act == 32 ? 4 : 2; }
+// Bytes from the first element of row 0 to the last valid one of row rows - 1.
+uint64_t rows_bytes(uint64_t rows, uint64_t ld, uint64_t width, uint64_t elem) { return ((rows - 1) * ld + width) * elem; }
+
+// x, [mix: has_mix], [routes, weight, index, prev: top > 0], [step: has_step], [w1, h1: has_h1], [w2, h2: has_h2]
+//   {rows, width, ld, act, eps, top, experts}
+fk_status plan_residual_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    ResidualNormArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.width = d.u("width"); a.ldx = d.u("ld", a.width); a.top = d.u("top"); a.experts = d.u("experts");
+    a.eps = (float)d.param("eps", 1e-6);
+    if (!a.rows || !a.width) return set_error(FK_ERR_INVALID, d.kernel + ": rows / width parameters missing");
+    const uint64_t x4 = (uint64_t)a.rows * a.ldx * 4, xa = (uint64_t)a.rows * a.ldx * act_bytes(act);
+    SlotCursor s{d, rw};
+    a.x = s.inout<float>(x4);
+    if (d.u("has_mix")) a.mix = s.in<float>(x4);
+    if (a.top) {
+        a.routes = s.in(xa * a.top);
+        a.weight = s.in<float>((uint64_t)a.rows * a.top * 4);
+        a.index = s.in<uint32_t>((uint64_t)a.rows * a.top * 4);
+        a.prev = s.in(xa);
+    }
+    if (d.u("has_step")) a.step = s.in<uint16_t>((uint64_t)a.ldx * 2);
+    if (d.u("has_h1")) { a.w1 = s.in<uint16_t>((uint64_t)a.ldx * 2); a.h1 = s.out(xa); }
+    if (d.u("has_h2")) { a.w2 = s.in<uint16_t>((uint64_t)a.ldx * 2); a.h2 = s.out(xa); }
+    FK_TRY(s.end());
+    return plan_residual_norm(a, act, l);
+}
+
+// x, [z: has_z], w, y   {rows, width, groups=1, ldx, ldz, ldy, x32, act, eps}
+fk_status plan_group_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    GroupNormArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.width = d.u("width"); a.groups = d.u("groups", 1); a.x32 = d.u("x32");
+    a.ldx = d.u("ldx"); a.ldz = d.u("ldz"); a.ldy = d.u("ldy"); a.eps = (float)d.param("eps", 1e-6);
+    if (!a.rows || !a.width || a.ldx < a.width || a.ldy < a.width) return set_error(FK_ERR_INVALID, d.kernel + ": rows / width / strides missing");
+    SlotCursor s{d, rw};
+    a.x = s.in(rows_bytes(a.rows, a.ldx, a.width, a.x32 ? 4 : act_bytes(act)));
+    if (d.u("has_z")) a.z = s.in(rows_bytes(a.rows, a.ldz, a.width, act_bytes(act)));
+    a.w = s.in<uint16_t>((uint64_t)a.width * 2);
+    a.y = s.out(rows_bytes(a.rows, a.ldy, a.width, act_bytes(act)));
+    FK_TRY(s.end());
+    return plan_group_norm(a, act, l);
+}
+
+// x, w, [row_base: ring > 0], y   {rows, n, k, ldx, ldw, ldy, batch=1, xb, wb, yb, y32, transposed, ring, row_back, act}
+fk_status plan_dense_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    DenseArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.m = d.u("rows", 1); a.n = d.u("n"); a.k = d.u("k"); a.ldx = d.u("ldx", a.k); a.ldw = d.u("ldw", a.k); a.ldy = d.u("ldy");
+    a.batch = d.u("batch", 1);
+    a.xb = (uint64_t)d.param("xb", 0); a.wb = (uint64_t)d.param("wb", 0); a.yb = (uint64_t)d.param("yb", 0);
+    a.y32 = d.u("y32"); a.transposed = d.u("transposed"); a.ring = d.u("ring"); a.row_back = d.u("row_back");
+    if (!a.m || !a.n || !a.k || !a.batch) return set_error(FK_ERR_INVALID, d.kernel + ": rows / n / k parameters missing");
+    const uint64_t e = act_bytes(act), ye = a.y32 ? 4 : e;
+    SlotCursor s{d, rw};
+    a.x = s.in(((a.batch - 1) * a.xb + (uint64_t)((a.ring ? a.ring : a.m) - 1) * a.ldx + a.k) * e);
+    a.w = s.in<uint16_t>(((a.batch - 1) * a.wb + (uint64_t)(a.n - 1) * a.ldw + a.k) * 2);
+    if (a.ring) a.row_base = s.in<uint32_t>(4);
+    const uint64_t rows = a.transposed ? a.n : a.m, cols = a.transposed ? a.m : a.n;
+    if (a.ldy < cols && rows > 1) return set_error(FK_ERR_INVALID, d.kernel + ": ldy below the output width");
+    a.y = s.out(((a.batch - 1) * a.yb + (rows - 1) * a.ldy + cols) * ye);
+    FK_TRY(s.end());
+    return plan_dense(a, act, l);
+}
+
+// logits, correction, index, weight   {rows, outputs, top, ld}
+fk_status plan_route_rows_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    RouteArgs a;
+    memset(&a, 0, sizeof(a));
+    a.rows = d.u("rows", 1); a.outputs = d.u("outputs"); a.top = d.u("top"); a.ldl = d.u("ld", a.outputs);
+    if (!a.rows || !a.outputs || a.ldl < a.outputs) return set_error(FK_ERR_INVALID, d.kernel + ": rows / outputs parameters missing");
+    SlotCursor s{d, rw};
+    a.logits = s.in<float>(rows_bytes(a.rows, a.ldl, a.outputs, 4));
+    a.correction = s.in<uint16_t>((uint64_t)a.outputs * 2);
+    a.index = s.out<uint32_t>((uint64_t)a.rows * a.top * 4);
+    a.weight = s.out<float>((uint64_t)a.rows * a.top * 4);
+    FK_TRY(s.end());
+    return plan_route_rows(a, l);
+}
+
+// index, perm, tiles, count   {routes, experts, tile_rows}; tiles holds 16 bytes per tile
+fk_status plan_route_group_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    RouteGroupArgs a;
+    memset(&a, 0, sizeof(a));
+    a.routes = d.u("routes"); a.experts = d.u("experts"); a.tile_rows = d.u("tile_rows", 64);
+    if (!a.routes || !a.experts || !a.tile_rows || d.args.size() != 4) return set_error(FK_ERR_INVALID, d.kernel + ": four buffers and routes / experts / tile_rows needed");
+    a.max_tiles = (uint32_t)(d.args[2].nbytes / 16);
+    SlotCursor s{d, rw};
+    a.index = s.in<uint32_t>((uint64_t)a.routes * 4);
+    a.perm = s.out<uint32_t>((uint64_t)a.routes * 4);
+    a.tiles = s.out<uint32_t>(((uint64_t)a.routes / a.tile_rows + a.experts) * 16);
+    a.count = s.out<uint32_t>(4);
+    FK_TRY(s.end());
+    return plan_route_group(a, l);
+}
+
+// x, wa, [wb: pair], index, [perm, tiles, count: grouped], y
+//   {routes, experts, n, k, ldx, ldw, ldy, x_div, tile_rows, x_rows, act}
+fk_status plan_experts_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    ExpertArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.routes = d.u("routes"); a.experts = d.u("experts"); a.n = d.u("n"); a.k = d.u("k"); a.ldx = d.u("ldx"); a.ldw = d.u("ldw");
+    a.ldy = d.u("ldy"); a.x_div = d.u("x_div", 1); a.tile_rows = d.u("tile_rows", 64);
+    if (!a.routes || !a.experts || !a.n || !a.k || !a.x_div || a.ldy < a.n) return set_error(FK_ERR_INVALID, d.kernel + ": routes / experts / n / k parameters missing");
+    const uint64_t w = (uint64_t)a.experts * a.n * a.ldw * 2;
+    SlotCursor s{d, rw};
+    a.x = s.in((uint64_t)((a.routes - 1) / a.x_div + 1) * a.ldx * act_bytes(act));
+    a.wa = s.in<uint16_t>(w);
+    if (d.u("pair")) a.wb = s.in<uint16_t>(w);
+    a.index = s.in<uint32_t>((uint64_t)a.routes * 4);
+    if (d.u("grouped")) {
+        a.perm = s.in<uint32_t>((uint64_t)a.routes * 4);
+        a.max_tiles = a.routes / a.tile_rows + a.experts;
+        a.tiles = s.in<uint32_t>((uint64_t)a.max_tiles * 16);
+        a.count = s.in<uint32_t>(4);
+    }
+    a.y = s.out(rows_bytes(a.routes, a.ldy, a.n, act_bytes(act)));
+    FK_TRY(s.end());
+    return plan_experts(a, act, l);
+}
+
+// kv, norm, freq, cache, q, offset   {rows, rank, rank_ld, ldkv, ldc, ring, heads, hs, dim_ld, rot, rot_dims, ldq, eps, act}
+fk_status plan_latent_store_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    LatentStoreArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.rank = d.u("rank"); a.rank_ld = d.u("rank_ld"); a.ldkv = d.u("ldkv"); a.ldc = d.u("ldc"); a.ring = d.u("ring");
+    a.heads = d.u("heads"); a.hs = d.u("hs"); a.dim_ld = d.u("dim_ld"); a.rot = d.u("rot"); a.rot_dims = d.u("rot_dims", a.rot); a.ldq = d.u("ldq");
+    a.eps = (float)d.param("eps", 1e-6);
+    if (!a.rows || !a.rank || !a.heads || a.ldkv < a.rank + a.rot || a.hs < a.dim_ld + a.rot || a.ldq < a.heads * a.hs)
+        return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.kv = s.in<float>(rows_bytes(a.rows, a.ldkv, a.rank + a.rot, 4));
+    a.norm = s.in<uint16_t>((uint64_t)a.rank * 2);
+    a.freq = s.in<double>(a.rot_dims >= 2 ? (uint64_t)(a.rot_dims / 2) * 8 : 1);
+    a.cache = s.inout((uint64_t)a.ring * a.ldc * act_bytes(act));
+    a.q = s.inout(rows_bytes(a.rows, a.ldq, a.heads * a.hs, act_bytes(act)));
+    a.offset = s.in<uint32_t>(4);
+    FK_TRY(s.end());
+    return plan_latent_store(a, act, l);
+}
+
+// qa, q, cache, sink, offset, out   {rows, heads, hs, dim_ld, rot, rank, rank_ld, ldc, ldq, ring, window, scale, act}
+fk_status plan_latent_attn_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    LatentAttnArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.hs = d.u("hs"); a.dim_ld = d.u("dim_ld"); a.rot = d.u("rot"); a.rank = d.u("rank"); a.rank_ld = d.u("rank_ld");
+    a.ldc = d.u("ldc"); a.ldq = d.u("ldq"); a.ring = d.u("ring"); a.window = d.u("window"); a.scale = (float)d.param("scale", 1.0);
+    if (!a.rows || !a.heads || !a.rank_ld || a.hs < a.dim_ld + a.rot || a.ldq < a.heads * a.hs) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    const uint64_t lat = (uint64_t)a.rows * a.heads * a.rank_ld * act_bytes(act);
+    SlotCursor s{d, rw};
+    a.qa = s.in(lat);
+    a.q = s.in(rows_bytes(a.rows, a.ldq, a.heads * a.hs, act_bytes(act)));
+    a.cache = s.in((uint64_t)a.ring * a.ldc * act_bytes(act));
+    a.sink = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.offset = s.in<uint32_t>(4);
+    a.out = s.out(lat);
+    FK_TRY(s.end());
+    return plan_latent_attn(a, act, l);
+}
+
+// u, w, b, hist, offset, y   {rows, channels, taps, ldu, ldy, ldh, act}
+fk_status plan_ssm_conv_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    SsmConvArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.channels = d.u("channels"); a.taps = d.u("taps"); a.ldu = d.u("ldu"); a.ldy = d.u("ldy"); a.ldh = d.u("ldh");
+    if (!a.rows || !a.channels || !a.taps || a.ldy < a.channels || a.ldh < a.channels) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    const uint64_t e = act_bytes(act);
+    SlotCursor s{d, rw};
+    a.u = s.in(rows_bytes(a.rows, a.ldu, a.channels, e));
+    a.w = s.in<uint16_t>((uint64_t)a.channels * a.taps * 2);
+    a.b = s.in<uint16_t>((uint64_t)a.channels * 2);
+    a.hist = s.in((uint64_t)a.taps * a.ldh * e);
+    a.offset = s.in<uint32_t>(4);
+    a.y = s.out(rows_bytes(a.rows, a.ldy, a.channels, e));
+    FK_TRY(s.end());
+    return plan_ssm_conv(a, act, l);
+}
+
+// xbc, dt, dt_bias, a_log, d, u, offset, state, hist, y
+//   {rows, heads, groups, n, p, state_ld, ldx, lddt, ldy, ldu, ldh, channels, taps, act}
+fk_status plan_ssm_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    SsmScanArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.groups = d.u("groups"); a.n = d.u("n"); a.p = d.u("p"); a.state_ld = d.u("state_ld");
+    a.ldx = d.u("ldx"); a.lddt = d.u("lddt"); a.ldy = d.u("ldy"); a.ldu = d.u("ldu"); a.ldh = d.u("ldh"); a.channels = d.u("channels"); a.taps = d.u("taps");
+    const uint64_t e = act_bytes(act);
+    if (!a.rows || !a.heads || !a.p || a.channels != a.heads * a.p + 2 * a.groups * a.n || a.ldx < a.channels || a.lddt < a.heads || a.ldh < a.channels)
+        return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.xbc = s.in(rows_bytes(a.rows, a.ldx, a.channels, e));
+    a.dt = s.in<float>(rows_bytes(a.rows, a.lddt, a.heads, 4));
+    a.dt_bias = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.a_log = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.d = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.u = s.in(rows_bytes(a.rows, a.ldu, a.channels, e));
+    a.offset = s.in<uint32_t>(4);
+    a.state = s.inout<float>((uint64_t)a.heads * a.p * a.state_ld * 4);
+    a.hist = s.inout((uint64_t)a.taps * a.ldh * e);
+    a.y = s.out(rows_bytes(a.rows, a.ldy, a.heads * a.p, e));
+    FK_TRY(s.end());
+    return plan_ssm_scan(a, act, l);
+}

@@ -305,13 +305,13 @@ fk_status plan_sdpa_prefill(const uint16_t* q, const uint16_t* cache_k, const ui
                             uint32_t rows, uint32_t kv_len, uint32_t n_heads, uint32_t n_kv, uint32_t head_dim,
                             uint32_t capacity, float scale, Launch* out_launch, const uint32_t* kv_len_ptr = nullptr);
 fk_status plan_embed(const fk_weight* E, const uint32_t* token_ptr, uint32_t token_imm, float out_scale,
-                     uint16_t* x, Launch* out, uint32_t rows = 1);
+                     uint16_t* x, Launch* out, uint32_t rows = 1, uint32_t x_stride = 0, bool x32 = false);
 fk_status plan_rmsnorm_rows(const uint16_t* x, const uint16_t* w, float eps, uint32_t rows, uint32_t hidden, uint16_t* y,
                             Launch* out);
 // workspace: 8 bytes (counter, zeroed once) + 8 bytes per block (<= 160 blocks)
 constexpr size_t kArgmaxWorkspaceBytes = 8 + 8 * 160;
 fk_status plan_argmax(const uint16_t* logits, uint32_t n, uint32_t* next_token, uint32_t* history,
-                      uint32_t* hist_counter, uint32_t hist_capacity, void* workspace, Launch* out);
+                      uint32_t* hist_counter, uint32_t hist_capacity, void* workspace, Launch* out, bool logits32 = false);
 fk_status plan_step_init(uint32_t* step_counter, uint32_t* offset, uint32_t* kv_len, Launch* out,
                          float* rope_tab = nullptr, uint32_t rope_dims = 0, float base_log2 = 0.f);
 fk_status plan_fill_u32(void* p, uint32_t value, size_t count, Launch* out);

@@ -1,0 +1,174 @@
+// Planners and argument blocks of the layer-list decoder: a decoder whose layers are described one by one (a mixer
+// and an optional feed-forward each), with a 32-bit residual stream.
+//
+// Conventions shared by all of them.
+//  * `act` is the width of an activation element: 16 (bf16) or 32 (fp32).  The same kernels serve both; matrices are
+//    bf16 in either case (they are stored so) and accumulation is fp32.
+//  * Rows of matrices and of activations are padded with zeros to a multiple of kRowPad elements (`ld*` is the padded
+//    length), so that no kernel needs a tail along K.  Buffers start as zeros and kernels write valid columns only.
+//  * Positions are device words: row r of a pass is position *offset + r.
+#pragma once
+#include "fk_host.hpp"
+
+namespace fk {
+
+constexpr uint32_t kRowPad = 64;
+
+// x += mixer output + feed-forward output (+ a constant vector), then up to two RMS norms of the new x.
+struct ResidualNormArgs {
+    float* x;               // [rows, ldx]
+    const float* mix;       // [rows, ldx] or null
+    const void* routes;     // [rows * top, ldx] expert outputs (act) or null
+    const float* weight;    // [rows, top] route weights
+    const uint32_t* index;  // [rows, top] chosen experts; >= experts: the identity, whose output is prev
+    const void* prev;       // [rows, ldx] the feed-forward's input (act)
+    const uint16_t* step;   // [width] added as well, or null
+    const uint16_t* w1;     // norm weights [ldx] or null
+    const uint16_t* w2;
+    void* h1;               // [rows, ldx] (act)
+    void* h2;
+    uint32_t rows, width, ldx, top, experts;
+    float eps;
+};
+fk_status plan_residual_norm(const ResidualNormArgs& a, uint32_t act, Launch* out);
+
+// y[r] = x[r] / rms(x[r]) * w in `groups` equal parts, optionally of x * silu(z) (the gate comes before the norm).
+struct GroupNormArgs {
+    const void* x;      // [rows, ldx]; fp32 when x32, else act
+    const void* z;      // [rows, ldz] (act) or null
+    const uint16_t* w;  // [width]
+    void* y;            // [rows, ldy] (act)
+    uint32_t rows, width, groups, ldx, ldz, ldy, x32;
+    float eps;
+};
+fk_status plan_group_norm(const GroupNormArgs& a, uint32_t act, Launch* out);
+
+// y[b][m, n] = x[b][m, k] . w[b][n, k]^T.
+struct DenseArgs {
+    const void* x;
+    const uint16_t* w;
+    void* y;                   // fp32 when y32, else act
+    const uint32_t* row_base;  // with ring: row r of x is row (*row_base + r - row_back) & (ring - 1)
+    uint32_t ring, row_back;   // ring 0: plain rows; rows of negative position are skipped tile by tile
+    uint32_t m, n, k;          // k: padded length of the dot products
+    uint32_t ldx, ldw, ldy, batch;
+    uint64_t xb, wb, yb;       // elements between batches
+    uint32_t y32, transposed;  // transposed: y[b][n, m] (bf16 matrix-core form only)
+};
+fk_status plan_dense(const DenseArgs& a, uint32_t act, Launch* out);
+
+// Router: softmax over all outputs, choice by score + correction, weights = chosen scores over their sum.
+struct RouteArgs {
+    const float* logits;         // [rows, ldl]
+    const uint16_t* correction;  // [outputs]
+    uint32_t* index;             // [rows, top]
+    float* weight;               // [rows, top]
+    uint32_t rows, outputs, top, ldl;
+};
+fk_status plan_route_rows(const RouteArgs& a, Launch* out);
+constexpr uint32_t kMaxRouterOutputs = 1024, kMaxRouterTop = 64;
+
+// The routes of a pass grouped by expert for the tiled expert products: `perm` lists routes expert by expert,
+// `tiles` holds (expert, first place in perm, routes) per tile of `tile_rows` routes, `count` the number of tiles.
+struct RouteGroupArgs {
+    const uint32_t* index;  // [routes]
+    uint32_t* perm;         // [routes]
+    uint32_t* tiles;        // [max_tiles][4]
+    uint32_t* count;
+    uint32_t routes, experts, tile_rows, max_tiles;
+};
+fk_status plan_route_group(const RouteGroupArgs& a, Launch* out);
+
+// One matrix (or a gate / up pair with silu(gate) * up) of the chosen experts.  Route r reads row r / x_div of x.
+struct ExpertArgs {
+    const void* x;          // [.., ldx] (act)
+    const uint16_t* wa;     // [experts][n, ldw]
+    const uint16_t* wb;     // the up matrices, or null
+    const uint32_t* index;  // [routes]
+    void* y;                // [routes, ldy] (act)
+    const uint32_t* perm;   // grouped form (bf16): from fusekit_route_group
+    const uint32_t* tiles;
+    const uint32_t* count;
+    uint32_t routes, experts, n, k, ldx, ldw, ldy, x_div, tile_rows, max_tiles;
+};
+fk_status plan_experts(const ExpertArgs& a, uint32_t act, Launch* out);
+
+// ---- latent attention ----
+// The cache of one layer run is a ring of rows [latent, padded | rotated key part, padded] (act); position p lives in
+// row p & (ring - 1).  A pass writes its rows, then reads the window behind each of its own positions, so a ring of
+// window + rows - 1 positions is enough whatever the length of the sequence.
+struct LatentStoreArgs {
+    const float* kv;          // [rows, ldkv]: latent | key part
+    const uint16_t* norm;     // [rank]
+    const double* freq;       // [rot / 2] radians per position
+    void* cache;              // [ring, ldc]
+    void* q;                  // rows of ldq (act), head h at h * hs: the rot part, at dim_ld, is rotated in place
+    const uint32_t* offset;
+    uint32_t rows, rank, ldkv, ldc, rank_ld, ring, heads, hs, dim_ld, rot, rot_dims, ldq;
+    float eps;
+};
+fk_status plan_latent_store(const LatentStoreArgs& a, uint32_t act, Launch* out);
+
+// Attention in the latent space, one query row after the other: qa = W_uk^T q per head meets the cached latents, the
+// weighted sum of latents is left to W_uv.
+struct LatentAttnArgs {
+    const void* qa;         // [rows, heads, rank_ld]; fp32 when act is 32, else bf16
+    const void* q;          // [rows, ldq] (act), rotated
+    const void* cache;      // [ring, ldc]
+    const uint16_t* sink;   // [heads]
+    void* out;              // [rows, heads, rank_ld] (act)
+    float* part;            // split form: [rows, splits, heads, rank_ld + 2]
+    const uint32_t* offset;
+    uint32_t rows, heads, hs, dim_ld, rot, rank, rank_ld, ldc, ldq, ring, window, splits;
+    float scale;
+};
+fk_status plan_latent_attn(const LatentAttnArgs& a, uint32_t act, Launch* out);
+
+// Attention of a pass with keys and values formed from the latents (bf16): row 0 of k / column 0 of vt is position
+// *offset - (window - 1).
+struct LatentPrefillArgs {
+    const uint16_t* q;      // [rows, ldq], rotated; a head is [dim_ld | rot_ld], zero padded
+    const uint16_t* k;      // [window - 1 + rows, ldk]: unrotated key parts, dim_ld per head
+    const uint16_t* vt;     // [heads * vdim_ld, ldv]: values, transposed
+    const uint16_t* cache;  // [ring, ldc]: the rotated key parts
+    const uint16_t* sink;
+    uint16_t* out;          // [rows, ldo]: heads * vdim_ld
+    const uint32_t* offset;
+    uint32_t rows, heads, dim_ld, rot_ld, vdim_ld, ldq, ldk, ldv, ldo, ldc, rank_ld, ring, window;
+    float scale;
+};
+bool latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld);
+fk_status plan_latent_prefill(const LatentPrefillArgs& a, Launch* out);
+
+// ---- state-space mixer ----
+// conv: y[r, c] = silu(b[c] + sum_k w[c, k] u[r - taps + 1 + k, c]); rows before the pass come from `hist`
+// [taps, ldh], where position p lies in row p % taps.
+struct SsmConvArgs {
+    const void* u;      // [rows, ldu] (act), at the first convolved column
+    const uint16_t* w;  // [channels, taps]
+    const uint16_t* b;  // [channels]
+    const void* hist;   // (act)
+    void* y;            // [rows, ldy] (act)
+    const uint32_t* offset;
+    uint32_t rows, channels, taps, ldu, ldy, ldh;
+};
+fk_status plan_ssm_conv(const SsmConvArgs& a, uint32_t act, Launch* out);
+
+// The recurrence over the rows of a pass, row after row, and the update of the convolution's history.
+struct SsmScanArgs {
+    const void* xbc;          // [rows, ldx] (act) after the convolution: x | B | C
+    const float* dt;          // [rows, lddt] before bias and softplus
+    const uint16_t* dt_bias;  // [heads]
+    const uint16_t* a_log;
+    const uint16_t* d;
+    float* state;             // [heads][vdim][state_ld]
+    void* y;                  // [rows, ldy] (act)
+    const void* u;            // [rows, ldu] (act) and hist [taps, ldh]: the rows to remember
+    void* hist;
+    const uint32_t* offset;
+    uint32_t rows, heads, groups, n, p, state_ld, ldx, lddt, ldy, ldu, ldh, channels, taps;
+};
+fk_status plan_ssm_scan(const SsmScanArgs& a, uint32_t act, Launch* out);
+constexpr uint32_t kMaxSsmState = 256;
+
+}  // namespace fk

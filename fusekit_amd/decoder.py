@@ -20,7 +20,7 @@ import numpy as np
 
 from . import native
 from .native import DeviceBuffer, DeviceWeight, check, lib
-from .runtime import FK_CHUNK, Dispatch, Dispatcher, arg, make_uniforms
+from .runtime import FK_CHUNK, Dispatch, Dispatcher, TokenSteps, arg, make_uniforms
 
 
 @dataclass
@@ -185,7 +185,7 @@ class DecoderWeights:
         return sum(m.nbytes for m in self.mats.values()) + sum(v.nbytes for v in self.vecs.values())
 
 
-class DecoderRuntime:
+class DecoderRuntime(TokenSteps):
     """Scratch arena, KV caches, uniforms and the captured decode graph of one model."""
 
     def __init__(self, cfg: DecoderConfig, weights: DecoderWeights, dispatcher: Optional[Dispatcher] = None,
@@ -419,6 +419,7 @@ class DecoderRuntime:
 
     # -- generation ------------------------------------------------------------------
     def reset(self) -> None:
+        self.position = 0
         for b in (self.step_counter, self.offset, self.kv_len, self.hist_counter):
             b.upload(np.zeros(1, np.uint32))
         if self.xcd:

@@ -26,7 +26,7 @@ import numpy as np
 from . import native
 from .decoder import _synth, quantize_on_device
 from .native import DeviceBuffer, DeviceWeight
-from .runtime import FK_CHUNK, Dispatch, Dispatcher, arg, make_uniforms
+from .runtime import FK_CHUNK, Dispatch, Dispatcher, TokenSteps, arg, make_uniforms
 
 
 @dataclass
@@ -179,7 +179,7 @@ def _rows(W: DeviceWeight, r0: int, r1: int):
     return (arg(W.w, (r1 - r0) * wb, r0 * wb), arg(W.scales, (r1 - r0) * sb, r0 * sb), arg(W.biases, (r1 - r0) * sb, r0 * sb))
 
 
-class MoeRuntime:
+class MoeRuntime(TokenSteps):
     """Scratch arena, KV caches, uniforms and the captured decode graph of one MoE model."""
 
     def __init__(self, cfg: MoeConfig, weights: MoeWeights, dispatcher: Optional[Dispatcher] = None,
@@ -519,6 +519,7 @@ class MoeRuntime:
 
     # -- generation (the dense runtime's loop: prompt with forced tokens, then chunks fed back on the GPU)
     def reset(self) -> None:
+        self.position = 0
         for b in (self.step_counter, self.offset, self.kv_len, self.hist_counter):
             b.upload(np.zeros(1, np.uint32))
         if self.xcd:

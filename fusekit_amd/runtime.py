@@ -101,6 +101,16 @@ class Dispatcher:
         check(lib.fk_dispatch_batch(self.handle, arr, C.c_size_t(len(ds)), C.byref(sec)))
         return sec.value
 
+    def prepare(self, ds: Sequence[Dispatch]):
+        """A task list marshalled once for repeated `dispatch_prepared` calls."""
+        return _marshal(ds) + (len(ds),)
+
+    def dispatch_prepared(self, prepared) -> float:
+        arr, _, n = prepared
+        sec = C.c_double()
+        check(lib.fk_dispatch_batch(self.handle, arr, C.c_size_t(n), C.byref(sec)))
+        return sec.value
+
     def build_graph(self, ds: Sequence[Dispatch], barriers: Optional[Sequence[bool]] = None) -> int:
         arr, keep = _marshal(ds)
         gid = C.c_uint32()
@@ -188,6 +198,26 @@ class Dispatcher:
         check(lib.fk_decode_chunk_host_loop(self.handle, C.c_uint32(gid), C.byref(uniforms),
                                             C.c_uint32(start_offset), tin, C.c_uint32(n), out, C.byref(sec)))
         return list(out), sec.value
+
+
+class TokenSteps:
+    """`step` for runtimes that feed a prompt token by token through their decode graph (bf16 logits)."""
+
+    position = 0
+
+    def step(self, tokens: Sequence[int], want: Sequence[int] = ()) -> np.ndarray:
+        """Runs the sequence's next tokens; logits [len(want), vocab] at the wanted places among them."""
+        c, rows = self.cfg, {}
+        if self.position + len(tokens) > c.capacity:
+            raise ValueError("the sequence exceeds the KV-cache capacity")
+        for k, t in enumerate(tokens):
+            if not 0 <= t < c.vocab:
+                raise ValueError("token ids must lie in 0 .. vocab - 1")
+            self.d.decode_host_loop(self.graph, self.uniforms, self.position, [t])
+            self.position += 1
+            if k in want:
+                rows[k] = (self.logits.to_numpy(np.uint16).astype(np.uint32) << 16).view(np.float32)
+        return np.stack([rows[k] for k in want]) if len(want) else np.empty((0, c.vocab), np.float32)
 
 
 def make_uniforms(token: DeviceBuffer, step_counter: DeviceBuffer, hist_counter: DeviceBuffer,
