@@ -1,13 +1,13 @@
 """python -m fusekit_amd <command>
 
   info                                   the device as the backend sees it (fk_target_describe)
-  generate --model DIR --ids 1,2,3 [--max-tokens N] [--capacity C]
-                                         greedy decode of an mlx-lm format checkpoint (token ids in,
-                                         token ids out; no tokenizer is bundled)
-  export-random --out DIR [--bits 4] [--layers 2] [--moe] ...
+  generate --model DIR --ids 1,2,3 [--max-tokens N] [--capacity C] [--dtype float32]
+                                         greedy decode of a checkpoint (token ids in, token ids out; no
+                                         tokenizer is bundled); config.json chooses the model family
+  export-random --out DIR [--bits 4] [--layers 2] [--moe | --pusavik] ...
                                          write a small random-init model in the mlx-lm file layout (--moe: a
-                                         mixture-of-experts model in the deepseek_v2 layout; generate / patch
-                                         recognise it by config.json's model_type)
+                                         mixture-of-experts model in the deepseek_v2 layout; --pusavik: a
+                                         layer-list model; generate / patch / bench recognise it)
   patch --model DIR [--out DIR/.fusekit] [--prefill-m 32,128] [--capacity C]
                                          the reference's `fusekit patch`: write task_graph.json, manifest.json and
                                          variants/prefill_mN/task_graph.json for a checkpoint
@@ -32,6 +32,7 @@ def main() -> int:
     g.add_argument("--max-tokens", type=int, default=32)
     g.add_argument("--capacity", type=int, default=1024)
     g.add_argument("--artifact", default=None, help="directory written by `patch`")
+    g.add_argument("--dtype", choices=["bfloat16", "float32"], default="bfloat16", help="float32: everything in fp32, where the family has it")
     pa = sub.add_parser("patch")
     pa.add_argument("--model", required=True)
     pa.add_argument("--out", default=None)
@@ -49,6 +50,7 @@ def main() -> int:
     e.add_argument("--vocab", type=int, default=2000)
     e.add_argument("--seed", type=int, default=0)
     e.add_argument("--moe", action="store_true", help="a small mixture-of-experts model with low-rank keys (deepseek_v2 layout)")
+    e.add_argument("--pusavik", action="store_true", help="a small layer-list model: latent attention and Mamba-2 mixers, routed experts")
     from . import bench_cli
     bench_cli.add_arguments(sub)
     args = ap.parse_args()
@@ -61,7 +63,14 @@ def main() -> int:
         print(json.dumps({f: (getattr(t, f).decode() if isinstance(getattr(t, f), bytes) else getattr(t, f))
                           for f, _ in t._fields_}, indent=1))
         return 0
-    from .decoder import DecoderConfig, DecoderRuntime, DecoderWeights
+    if args.cmd == "export-random" and args.pusavik:
+        from .checkpoint import save_layer_checkpoint
+        from .layer_decoder import random_tensors, small_config
+        lc = small_config(width=args.hidden, vocab=args.vocab, heads=args.heads, ff=args.inter)
+        save_layer_checkpoint(args.out, lc, random_tensors(lc, seed=args.seed))
+        print(f"wrote {args.out}/config.json and model.safetensors (Pusavik)")
+        return 0
+    from .decoder import DecoderConfig, DecoderWeights
     if args.cmd == "export-random" and args.moe:
         from .checkpoint import save_moe_checkpoint
         from .moe_decoder import MoeConfig, MoeWeights
@@ -80,45 +89,34 @@ def main() -> int:
         print(f"wrote {args.out}/config.json and model.safetensors")
         return 0
     import os
-    model_type = json.load(open(os.path.join(args.model, "config.json"))).get("model_type", "")
-    if model_type.startswith("deepseek"):   # mixture-of-experts decoder with low-rank keys
-        from .artifact import ArtifactRuntime, write_artifact
-        from .checkpoint import load_moe_checkpoint
-        from .moe_decoder import MoeRuntime
-        cfg, w = load_moe_checkpoint(args.model, capacity=args.capacity)
-        if args.cmd == "patch":
-            rt = MoeRuntime(cfg, w)
-            out = args.out or os.path.join(args.model, ".fusekit")
-            write_artifact(rt, out, os.path.basename(os.path.normpath(args.model)))
-            print(json.dumps({"artifact": out, "tasks": len(rt.tasks), "variants": []}))
-            return 0
-        prompt = [int(t) for t in args.ids.split(",") if t.strip()]
-        if args.artifact:
-            print(json.dumps({"tokens": ArtifactRuntime(args.artifact, w).generate(prompt, args.max_tokens)}))
-            return 0
-        toks, gpu_s, steps = MoeRuntime(cfg, w).generate(prompt, args.max_tokens)
-        print(json.dumps({"tokens": toks, "decode_tok_per_s": round(steps / gpu_s, 1) if gpu_s else None}))
-        return 0
-    from .checkpoint import load_mlx_checkpoint
-    cfg, w = load_mlx_checkpoint(args.model, capacity=args.capacity)
+
+    from . import registry
+    from .artifact import ArtifactRuntime, write_artifact
+    family = registry.family_of(registry.read_config(args.model))
+    act = {"bfloat16": 16, "float32": 32}[getattr(args, "dtype", "bfloat16")]
+    if act not in family.acts:
+        print(f"models of family '{family.name}' do not run in {args.dtype}", file=sys.stderr)
+        return 2
+    cfg, w = family.load(args.model, args.capacity, act)
     if args.cmd == "patch":
-        import os
-        from .artifact import write_artifact
-        from .prefill_variant import PrefillVariant
-        rt = DecoderRuntime(cfg, w)
+        rt = family.runtime(cfg, w)
         out = args.out or os.path.join(args.model, ".fusekit")
-        ms = [int(v) for v in args.prefill_m.split(",") if v.strip()]
-        write_artifact(rt, out, os.path.basename(os.path.normpath(args.model)), prefill_variants=[PrefillVariant(rt, m) for m in ms])
-        print(json.dumps({"artifact": out, "tasks": len(rt.tasks), "variants": [f"prefill_m{m}" for m in ms]}))
+        variants = []
+        if family.name == "dense":
+            from .prefill_variant import PrefillVariant
+            variants = [PrefillVariant(rt, int(v)) for v in args.prefill_m.split(",") if v.strip()]
+        write_artifact(rt, out, os.path.basename(os.path.normpath(args.model)), prefill_variants=variants)
+        print(json.dumps({"artifact": out, "tasks": len(rt.tasks), "variants": [v.name for v in variants]}))
         return 0
     prompt = [int(t) for t in args.ids.split(",") if t.strip()]
     if args.artifact:
-        from .artifact import ArtifactRuntime
         art = ArtifactRuntime(args.artifact, w)
-        print(json.dumps({"tokens": art.generate(prompt, args.max_tokens), "variants": sorted(art.variants)}))
+        out = {"tokens": art.generate(prompt, args.max_tokens)}
+        if family.name == "dense":
+            out["variants"] = sorted(art.variants)
+        print(json.dumps(out))
         return 0
-    rt = DecoderRuntime(cfg, w)
-    toks, gpu_s, steps = rt.generate(prompt, args.max_tokens)
+    toks, gpu_s, steps = family.runtime(cfg, w).generate(prompt, args.max_tokens)
     print(json.dumps({"tokens": toks, "decode_tok_per_s": round(steps / gpu_s, 1) if gpu_s else None}))
     return 0
 

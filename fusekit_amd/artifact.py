@@ -99,7 +99,8 @@ def _parameter_symbols(rt, sym: Dict[int, dict]) -> None:
             sym[W.biases.ptr] = dict(role="external", source_path=path + ".biases", dtype="bfloat16",
                                      shape=lead + [W.n, W.k // W.group], size_bytes=W.biases.nbytes)
     for path, v in rt.w.vecs.items():
-        sym[v.ptr] = dict(role="external", source_path=path, dtype="bfloat16", shape=[v.nbytes // 2], size_bytes=v.nbytes)
+        dtype = getattr(rt.w, "vec_dtype", {}).get(path, "bfloat16")
+        sym[v.ptr] = dict(role="external", source_path=path, dtype=dtype, shape=[v.nbytes // (8 if dtype == "float64" else 2)], size_bytes=v.nbytes)
 
 
 def _resolve(sym: Dict[int, dict], ptr: int):
@@ -146,7 +147,7 @@ def _graph_dict(rt: DecoderRuntime, task_list: List[Dispatch], graph_id: int, sy
                 b.update(scratch_id=scratch_ids[name], role_name=name)
             bindings.append(b)
         m = re.search(r"cache_k\.(\d+)", " ".join(b.get("role_name", "") for b in bindings))
-        lm = [re.match(r"layers\.(\d+)\.", b.get("source_path", "")) for b in bindings]
+        lm = [re.match(r"(?:layers\.|l)(\d+)\.", b.get("source_path", "")) for b in bindings]
         layer = next((int(x.group(1)) for x in lm if x), int(m.group(1)) if m else None)
         kernels = [dict(grid=list(geo.grid[i]), threadgroup=list(geo.threadgroup[i]), lds_bytes=geo.lds_bytes[i])
                    for i in range(geo.n_kernels)]
@@ -207,7 +208,7 @@ def write_artifact(rt: DecoderRuntime, out_dir: str, model_name: str = "syntheti
     manifest = dict(
         schema_version=SCHEMA_VERSION, fusekit_version=BACKEND_VERSION,
         compiled_at=time.strftime("%Y-%m-%dT%H:%M:%SZ", time.gmtime()),
-        model=dict(name=model_name, model_type="moe-decoder" if hasattr(c, "n_experts") else "dense-decoder",
+        model=dict(name=model_name, model_type=getattr(c, "artifact_type", None) or ("moe-decoder" if hasattr(c, "n_experts") else "dense-decoder"),
                    hidden_size=c.hidden, num_hidden_layers=c.n_layers, num_kv_shared_layers=0, num_attention_heads=c.n_heads,
                    num_key_value_heads=getattr(c, "n_kv", c.n_heads), head_dim=getattr(c, "head_dim", None) or c.qk_dim,
                    vocab_size=c.vocab),
@@ -297,7 +298,7 @@ class ArtifactRuntime:
         from .prefill_variant import run_variant
         prompt = list(prompt)
         pos, nxt = 0, None
-        cap = int(self.model_config["capacity"])
+        cap = int(self.model_config.get("capacity", 1 << 31))   # a windowed state does not bound the sequence
         while pos < len(prompt):
             fit = [m for m in self.variants if m <= len(prompt) - pos]
             if not fit:
@@ -310,6 +311,10 @@ class ArtifactRuntime:
         return nxt
 
     def generate(self, prompt, max_tokens: int) -> List[int]:
+        for name, buf in self.scratch.items():   # recurrent states of a new sequence start at zero
+            if name.startswith("state."):
+                native.fill_u32(buf, 0, buf.nbytes // 4)
+        native.sync()
         out = [self.prefill(prompt)]
         offset = len(prompt)
         while len(out) < max_tokens:

@@ -4,7 +4,7 @@ Same arguments and the same `[bench:N] key=value` lines as `fusekit bench` (src/
 src/commands/bench.rs:13-37, scripts/bench.py:131-150): --tokens, --prompt, --repeat, --max-kv-size, --kv-bits,
 --kv-group-size, --raw, --per-kernel, --dump-tokens.  Differences a caller has to know:
 
-  * MODEL is a checkpoint directory (mlx-lm file layout), not a name in a model registry.
+  * MODEL is a checkpoint directory (its config.json chooses the model family), not a name in a model registry.
   * The prompt is tokenised with MODEL/tokenizer.json when it is there (the `tokenizers` package); without one
     the prompt's UTF-8 bytes are the token ids (every vocabulary here has at least 256 entries), or --ids gives
     them directly.
@@ -12,7 +12,6 @@ src/commands/bench.rs:13-37, scripts/bench.py:131-150): --tokens, --prompt, --re
   * --per-kernel prints, after the run, the GPU time of every node of ONE decode step's graph
     (`[fusekit-profile]` lines, aggregate by kernel family first; python/fusekit_runtime/dispatch.py:4732-4790).
 """
-import json
 import os
 import time
 from typing import List
@@ -77,30 +76,23 @@ def run(args) -> int:
     if args.raw:
         raise SystemExit("bench: --raw measures the model through plain mlx-lm; there is no such path on this platform")
     from . import native as fk
-    cfg_json = json.load(open(os.path.join(args.model, "config.json")))
-    moe = cfg_json.get("model_type", "").startswith("deepseek")
+    from . import registry
+    cfg_json = registry.read_config(args.model)
+    family = registry.family_of(cfg_json)
     free0, total = fk.mem_info()
-    vocab = int(cfg_json.get("text_config", cfg_json)["vocab_size"])
+    vocab = registry.vocab_of(cfg_json)
     prompt = _prompt_ids(args, vocab)
     capacity = args.max_kv_size or max(1024, 1 << (len(prompt) + args.tokens - 1).bit_length())
     if len(prompt) + args.tokens > capacity:
         raise SystemExit(f"bench: prompt ({len(prompt)}) + tokens ({args.tokens}) exceed --max-kv-size {capacity}")
     print(f"[bench] model={os.path.abspath(args.model)} mode=fusekit"
           + (" + per-kernel profile" if args.per_kernel else ""), flush=True)
-    if moe:
-        if args.kv_bits:
-            raise SystemExit("bench: the mixture-of-experts runtime keeps a bf16 KV cache (--kv-bits is for dense models)")
-        from .checkpoint import load_moe_checkpoint
-        from .moe_decoder import MoeRuntime
-        cfg, w = load_moe_checkpoint(args.model, capacity=capacity)
-        rt = MoeRuntime(cfg, w)
-    else:
-        from .checkpoint import load_mlx_checkpoint
-        from .decoder import DecoderRuntime
-        cfg, w = load_mlx_checkpoint(args.model, capacity=capacity)
-        if args.kv_bits:
-            cfg.kv_bits, cfg.kv_group = args.kv_bits, args.kv_group_size
-        rt = DecoderRuntime(cfg, w)
+    if args.kv_bits and not family.kv_bits:
+        raise SystemExit(f"bench: models of family '{family.name}' keep a bf16 cache (--kv-bits is for dense models)")
+    cfg, w = family.load(args.model, capacity, 16)
+    if args.kv_bits:
+        cfg.kv_bits, cfg.kv_group = args.kv_bits, args.kv_group_size
+    rt = family.runtime(cfg, w)
     for rep in range(args.repeat):
         rt.reset()
         fk.sync()

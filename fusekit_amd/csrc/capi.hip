@@ -6,6 +6,7 @@
 #include <mutex>
 
 #include "fk_host.hpp"
+#include "layered.hpp"
 #include "xcd_layer.hpp"
 
 namespace fk {
@@ -885,5 +886,8 @@ fk_status fk_xcd_check(void* workspace, fk_stream s) {
     FK_HIP(hipStreamSynchronize((hipStream_t)s));
     return xcd_check_control(workspace);
 }
+
+int fk_latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld) { return latent_prefill_supported(dim_ld, rot_ld, vdim_ld) ? 1 : 0; }
+int fk_ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n) { return ssm_chunk_supported(heads, p, n) ? 1 : 0; }
 
 }  // extern "C"

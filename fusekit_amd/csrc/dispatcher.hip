@@ -1560,6 +1560,8 @@ const Family kFamilies[] = {
     {"fusekit_latent_attn", plan_latent_attn_d},
     {"fusekit_ssm_conv", plan_ssm_conv_d},
     {"fusekit_ssm_scan", plan_ssm_scan_d},
+    {"fusekit_latent_prefill", plan_latent_prefill_d},
+    {"fusekit_ssm_chunk", plan_ssm_chunk_d},
 };
 
 const Family* find_family(const std::string& kernel) {

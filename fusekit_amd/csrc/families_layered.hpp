@@ -234,7 +234,7 @@ fk_status plan_ssm_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.groups = d.u("groups"); a.n = d.u("n"); a.p = d.u("p"); a.state_ld = d.u("state_ld");
     a.ldx = d.u("ldx"); a.lddt = d.u("lddt"); a.ldy = d.u("ldy"); a.ldu = d.u("ldu"); a.ldh = d.u("ldh"); a.channels = d.u("channels"); a.taps = d.u("taps");
     const uint64_t e = act_bytes(act);
-    if (!a.rows || !a.heads || !a.p || a.channels != a.heads * a.p + 2 * a.groups * a.n || a.ldx < a.channels || a.lddt < a.heads || a.ldh < a.channels)
+    if (!a.rows || !a.heads || !a.p || a.channels != a.heads * a.p + 2 * a.groups * a.n || a.ldx < a.channels || a.lddt < a.heads || a.ldh < a.channels || a.ldy < a.heads * a.p)
         return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
     SlotCursor s{d, rw};
     a.xbc = s.in(rows_bytes(a.rows, a.ldx, a.channels, e));
@@ -249,4 +249,53 @@ fk_status plan_ssm_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     a.y = s.out(rows_bytes(a.rows, a.ldy, a.heads * a.p, e));
     FK_TRY(s.end());
     return plan_ssm_scan(a, act, l);
+}
+
+// q, k, vt, cache, sink, offset, out
+//   {rows, heads, dim_ld, rot_ld, vdim_ld, rank_ld, ldq, ldk, ldv, ldo, ldc, ring, window, scale}
+fk_status plan_latent_prefill_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    LatentPrefillArgs a;
+    memset(&a, 0, sizeof(a));
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.dim_ld = d.u("dim_ld"); a.rot_ld = d.u("rot_ld"); a.vdim_ld = d.u("vdim_ld");
+    a.rank_ld = d.u("rank_ld"); a.ldq = d.u("ldq"); a.ldk = d.u("ldk"); a.ldv = d.u("ldv"); a.ldo = d.u("ldo"); a.ldc = d.u("ldc");
+    a.ring = d.u("ring"); a.window = d.u("window"); a.scale = (float)d.param("scale", 1.0);
+    if (!a.rows || !a.heads || !a.window || a.ldq < a.heads * (a.dim_ld + a.rot_ld) || a.ldk < a.heads * a.dim_ld || a.ldo < a.heads * a.vdim_ld ||
+        a.ldc < a.rank_ld + a.rot_ld)
+        return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.q = s.in<uint16_t>(rows_bytes(a.rows, a.ldq, a.heads * (a.dim_ld + a.rot_ld), 2));
+    a.k = s.in<uint16_t>(rows_bytes((uint64_t)a.window - 1 + a.rows, a.ldk, a.heads * a.dim_ld, 2));
+    a.vt = s.in<uint16_t>((uint64_t)a.heads * a.vdim_ld * a.ldv * 2);
+    a.cache = s.in<uint16_t>((uint64_t)a.ring * a.ldc * 2);
+    a.sink = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.offset = s.in<uint32_t>(4);
+    a.out = s.out<uint16_t>(rows_bytes(a.rows, a.ldo, a.heads * a.vdim_ld, 2));
+    FK_TRY(s.end());
+    return plan_latent_prefill(a, l);
+}
+
+// xbc, dt, dt_bias, a_log, d, u, offset, state, hist, y, chunks, decay   (parameters of fusekit_ssm_scan, bf16)
+fk_status plan_ssm_chunk_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    SsmChunkArgs a;
+    memset(&a, 0, sizeof(a));
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.groups = d.u("groups"); a.n = d.u("n"); a.p = d.u("p"); a.state_ld = d.u("state_ld");
+    a.ldx = d.u("ldx"); a.lddt = d.u("lddt"); a.ldy = d.u("ldy"); a.ldu = d.u("ldu"); a.ldh = d.u("ldh"); a.channels = d.u("channels"); a.taps = d.u("taps");
+    if (!a.rows || !a.heads || !a.p || a.channels != a.heads * a.p + 2 * a.groups * a.n || a.ldx < a.channels || a.lddt < a.heads || a.ldh < a.channels || a.ldy < a.heads * a.p)
+        return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    const uint64_t chunks = (a.rows + kSsmChunk - 1) / kSsmChunk;
+    SlotCursor s{d, rw};
+    a.xbc = s.in<uint16_t>(rows_bytes(a.rows, a.ldx, a.channels, 2));
+    a.dt = s.in<float>(rows_bytes(a.rows, a.lddt, a.heads, 4));
+    a.dt_bias = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.a_log = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.d = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.u = s.in<uint16_t>(rows_bytes(a.rows, a.ldu, a.channels, 2));
+    a.offset = s.in<uint32_t>(4);
+    a.state = s.inout<float>((uint64_t)a.heads * a.p * a.state_ld * 4);
+    a.hist = s.inout<uint16_t>((uint64_t)a.taps * a.ldh * 2);
+    a.y = s.out<uint16_t>(rows_bytes(a.rows, a.ldy, a.heads * a.p, 2));
+    a.chunks = s.inout<float>(chunks * a.heads * a.p * a.state_ld * 4);
+    a.decay = s.inout<float>(chunks * a.heads * 4);
+    FK_TRY(s.end());
+    return plan_ssm_chunk(a, l);
 }

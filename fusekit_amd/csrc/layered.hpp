@@ -171,4 +171,24 @@ struct SsmScanArgs {
 fk_status plan_ssm_scan(const SsmScanArgs& a, uint32_t act, Launch* out);
 constexpr uint32_t kMaxSsmState = 256;
 
+// The same in chunks of 64 tokens on the matrix cores (bf16).
+struct SsmChunkArgs {
+    const uint16_t* xbc;
+    const float* dt;
+    const uint16_t* dt_bias;
+    const uint16_t* a_log;
+    const uint16_t* d;
+    float* state;
+    uint16_t* y;
+    const uint16_t* u;
+    uint16_t* hist;
+    const uint32_t* offset;
+    float* chunks;  // [chunks][heads][p][state_ld]
+    float* decay;   // [chunks][heads]
+    uint32_t rows, heads, groups, n, p, state_ld, ldx, lddt, ldy, ldu, ldh, channels, taps;
+};
+constexpr uint32_t kSsmChunk = 64;
+bool ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n);
+fk_status plan_ssm_chunk(const SsmChunkArgs& a, Launch* out);
+
 }  // namespace fk

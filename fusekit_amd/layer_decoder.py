@@ -135,6 +135,8 @@ class LayerConfig:
     loop_times: int = 1
     act: int = 16                # 16: bf16 matrices and activations, 32-bit residual, norms, router, softmax and state; 32: all fp32
     rows_per_pass: int = 2048    # most tokens of one rows pass
+    artifact_type = "layer-list-decoder"
+    tiled: bool = True           # the matrix-core forms of attention, recurrence and experts for portions (False: the row forms)
     fuse: bool = True            # the decode list's fused launches (False: the rows list at one row)
 
     @property
@@ -166,6 +168,16 @@ class LayerConfig:
         for t in range(self.loop_times):
             out += [(i, t if i == self.loop_start else None) for i in range(self.loop_start, self.loop_stop)]
         return out + [(i, None) for i in range(self.loop_stop, n)]
+
+
+def small_config(width: int = 256, vocab: int = 1000, heads: int = 4, ff: int = 96, window: int = 48, **more) -> LayerConfig:
+    """A four-layer model of both mixers with a loop, for examples and tests."""
+    lat = LatentAttention(heads=heads, dim=40, rot_dim=16, vdim=48, kv_rank=72, q_rank=80, window=window, scale=56 ** -0.5,
+                          rot_base=10000.0, rot_dims=16)
+    ssm = Mamba2(heads=2 * heads, vdim=24, state=40, groups=2, conv=3, norm_groups=4)
+    moe = Experts(experts=6, identity=1, top=3, ff=ff)
+    return LayerConfig(width=width, vocab=vocab, layers=[Layer(lat, moe), Layer(ssm, moe), Layer(lat), Layer(ssm, moe)], embed_scale=0.7,
+                       loop_start=1, loop_stop=3, loop_times=2, **more)
 
 
 def tensor_shapes(cfg: LayerConfig) -> Dict[str, Tuple[int, ...]]:
@@ -475,20 +487,48 @@ class LayerRuntime:
                 want("qa", R * m.heads * m.rank_ld * e)
                 want("ol", R * m.heads * m.rank_ld * e)
                 want("att", R * pad(m.heads * m.vdim_ld) * e)
+                if self._long_latent(m, R):
+                    want("kx", (m.window - 1 + R) * m.heads * m.dim_ld * e)
+                    want("vx", m.heads * m.vdim_ld * self._ldv(m) * e)
             else:
                 want("u", R * pad(m.inner + m.channels) * e)
                 want("dt", R * pad(m.heads) * 4)
                 want("xbc", R * pad(m.channels) * e)
                 want("y", R * pad(m.inner) * e)
                 want("g", R * pad(m.inner) * e)
+                if self._long_ssm(m, R):
+                    want("chunks", -(-R // 64) * m.heads * m.vdim * m.state_ld * 4)
+                    want("decay", -(-R // 64) * m.heads * 4)
             if f:
                 want("rl", R * pad(f.outputs) * 4)
                 want("ridx", R * f.top * 4)
                 want("rwt", R * f.top * 4)
                 want("eh", R * f.top * pad(f.ff) * e)
                 want("eo", R * f.top * D * e)
+                want("perm", R * f.top * 4)
+                want("tiles", (R * f.top // 32 + f.experts) * 16)
+                want("tile_count", 4)
         for name, nbytes in need.items():
             self.buf[name] = native.zeros(nbytes)
+
+    # -- which form a portion takes
+    def _long_latent(self, m: LatentAttention, rows: int) -> bool:
+        """Keys and values formed once for the pass (instead of queries carried into the latent space)."""
+        return self.cfg.act == 16 and self.cfg.tiled and rows >= 64 and native.latent_prefill_supported(m.dim_ld, m.rot_ld, m.vdim_ld)
+
+    def _ldv(self, m: LatentAttention) -> int:
+        return pad(m.window - 1 + self.R + 64)
+
+    def _long_ssm(self, m: Mamba2, rows: int) -> bool:
+        """The recurrence in chunks (instead of token after token)."""
+        return self.cfg.act == 16 and self.cfg.tiled and rows >= 64 and native.ssm_chunk_supported(m.heads, m.vdim, m.state)
+
+    def _grouped(self, f: Experts, rows: int) -> int:
+        """Routes per tile of the grouped expert products, 0: route by route."""
+        if self.cfg.act != 16 or not self.cfg.tiled or rows <= 8:
+            return 0
+        per = rows * f.top / f.outputs
+        return 32 if per <= 32 else 64 if per <= 96 else 128
 
     # -- task lists
     def _name(self, kind: str) -> str:
@@ -545,6 +585,17 @@ class LayerRuntime:
                           [arg(b["low"], None, m.q_rank * 4), arg(w.vecs[p + "dkv.norm"]), arg(w.vecs[p + "rot_freq"]), arg(cache), arg(b["q"]), off],
                           dict(rows=rows, rank=m.kv_rank, rank_ld=m.rank_ld, ldkv=L, ldc=m.ldc, ring=ring, heads=m.heads, hs=m.hs,
                                dim_ld=m.dim_ld, rot=m.rot_dim, rot_dims=m.rot_dims, ldq=Q, eps=c.eps, act=act)))
+        if self._long_latent(m, rows):
+            ldk, ldv, seen = m.heads * m.dim_ld, self._ldv(m), m.window - 1 + rows
+            back = dict(ring=ring, row_back=m.window - 1)
+            self._dense(t, arg(cache), w.mats[p + "uk"], arg(b["kx"]), seen, m.ldc, ldk, base=[off], **back)
+            self._dense(t, arg(cache), w.mats[p + "uv"], arg(b["vx"]), seen, m.ldc, ldv, base=[off], transposed=1, **back)
+            t.append(Dispatch(self._name("latent_prefill"),
+                              [arg(b["q"]), arg(b["kx"]), arg(b["vx"]), arg(cache), arg(w.vecs[p + "sink"]), off, arg(b["att"])],
+                              dict(rows=rows, heads=m.heads, dim_ld=m.dim_ld, rot_ld=m.rot_ld, vdim_ld=m.vdim_ld, rank_ld=m.rank_ld, ldq=Q,
+                                   ldk=ldk, ldv=ldv, ldo=A, ldc=m.ldc, ring=ring, window=m.window, scale=m.scale)))
+            self._dense(t, arg(b["att"]), w.mats[p + "o"], arg(b["mix"]), rows, A, D, y32=True)
+            return
         lat = m.heads * m.rank_ld
         self._dense(t, arg(b["q"]), w.mats[p + "uk_t"], arg(b["qa"]), rows, Q, lat, n=m.kv_rank, batch=m.heads, xb=m.hs,
                     wb=m.kv_rank * w.mats[p + "uk_t"].k, yb=m.rank_ld)
@@ -569,9 +620,10 @@ class LayerRuntime:
         t.append(Dispatch(self._name("ssm_conv"),
                           [u, arg(w.vecs[p + "conv"]), arg(w.vecs[p + "conv.b"]), arg(st["hist"]), off, arg(b["xbc"])],
                           dict(rows=rows, channels=m.channels, taps=m.conv, ldu=U, ldy=X, ldh=H, act=act)))
-        t.append(Dispatch(self._name("ssm_scan"),
+        long = self._long_ssm(m, rows)
+        t.append(Dispatch(self._name("ssm_chunk" if long else "ssm_scan"),
                           [arg(b["xbc"]), arg(b["dt"]), arg(w.vecs[p + "dt_bias"]), arg(w.vecs[p + "A_log"]), arg(w.vecs[p + "D"]), u, off,
-                           arg(st["state"]), arg(st["hist"]), arg(b["y"])],
+                           arg(st["state"]), arg(st["hist"]), arg(b["y"])] + ([arg(b["chunks"]), arg(b["decay"])] if long else []),
                           dict(rows=rows, heads=m.heads, groups=m.groups, n=m.state, p=m.vdim, state_ld=m.state_ld, ldx=X, lddt=T, ldy=Y,
                                ldu=U, ldh=H, channels=m.channels, taps=m.conv, act=act)))
         t.append(Dispatch(self._name("group_norm"), [arg(b["y"]), arg(b["u"]), arg(w.vecs[p + "norm"]), arg(b["g"])],
@@ -587,10 +639,15 @@ class LayerRuntime:
         t.append(Dispatch(self._name("route_rows"), [arg(b["rl"]), arg(w.vecs[p + "correction"]), arg(b["ridx"]), arg(b["rwt"])],
                           dict(rows=rows, outputs=f.outputs, top=f.top, ld=O)))
         q = dict(routes=rows * f.top, experts=f.experts, act=act)
+        tile, groups = self._grouped(f, rows), []
+        if tile:
+            groups = [arg(b["perm"]), arg(b["tiles"]), arg(b["tile_count"])]
+            t.append(Dispatch(self._name("route_group"), [arg(b["ridx"])] + groups, dict(routes=rows * f.top, experts=f.experts, tile_rows=tile)))
+            q.update(grouped=1, tile_rows=tile)
         t.append(Dispatch(self._name("experts"),
-                          [arg(b["h2"]), arg(w.mats[p + "gate"].w), arg(w.mats[p + "up"].w), arg(b["ridx"]), arg(b["eh"])],
+                          [arg(b["h2"]), arg(w.mats[p + "gate"].w), arg(w.mats[p + "up"].w), arg(b["ridx"])] + groups + [arg(b["eh"])],
                           dict(q, n=f.ff, k=D, ldx=D, ldw=D, ldy=F, x_div=f.top, pair=1)))
-        t.append(Dispatch(self._name("experts"), [arg(b["eh"]), arg(w.mats[p + "down"].w), arg(b["ridx"]), arg(b["eo"])],
+        t.append(Dispatch(self._name("experts"), [arg(b["eh"]), arg(w.mats[p + "down"].w), arg(b["ridx"])] + groups + [arg(b["eo"])],
                           dict(q, n=c.width, k=F, ldx=F, ldw=F, ldy=D, x_div=1)))
 
     def _body_tasks(self, t, tokens, off, rows: int) -> None:

@@ -640,6 +640,16 @@ def read_reduce(src, nbytes, out, stream=None):
     check(lib.fk_read_reduce(_ptr(src), C.c_size_t(nbytes), _ptr(out), C.c_size_t(out.nbytes), _ptr(stream)))
 
 
+def latent_prefill_supported(dim_ld: int, rot_ld: int, vdim_ld: int) -> bool:
+    """Whether padded head widths have the matrix-core form of windowed latent attention."""
+    return bool(lib.fk_latent_prefill_supported(C.c_uint32(dim_ld), C.c_uint32(rot_ld), C.c_uint32(vdim_ld)))
+
+
+def ssm_chunk_supported(heads: int, vdim: int, state: int) -> bool:
+    """Whether a state-space mixer's widths have the chunked matrix-core form."""
+    return bool(lib.fk_ssm_chunk_supported(C.c_uint32(heads), C.c_uint32(vdim), C.c_uint32(state)))
+
+
 def fill_u32(buf, value, count, stream=None):
     check(lib.fk_fill_u32(_ptr(buf), C.c_uint32(value), C.c_size_t(count), _ptr(stream)))
 

@@ -648,6 +648,18 @@ fk_status fk_xcd_kslice_meta(const uint16_t *src, uint32_t n, uint32_t groups, u
  * graph's sum rows when it fails. */
 fk_status fk_xcd_check(void *workspace, fk_stream s);
 
+/* ---- layer-list decoder (dispatch families only; slots and parameters at the planners,
+ *      fusekit_amd/csrc/families_layered.hpp) ----------------------------------------------
+ * A decoder described layer by layer: latent attention over a sliding window with a sink, a Mamba-2 state-space mixer,
+ * experts chosen by a corrected softmax (some of them identities), a 32-bit residual stream.  Families
+ * fusekit_residual_norm, _group_norm, _dense, _route_rows, _route_group, _experts, _latent_store, _latent_attn,
+ * _ssm_conv, _ssm_scan take bf16 or fp32 activations (parameter act = 16 / 32) and any widths;
+ * fusekit_latent_prefill and fusekit_ssm_chunk are the matrix-core forms of attention and recurrence for portions of
+ * many rows (bf16).  These two answer whether a shape has such a form (padded head widths; heads, head width, state
+ * width). */
+int fk_latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld);
+int fk_ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n);
+
 /* ---- dispatcher: replaces `_fusekit_runtime_native` ------------------------
  *
  * A dispatch names a kernel family by prefix ("fusekit_rmsnorm_qkv_f12" ->
