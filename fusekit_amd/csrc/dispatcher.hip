@@ -26,6 +26,7 @@
 #include "decode_token.hpp"
 #include "fk_host.hpp"
 #include "fk_json.hpp"
+#include "layer_decode.hpp"
 #include "layered.hpp"
 #include "xcd_layer.hpp"
 
@@ -1562,6 +1563,9 @@ const Family kFamilies[] = {
     {"fusekit_ssm_scan", plan_ssm_scan_d},
     {"fusekit_latent_prefill", plan_latent_prefill_d},
     {"fusekit_ssm_chunk", plan_ssm_chunk_d},
+    {"fusekit_latent_split", plan_latent_split_d},
+    {"fusekit_layer_jobs", plan_layer_jobs_d},
+    {"fusekit_layer_out", plan_layer_out_d},
 };
 
 const Family* find_family(const std::string& kernel) {

@@ -299,3 +299,151 @@ fk_status plan_ssm_chunk_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     FK_TRY(s.end());
     return plan_ssm_chunk(a, l);
 }
+
+// qa, q, cache, offset, [freq: rotate], part, [sink, out: combine]
+//   {rows, heads, hs, dim_ld, rot, rot_dims, rank_ld, ldc, ldq, ring, window, splits, span, scale}
+fk_status plan_latent_split_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    LatentSplitArgs a;
+    memset(&a, 0, sizeof(a));
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.hs = d.u("hs"); a.dim_ld = d.u("dim_ld"); a.rot = d.u("rot"); a.rot_dims = d.u("rot_dims", a.rot);
+    a.rank_ld = d.u("rank_ld"); a.ldc = d.u("ldc"); a.ldq = d.u("ldq"); a.ring = d.u("ring"); a.window = d.u("window");
+    a.splits = d.u("splits"); a.span = d.u("span"); a.scale = (float)d.param("scale", 1.0);
+    if (!a.rows || !a.heads || !a.rank_ld || a.hs < a.dim_ld + a.rot || a.ldq < a.heads * a.hs) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.qa = s.in<uint16_t>((uint64_t)a.rows * a.heads * a.rank_ld * 2);
+    a.q = s.in<uint16_t>(rows_bytes(a.rows, a.ldq, a.heads * a.hs, 2));
+    a.cache = s.in<uint16_t>((uint64_t)a.ring * a.ldc * 2);
+    a.offset = s.in<uint32_t>(4);
+    if (d.u("rotate")) a.freq = s.in<double>(a.rot_dims >= 2 ? (uint64_t)(a.rot_dims / 2) * 8 : 1);
+    a.part = s.inout<float>((uint64_t)a.rows * a.splits * a.heads * (a.rank_ld + 2) * 4);
+    const bool combine = d.u("combine") != 0;
+    if (combine) {
+        a.sink = s.in<uint16_t>((uint64_t)a.heads * 2);
+        a.out = s.out<uint16_t>((uint64_t)a.rows * a.heads * a.rank_ld * 2);
+    }
+    FK_TRY(s.end());
+    return plan_latent_split(a, combine, l);
+}
+
+// Jobs side by side; every part is announced by a parameter, slots in this order:
+//   products i = 0, 1 (g<i>): g<i>_mode 0: x | 1: x, [step: g<i>_step], norm weights, [kept row: g<i>_keep] | 2: x, z, norm
+//     weights | 3: partial rows, sinks; then w, [y: n_act > 0], [y32: n_act < n]
+//     {g<i>_n, _k, _ldw, _width, _n_act, _rows_per_head, _x_head, _y_head, _groups, _splits, _heads, _eps}
+//   pair: x, gate, up, index, y                     {pair_n, _k, _ldw, _ldy, _top, _experts}
+//   route: logits, correction, index, weight        {route_outputs, _top}
+//   store: kv, norm, freq, offset, cache            {store_rank, _rank_ld, _ldc, _ring, _rot, _rot_dims, _eps}
+//   scan: u, dt, conv, conv bias, dt_bias, a_log, d, offset, state, hist, y
+//                                                   {scan_heads, _groups, _n, _p, _state_ld, _ldh, _taps}
+fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    LayerJobsArgs a;
+    memset(&a, 0, sizeof(a));
+    SlotCursor s{d, rw};
+    for (uint32_t i = 0; i < kMaxGemvJobs; ++i) {
+        const std::string g = "g" + std::to_string(i) + "_";
+        auto u = [&](const char* k, uint32_t dflt = 0) { return d.u((g + k).c_str(), dflt); };
+        if (!d.has((g + "n").c_str())) continue;
+        GemvJob& j = a.gemv[i];
+        j.mode = u("mode"); j.n = u("n"); j.k = u("k"); j.ldw = u("ldw", j.k); j.width = u("width", j.k); j.n_act = u("n_act");
+        j.rows_per_head = u("rows_per_head"); j.x_head = u("x_head"); j.y_head = u("y_head", j.rows_per_head);
+        j.groups = u("groups", 1); j.splits = u("splits"); j.heads = u("heads"); j.eps = (float)d.param((g + "eps").c_str(), 1e-6);
+        if (!j.n || !j.k || !j.width || j.mode > kRowCombine) return set_error(FK_ERR_INVALID, d.kernel + ": product parameters missing");
+        const uint64_t nh = j.rows_per_head ? j.n / j.rows_per_head : 1;
+        if (nh == 0) return set_error(FK_ERR_INVALID, d.kernel + ": rows per head");
+        if (j.mode == kRowPlain) j.x = s.in(((nh - 1) * j.x_head + j.k) * 2);
+        else if (j.mode == kRowNorm) {
+            j.x = s.in((uint64_t)j.width * 4);
+            j.vec = ((uintptr_t)j.x & 15u) == 0;
+            if (u("step")) j.x2 = s.in((uint64_t)j.k * 2);
+            j.nw = s.in<uint16_t>((uint64_t)j.k * 2);
+            if (u("keep")) j.keep = s.out<uint16_t>((uint64_t)j.k * 2);
+        } else if (j.mode == kRowGated) {
+            j.x = s.in((uint64_t)j.width * 2);
+            j.x2 = s.in((uint64_t)j.width * 2);
+            j.nw = s.in<uint16_t>((uint64_t)j.width * 2);
+        } else {
+            j.pl = j.k + 2;
+            if (j.heads != nh) return set_error(FK_ERR_INVALID, d.kernel + ": heads of the partial rows");
+            j.x = s.in((uint64_t)j.splits * j.heads * j.pl * 4);
+            j.nw = s.in<uint16_t>((uint64_t)j.heads * 2);
+        }
+        j.w = s.in<uint16_t>(((uint64_t)(j.n - 1) * j.ldw + j.k) * 2);
+        const uint64_t outs = (nh - 1) * j.y_head + (j.rows_per_head ? j.rows_per_head : j.n);
+        if (j.n_act && j.n_act < j.n && j.rows_per_head) return set_error(FK_ERR_UNSUPPORTED, d.kernel + ": per-head products have one kind of output");
+        if (j.n_act) j.y = s.out((j.n_act < j.n ? j.n_act : outs) * 2);
+        if (j.n_act < j.n) j.y32 = s.out<float>((j.n_act ? (uint64_t)(j.n - j.n_act) : outs) * 4);
+    }
+    if (d.u("pair_n")) {
+        PairJob& j = a.pair;
+        j.n = d.u("pair_n"); j.k = d.u("pair_k"); j.ldw = d.u("pair_ldw", j.k); j.ldy = d.u("pair_ldy", j.n); j.top = d.u("pair_top"); j.experts = d.u("pair_experts");
+        if (!j.k || !j.top || !j.experts || j.ldy < j.n) return set_error(FK_ERR_INVALID, d.kernel + ": expert parameters missing");
+        j.x = s.in<uint16_t>((uint64_t)j.k * 2);
+        j.wa = s.in<uint16_t>((uint64_t)j.experts * j.n * j.ldw * 2);
+        j.wb = s.in<uint16_t>((uint64_t)j.experts * j.n * j.ldw * 2);
+        j.index = s.in<uint32_t>((uint64_t)j.top * 4);
+        j.y = s.out<uint16_t>(rows_bytes(j.top, j.ldy, j.n, 2));
+    }
+    if (d.u("route_outputs")) {
+        RouteJob& j = a.route;
+        j.outputs = d.u("route_outputs"); j.top = d.u("route_top");
+        j.logits = s.in<float>((uint64_t)j.outputs * 4);
+        j.correction = s.in<uint16_t>((uint64_t)j.outputs * 2);
+        j.index = s.out<uint32_t>((uint64_t)j.top * 4);
+        j.weight = s.out<float>((uint64_t)j.top * 4);
+    }
+    if (d.u("store_rank")) {
+        StoreJob& j = a.store;
+        j.rank = d.u("store_rank"); j.rank_ld = d.u("store_rank_ld"); j.ldc = d.u("store_ldc"); j.ring = d.u("store_ring"); j.rot = d.u("store_rot");
+        j.rot_dims = d.u("store_rot_dims", j.rot); j.eps = (float)d.param("store_eps", 1e-6);
+        j.kv = s.in<float>((uint64_t)(j.rank + j.rot) * 4);
+        j.norm = s.in<uint16_t>((uint64_t)j.rank * 2);
+        j.freq = s.in<double>(j.rot_dims >= 2 ? (uint64_t)(j.rot_dims / 2) * 8 : 1);
+        j.offset = s.in<uint32_t>(4);
+        j.cache = s.inout<uint16_t>((uint64_t)j.ring * j.ldc * 2);
+    }
+    if (d.u("scan_heads")) {
+        ScanJob& j = a.scan;
+        j.heads = d.u("scan_heads"); j.groups = d.u("scan_groups"); j.n = d.u("scan_n"); j.p = d.u("scan_p"); j.state_ld = d.u("scan_state_ld");
+        j.ldh = d.u("scan_ldh"); j.taps = d.u("scan_taps");
+        const uint64_t ch = (uint64_t)j.heads * j.p + 2ull * j.groups * j.n;
+        if (!j.p || !j.n || !j.taps || j.ldh < ch) return set_error(FK_ERR_INVALID, d.kernel + ": state-space parameters missing");
+        j.u = s.in<uint16_t>(ch * 2);
+        j.dt = s.in<float>((uint64_t)j.heads * 4);
+        j.w = s.in<uint16_t>(ch * j.taps * 2);
+        j.b = s.in<uint16_t>(ch * 2);
+        j.dt_bias = s.in<uint16_t>((uint64_t)j.heads * 2);
+        j.a_log = s.in<uint16_t>((uint64_t)j.heads * 2);
+        j.d = s.in<uint16_t>((uint64_t)j.heads * 2);
+        j.offset = s.in<uint32_t>(4);
+        j.state = s.inout<float>((uint64_t)j.heads * j.p * j.state_ld * 4);
+        j.hist = s.inout<uint16_t>((uint64_t)j.taps * j.ldh * 2);
+        j.y = s.out<uint16_t>((uint64_t)j.heads * j.p * 2);
+    }
+    FK_TRY(s.end());
+    return plan_layer_jobs(a, l);
+}
+
+// x, [mix: has_mix], [att, w: ko > 0], [expert rows, down, index, weight, h2: top > 0], [step: has_step]
+//   {n, ko, ldo, kf, top, experts}
+fk_status plan_layer_out_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    LayerOutArgs a;
+    memset(&a, 0, sizeof(a));
+    a.n = d.u("n"); a.ko = d.u("ko"); a.ldo = d.u("ldo", a.ko); a.kf = d.u("kf"); a.top = d.u("top"); a.experts = d.u("experts");
+    if (!a.n || a.top > kMaxRouterTop) return set_error(FK_ERR_INVALID, d.kernel + ": n / top parameters");
+    SlotCursor s{d, rw};
+    a.x = s.inout<float>((uint64_t)a.n * 4);
+    if (d.u("has_mix")) a.mix = s.in<float>((uint64_t)a.n * 4);
+    if (a.ko) {
+        a.att = s.in<uint16_t>((uint64_t)a.ko * 2);
+        a.wo = s.in<uint16_t>(((uint64_t)(a.n - 1) * a.ldo + a.ko) * 2);
+    }
+    if (a.top) {
+        a.eh = s.in<uint16_t>((uint64_t)a.top * a.kf * 2);
+        a.wd = s.in<uint16_t>((uint64_t)a.experts * a.n * a.kf * 2);
+        a.index = s.in<uint32_t>((uint64_t)a.top * 4);
+        a.weight = s.in<float>((uint64_t)a.top * 4);
+        a.h2 = s.in<uint16_t>((uint64_t)a.n * 2);
+    }
+    if (d.u("has_step")) a.step = s.in<uint16_t>((uint64_t)a.n * 2);
+    FK_TRY(s.end());
+    return plan_layer_out(a, l);
+}

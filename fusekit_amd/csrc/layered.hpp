@@ -124,6 +124,24 @@ struct LatentAttnArgs {
 };
 fk_status plan_latent_attn(const LatentAttnArgs& a, uint32_t act, Launch* out);
 
+// The same for a few rows on the matrix cores (bf16): the window in `splits` spans of whole 64-position tiles, partial
+// rows [rows, splits, heads, rank_ld + 2] = latent sums | maximum | sum of weights.
+struct LatentSplitArgs {
+    const uint16_t* qa;
+    const uint16_t* q;
+    const uint16_t* cache;
+    const uint16_t* sink;
+    uint16_t* out;          // [rows, heads, rank_ld] when combined here
+    float* part;
+    const double* freq;     // rotates q while it is read; null: q is rotated already
+    const uint32_t* offset;
+    uint32_t rows, heads, hs, dim_ld, rot, rot_dims, rank_ld, ldc, ldq, ring, window, splits, span;
+    float scale;
+};
+constexpr uint32_t kMaxSplitRot = 64;   // rotated pairs
+bool latent_split_supported(uint32_t rank_ld, uint32_t ldc, uint32_t rot_dims);
+fk_status plan_latent_split(LatentSplitArgs& a, bool combine, Launch* out);
+
 // Attention of a pass with keys and values formed from the latents (bf16): row 0 of k / column 0 of vt is position
 // *offset - (window - 1).
 struct LatentPrefillArgs {

@@ -487,6 +487,9 @@ class LayerRuntime:
                 want("qa", R * m.heads * m.rank_ld * e)
                 want("ol", R * m.heads * m.rank_ld * e)
                 want("att", R * pad(m.heads * m.vdim_ld) * e)
+                if self._split_latent(m):
+                    most = max(rows * self._splits(m, rows)[0] for rows in range(1, R + 1) if not self._long_latent(m, rows))
+                    want("part", most * m.heads * (m.rank_ld + 2) * 4)
                 if self._long_latent(m, R):
                     want("kx", (m.window - 1 + R) * m.heads * m.dim_ld * e)
                     want("vx", m.heads * m.vdim_ld * self._ldv(m) * e)
@@ -515,6 +518,17 @@ class LayerRuntime:
     def _long_latent(self, m: LatentAttention, rows: int) -> bool:
         """Keys and values formed once for the pass (instead of queries carried into the latent space)."""
         return self.cfg.act == 16 and self.cfg.tiled and rows >= 64 and native.latent_prefill_supported(m.dim_ld, m.rot_ld, m.vdim_ld)
+
+    def _split_latent(self, m: LatentAttention) -> bool:
+        """The window of a few query rows split over workgroups on the matrix cores (instead of a workgroup per head)."""
+        return self.cfg.act == 16 and self.cfg.tiled and native.latent_split_supported(m.rank_ld, m.ldc, m.rot_dims)
+
+    def _splits(self, m: LatentAttention, rows: int) -> Tuple[int, int]:
+        """(splits, positions per split): whole 64-position tiles, fewer and longer splits as rows fill the device."""
+        tiles = -(-m.window // 64)
+        groups = rows * -(-m.heads // 16)
+        span = 64 * max(1, -(-tiles // 32), min(tiles, tiles * groups // 1024))
+        return -(-m.window // span), span
 
     def _ldv(self, m: LatentAttention) -> int:
         return pad(m.window - 1 + self.R + 64)
@@ -599,13 +613,131 @@ class LayerRuntime:
         lat = m.heads * m.rank_ld
         self._dense(t, arg(b["q"]), w.mats[p + "uk_t"], arg(b["qa"]), rows, Q, lat, n=m.kv_rank, batch=m.heads, xb=m.hs,
                     wb=m.kv_rank * w.mats[p + "uk_t"].k, yb=m.rank_ld)
-        t.append(Dispatch(self._name("latent_attn"),
-                          [arg(b["qa"]), arg(b["q"]), arg(cache), arg(w.vecs[p + "sink"]), off, arg(b["ol"])],
-                          dict(rows=rows, heads=m.heads, hs=m.hs, dim_ld=m.dim_ld, rot=m.rot_dim, rank=m.kv_rank, rank_ld=m.rank_ld,
-                               ldc=m.ldc, ldq=Q, ring=ring, window=m.window, scale=m.scale, act=act)))
+        if self._split_latent(m):
+            t.append(self._split_task(m, p, run, rows, off, rotate=False))
+        else:
+            t.append(Dispatch(self._name("latent_attn"),
+                              [arg(b["qa"]), arg(b["q"]), arg(cache), arg(w.vecs[p + "sink"]), off, arg(b["ol"])],
+                              dict(rows=rows, heads=m.heads, hs=m.hs, dim_ld=m.dim_ld, rot=m.rot_dim, rank=m.kv_rank, rank_ld=m.rank_ld,
+                                   ldc=m.ldc, ldq=Q, ring=ring, window=m.window, scale=m.scale, act=act)))
         self._dense(t, arg(b["ol"]), w.mats[p + "uv"], arg(b["att"]), rows, lat, A, n=m.vdim_ld, batch=m.heads, xb=m.rank_ld,
                     wb=m.vdim_ld * w.mats[p + "uv"].k, yb=m.vdim_ld)
         self._dense(t, arg(b["att"]), w.mats[p + "o"], arg(b["mix"]), rows, A, D, y32=True)
+
+    def _split_task(self, m: LatentAttention, p: str, run: int, rows: int, off, rotate: bool) -> Dispatch:
+        """Split attention; `rotate`: q is not rotated yet and the partial rows are left to the product with W_uv."""
+        w, b = self.w, self.buf
+        splits, span = self._splits(m, rows)
+        cache = self.state.entries[run]["cache"]
+        a = [arg(b["qa"]), arg(b["q"]), arg(cache), off] + ([arg(w.vecs[p + "rot_freq"])] if rotate else []) + [arg(b["part"])]
+        a += [] if rotate else [arg(w.vecs[p + "sink"]), arg(b["ol"])]
+        return Dispatch(self._name("latent_split"), a,
+                        dict(rows=rows, heads=m.heads, hs=m.hs, dim_ld=m.dim_ld, rot=m.rot_dim, rot_dims=m.rot_dims, rank_ld=m.rank_ld,
+                             ldc=m.ldc, ldq=pad(m.heads * m.hs), ring=self.state.rings[run], window=m.window, splits=splits, span=span,
+                             scale=m.scale, rotate=int(rotate), combine=int(not rotate)))
+
+    # -- one decoded token in fused launches
+    def _fused(self) -> bool:
+        """Whether every layer has the fused decode launches."""
+        c = self.cfg
+        if c.act != 16 or not c.fuse or not c.tiled or pad(c.width) > 30720:
+            return False
+        for l in c.layers:
+            m, f = l.mixer, l.mlp
+            ko = 0
+            if m.kind == "latent_attention":
+                ko = pad(m.heads * m.vdim_ld)
+                if not self._split_latent(m) or max(pad(m.q_rank), m.rank_ld) > 30720:
+                    return False
+            elif m.norm_groups > 64 or pad(m.inner) > 30720 or m.state > 256:
+                return False
+            kf = f.top * pad(f.ff) if f else 0
+            items = -(-ko // 512) + (f.top * -(-pad(f.ff) // 512) if f else 0) + 2
+            if (ko + kf) * 2 + items * 24 + 16 > 60 * 1024:
+                return False
+        return True
+
+    def _jobs(self, t: List[Dispatch], args: list, **params) -> None:
+        t.append(Dispatch(self._name("layer_jobs"), args, params))
+
+    def _product(self, i: int, W: DeviceWeight, n_act: int, **more) -> Dict[str, float]:
+        return {f"g{i}_{k}": v for k, v in dict(more, n=W.n, k=W.k, ldw=W.k, n_act=n_act).items()}
+
+    def _fused_tasks(self, t: List[Dispatch]) -> None:
+        c, w, b = self.cfg, self.w, self.buf
+        off, D = arg(self.offset), pad(c.width)
+        t.append(Dispatch(self._name("embed_lookup_decode"), [arg(self.token), arg(w.mats["embed"].w), arg(b["x"])],
+                          dict(bits=16, hidden=c.width, vocab=c.vocab, output_scale=c.embed_scale, out_bits=32, x_row_stride=D)))
+        for run, (i, first) in enumerate(self.runs):
+            m, f, p = c.layers[i].mixer, c.layers[i].mlp, f"l{i}."
+            q = p + "mix."
+            st = self.state.entries[run]
+            step = [] if first is None else [arg(w.vecs["loop.step"], D * 2, first * D * 2)]
+            norm = dict(mode=1, width=c.width, eps=c.eps, step=len(step))
+            latent = m.kind == "latent_attention"
+            # 1: norms; the mixer's joint down / input projection and the router
+            Win = w.mats[q + ("down" if latent else "in")]
+            n_act = 0 if latent else m.inner + m.channels
+            a = [arg(b["x"])] + step + [arg(w.vecs[p + "norm1"]), arg(Win.w)]
+            a += [arg(b["low"])] if latent else [arg(b["u"]), arg(b["dt"])]
+            prm = self._product(0, Win, n_act, **norm)
+            if f:
+                Wr = w.mats[p + "mlp.router"]
+                a += [arg(b["x"])] + step + [arg(w.vecs[p + "norm2"]), arg(b["h2"]), arg(Wr.w), arg(b["rl"])]
+                prm.update(self._product(1, Wr, 0, keep=1, **norm))
+            self._jobs(t, a, **prm)
+            route = [arg(b["rl"]), arg(w.vecs[p + "mlp.correction"]), arg(b["ridx"]), arg(b["rwt"])] if f else []
+            prm_route = dict(route_outputs=f.outputs, route_top=f.top) if f else {}
+            pair, prm_pair = [], {}
+            if f:
+                F = pad(f.ff)
+                pair = [arg(b["h2"]), arg(w.mats[p + "mlp.gate"].w), arg(w.mats[p + "mlp.up"].w), arg(b["ridx"]), arg(b["eh"])]
+                prm_pair = dict(pair_n=f.ff, pair_k=D, pair_ldw=D, pair_ldy=F, pair_top=f.top, pair_experts=f.experts)
+            if latent:
+                # 2: queries, the cache row, the choice of experts
+                Wq, Wk, Wv = w.mats[q + "uq"], w.mats[q + "uk_t"], w.mats[q + "uv"]
+                a = [arg(b["low"]), arg(w.vecs[q + "dq.norm"]), arg(Wq.w), arg(b["q"])] + route
+                a += [arg(b["low"], None, m.q_rank * 4), arg(w.vecs[q + "dkv.norm"]), arg(w.vecs[q + "rot_freq"]), off, arg(st["cache"])]
+                self._jobs(t, a, **self._product(0, Wq, Wq.n, mode=1, width=m.q_rank, eps=c.eps), **prm_route, store_rank=m.kv_rank,
+                           store_rank_ld=m.rank_ld, store_ldc=m.ldc, store_ring=self.state.rings[run], store_rot=m.rot_dim,
+                           store_rot_dims=m.rot_dims, store_eps=c.eps)
+                # 3: queries into the latent space, gate / up
+                self._jobs(t, [arg(b["q"]), arg(Wk.w), arg(b["qa"])] + pair,
+                           **self._product(0, Wk, Wk.n, mode=0, rows_per_head=m.kv_rank, x_head=m.hs, y_head=m.rank_ld), **prm_pair)
+                # 4, 5: attention over the window, its combination and W_uv
+                t.append(self._split_task(m, q, run, 1, off, rotate=True))
+                self._jobs(t, [arg(b["part"]), arg(w.vecs[q + "sink"]), arg(Wv.w), arg(b["att"])],
+                           **self._product(0, Wv, Wv.n, mode=3, rows_per_head=m.vdim_ld, y_head=m.vdim_ld, heads=m.heads,
+                                           splits=self._splits(m, 1)[0]))
+            else:
+                # 2: convolution and state, the choice of experts
+                a = route + [arg(b["u"], None, m.inner * 2), arg(b["dt"]), arg(w.vecs[q + "conv"]), arg(w.vecs[q + "conv.b"]), arg(w.vecs[q + "dt_bias"]),
+                             arg(w.vecs[q + "A_log"]), arg(w.vecs[q + "D"]), off, arg(st["state"]), arg(st["hist"]), arg(b["y"])]
+                self._jobs(t, a, **prm_route, scan_heads=m.heads, scan_groups=m.groups, scan_n=m.state, scan_p=m.vdim, scan_state_ld=m.state_ld,
+                           scan_ldh=pad(m.channels), scan_taps=m.conv)
+                # 3: gated norm and output projection, gate / up
+                Wo = w.mats[q + "o"]
+                self._jobs(t, [arg(b["y"]), arg(b["u"]), arg(w.vecs[q + "norm"]), arg(Wo.w), arg(b["mix"])] + pair,
+                           **self._product(0, Wo, 0, mode=2, width=m.inner, groups=m.norm_groups, eps=c.eps), **prm_pair)
+            # last: everything into the residual row
+            a, prm = [arg(b["x"])], dict(n=c.width)
+            if latent:
+                A = pad(m.heads * m.vdim_ld)
+                a += [arg(b["att"]), arg(w.mats[q + "o"].w)]
+                prm.update(ko=A, ldo=A)
+            else:
+                a.append(arg(b["mix"]))
+                prm["has_mix"] = 1
+            if f:
+                a += [arg(b["eh"]), arg(w.mats[p + "mlp.down"].w), arg(b["ridx"]), arg(b["rwt"]), arg(b["h2"])]
+                prm.update(kf=pad(f.ff), top=f.top, experts=f.experts)
+            if step:
+                a += step
+                prm["has_step"] = 1
+            t.append(Dispatch(self._name("layer_out"), a, prm))
+        head = w.mats["head"]
+        self._jobs(t, [arg(b["x"]), arg(w.vecs["final.norm"]), arg(head.w), arg(self.logits)],
+                   **self._product(0, head, 0, mode=1, width=c.width, eps=c.eps))
 
     def _ssm_tasks(self, t, run: int, rows: int, off) -> None:
         c, w, b = self.cfg, self.w, self.buf
@@ -675,8 +807,12 @@ class LayerRuntime:
         self._fid = 0
         c = self.cfg
         t = [Dispatch("fusekit_step_init", [arg(self.step_counter), arg(self.offset), arg(self.kv_len)])]
-        self._body_tasks(t, arg(self.token), arg(self.offset), 1)
-        self._dense(t, arg(self.buf["h1"]), self.w.mats["head"], arg(self.logits), 1, pad(c.width), pad(c.vocab), y32=True)
+        self.fused = self._fused()
+        if self.fused:
+            self._fused_tasks(t)
+        else:
+            self._body_tasks(t, arg(self.token), arg(self.offset), 1)
+            self._dense(t, arg(self.buf["h1"]), self.w.mats["head"], arg(self.logits), 1, pad(c.width), pad(c.vocab), y32=True)
         t.append(self._argmax_task())
         return t
 
