@@ -888,7 +888,7 @@ fk_status fk_xcd_check(void* workspace, fk_stream s) {
 }
 
 int fk_latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld) { return latent_prefill_supported(dim_ld, rot_ld, vdim_ld) ? 1 : 0; }
-int fk_latent_split_supported(uint32_t rank_ld, uint32_t ldc, uint32_t rot_dims) { return latent_split_supported(rank_ld, ldc, rot_dims) ? 1 : 0; }
+int fk_latent_split_supported(uint32_t rank_ld, uint32_t ldc) { return latent_split_supported(rank_ld, ldc) ? 1 : 0; }
 int fk_ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n) { return ssm_chunk_supported(heads, p, n) ? 1 : 0; }
 
 }  // extern "C"

@@ -114,27 +114,30 @@ __global__ __launch_bounds__(kTileThreads) void dense_tile_kernel(const TileArgs
         pb[0][i] = wa + (size_t)r * a.ldw + sp * 8u;
         if (NB == 2) pb[NB - 1][i] = wb + (size_t)r * a.ldw + sp * 8u;
     }
-    dm_u32x4_t ra[LA], rb[NB][LB];
-    auto fetch = [&](uint32_t k0) __attribute__((always_inline)) {
+    struct Staged {
+        dm_u32x4_t a[LA], b[NB][LB];
+    };
+    Staged r0;
+    auto fetch = [&](Staged& r, uint32_t k0) __attribute__((always_inline)) {
 #pragma unroll
-        for (int i = 0; i < LA; ++i) ra[i] = *reinterpret_cast<const dm_u32x4_t*>(pa[i] + k0);
+        for (int i = 0; i < LA; ++i) r.a[i] = *reinterpret_cast<const dm_u32x4_t*>(pa[i] + k0);
 #pragma unroll
         for (int b = 0; b < NB; ++b)
 #pragma unroll
-            for (int i = 0; i < LB; ++i) rb[b][i] = *reinterpret_cast<const dm_u32x4_t*>(pb[b][i] + k0);
+            for (int i = 0; i < LB; ++i) r.b[b][i] = *reinterpret_cast<const dm_u32x4_t*>(pb[b][i] + k0);
     };
-    auto stage = [&](uint16_t* t) __attribute__((always_inline)) {
+    auto stage = [&](const Staged& q, uint16_t* t) __attribute__((always_inline)) {
 #pragma unroll
         for (int i = 0; i < LA; ++i) {
             const uint32_t r = sr + 32u * i;
-            *reinterpret_cast<dm_u32x4_t*>(t + r * kBK + ((sp ^ (r & 7u)) << 3)) = ra[i];
+            *reinterpret_cast<dm_u32x4_t*>(t + r * kBK + ((sp ^ (r & 7u)) << 3)) = q.a[i];
         }
 #pragma unroll
         for (int b = 0; b < NB; ++b)
 #pragma unroll
             for (int i = 0; i < LB; ++i) {
                 const uint32_t r = sr + 32u * i;
-                *reinterpret_cast<dm_u32x4_t*>(t + (BM + b * BN) * kBK + r * kBK + ((sp ^ (r & 7u)) << 3)) = rb[b][i];
+                *reinterpret_cast<dm_u32x4_t*>(t + (BM + b * BN) * kBK + r * kBK + ((sp ^ (r & 7u)) << 3)) = q.b[b][i];
             }
     };
 
@@ -147,12 +150,7 @@ __global__ __launch_bounds__(kTileThreads) void dense_tile_kernel(const TileArgs
             for (int j = 0; j < TN; ++j) acc[b][i][j] = dm_f32x4_t{0.f, 0.f, 0.f, 0.f};
 
     const uint32_t steps = a.k / kBK;
-    fetch(0);
-    stage(lds[0]);
-    __syncthreads();
-    for (uint32_t s = 0; s < steps; ++s) {
-        const uint16_t* t = lds[s & 1u];
-        if (s + 1u < steps) fetch((s + 1u) * kBK);
+    auto compute = [&](const uint16_t* t) __attribute__((always_inline)) {
 #pragma unroll
         for (uint32_t h = 0; h < 2; ++h) {
             dm_u32x4_t fa[TM], fb[NB][TN];
@@ -173,8 +171,36 @@ __global__ __launch_bounds__(kTileThreads) void dense_tile_kernel(const TileArgs
                                                     : __builtin_amdgcn_mfma_f32_16x16x32_bf16(vb, va, acc[b][i][j], 0, 0, 0);
                     }
         }
-        if (s + 1u < steps) stage(lds[(s + 1u) & 1u]);
+    };
+    fetch(r0, 0);
+    stage(r0, lds[0]);
+    if constexpr (BM + NB * BN <= 128) {
+        // small tiles: step s is multiplied from LDS buffer s % 2 while step s + 1 waits in registers and step s + 2 is
+        // on its way; past the end the last step is requested again
+        auto at = [&](uint32_t s) __attribute__((always_inline)) { return (s < steps ? s : steps - 1u) * kBK; };
+        Staged r1;
+        fetch(r1, at(1));
         __syncthreads();
+        for (uint32_t s = 0; s < steps; s += 2u) {
+            fetch(r0, at(s + 2u));
+            compute(lds[0]);
+            stage(r1, lds[1]);
+            __syncthreads();
+            if (s + 1u >= steps) break;
+            fetch(r1, at(s + 3u));
+            compute(lds[1]);
+            stage(r0, lds[0]);
+            __syncthreads();
+        }
+    } else {
+        // large tiles hold one step in registers: two would halve the waves per SIMD
+        __syncthreads();
+        for (uint32_t s = 0; s < steps; ++s) {
+            if (s + 1u < steps) fetch(r0, (s + 1u) * kBK);
+            compute(lds[s & 1u]);
+            if (s + 1u < steps) stage(r0, lds[(s + 1u) & 1u]);
+            __syncthreads();
+        }
     }
 
 #pragma unroll
@@ -333,7 +359,7 @@ fk_status plan_dense(const DenseArgs& a, uint32_t act, Launch* out) {
     const int o = a.transposed ? kOutT : (a.y32 ? kOut32 : kOutAct);
     auto blocks = [&](uint32_t bm, uint32_t bn) { return (uint64_t)((a.m + bm - 1) / bm) * ((a.n + bn - 1) / bn) * a.batch; };
     uint32_t bm, bn;
-    if (a.m <= 32) { bm = 32; bn = 64; out->func = tile_func<32, 64, 1, 4, 1, false>(o); }
+    if (a.m <= 32 || blocks(64, 64) < 128) { bm = 32; bn = 64; out->func = tile_func<32, 64, 1, 4, 1, false>(o); }
     else if (blocks(128, 128) >= 192) { bm = 128; bn = 128; out->func = tile_func<128, 128, 2, 2, 1, false>(o); }
     else { bm = 64; bn = 64; out->func = tile_func<64, 64, 2, 2, 1, false>(o); }
     t.tiles_m = (a.m + bm - 1) / bm;

@@ -300,7 +300,7 @@ fk_status plan_ssm_chunk_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     return plan_ssm_chunk(a, l);
 }
 
-// qa, q, cache, offset, [freq: rotate], part, [sink, out: combine]
+// qa, q, cache, offset, [tab: rotate], part, [sink, out: combine]
 //   {rows, heads, hs, dim_ld, rot, rot_dims, rank_ld, ldc, ldq, ring, window, splits, span, scale}
 fk_status plan_latent_split_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     LatentSplitArgs a;
@@ -314,7 +314,7 @@ fk_status plan_latent_split_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     a.q = s.in<uint16_t>(rows_bytes(a.rows, a.ldq, a.heads * a.hs, 2));
     a.cache = s.in<uint16_t>((uint64_t)a.ring * a.ldc * 2);
     a.offset = s.in<uint32_t>(4);
-    if (d.u("rotate")) a.freq = s.in<double>(a.rot_dims >= 2 ? (uint64_t)(a.rot_dims / 2) * 8 : 1);
+    if (d.u("rotate")) a.tab = s.in<float>((uint64_t)std::max(a.rot_dims, 1u) * 4);
     a.part = s.inout<float>((uint64_t)a.rows * a.splits * a.heads * (a.rank_ld + 2) * 4);
     const bool combine = d.u("combine") != 0;
     if (combine) {
@@ -331,7 +331,7 @@ fk_status plan_latent_split_d(const Dispatch& d, Launch* l, SlotRW* rw) {
 //     {g<i>_n, _k, _ldw, _width, _n_act, _rows_per_head, _x_head, _y_head, _groups, _splits, _heads, _eps}
 //   pair: x, gate, up, index, y                     {pair_n, _k, _ldw, _ldy, _top, _experts}
 //   route: logits, correction, index, weight        {route_outputs, _top}
-//   store: kv, norm, freq, offset, cache            {store_rank, _rank_ld, _ldc, _ring, _rot, _rot_dims, _eps}
+//   store: kv, norm, freq, offset, cache, tab            {store_rank, _rank_ld, _ldc, _ring, _rot, _rot_dims, _eps}
 //   scan: u, dt, conv, conv bias, dt_bias, a_log, d, offset, state, hist, y
 //                                                   {scan_heads, _groups, _n, _p, _state_ld, _ldh, _taps}
 fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
@@ -399,6 +399,7 @@ fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
         j.freq = s.in<double>(j.rot_dims >= 2 ? (uint64_t)(j.rot_dims / 2) * 8 : 1);
         j.offset = s.in<uint32_t>(4);
         j.cache = s.inout<uint16_t>((uint64_t)j.ring * j.ldc * 2);
+        j.tab = s.out<float>((uint64_t)std::max(j.rot_dims, 1u) * 4);
     }
     if (d.u("scan_heads")) {
         ScanJob& j = a.scan;

@@ -10,6 +10,7 @@
 // turn through the same LDS.  A lane owns one head in both products, so the running maximum and the rescale stay in it.
 #include "act_device.hpp"
 #include "layered.hpp"
+#include "split_device.hpp"
 
 namespace fk {
 
@@ -32,7 +33,7 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const LatentSplitArgs
     __shared__ __align__(16) uint16_t qs[16 * QS];
     __shared__ __align__(16) uint16_t ct[kLsHalf * kLsCs];
     __shared__ __align__(16) uint16_t ps[16 * kLsCs];
-    __shared__ float wmax[4][16], wsum[4][16], cs[2 * kMaxSplitRot];
+    __shared__ float wmax[4][16], wsum[4][16];
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, l16 = lane & 15u, kq = lane >> 4;
     const uint32_t split = blockIdx.x, h0 = blockIdx.y * 16u, r = blockIdx.z;
     const uint32_t pos = *a.offset + r, lo = pos + 1u > a.window ? pos + 1u - a.window : 0u;
@@ -40,13 +41,10 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const LatentSplitArgs
     const uint32_t pl = a.rank_ld + 2u;
     float* part = a.part + ((size_t)r * a.splits + split) * a.heads * pl;
     if (j0 > pos) {   // nothing of the window here
-        if (tid < 16u && h0 + tid < a.heads) {
-            part[(size_t)(h0 + tid) * pl + a.rank_ld] = -INFINITY;
-            part[(size_t)(h0 + tid) * pl + a.rank_ld + 1u] = 0.f;
-        }
+        const uint32_t hs = a.heads - h0 < 16u ? a.heads - h0 : 16u;
+        for (uint32_t i = tid; i < hs * pl; i += 256u) part[(size_t)h0 * pl + i] = i % pl == a.rank_ld ? -INFINITY : 0.f;
         return;
     }
-    const uint32_t half = a.rot_dims / 2u;
     auto load_k = [&](uint32_t j, ls_u32x4_t* k) __attribute__((always_inline)) {
         uint32_t p = j + wave * 16u + l16;
         p = p < j1 ? p : j1 - 1u;
@@ -56,35 +54,26 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const LatentSplitArgs
     };
     ls_u32x4_t k[S];
     load_k(j0, k);
-    if (a.freq) {
-        for (uint32_t i = tid; i < half; i += 256u) position_cos_sin(pos, a.freq[i], cs[2 * i], cs[2 * i + 1]);
-        __syncthreads();
-    }
     for (uint32_t i = tid; i < 16u * (S * 4u); i += 256u) {   // [carried query | rotated part | zeros], 16 bytes at a time
         const uint32_t h = i / (S * 4u), c = (i % (S * 4u)) * 8u;
         ls_u32x4_t v = {0u, 0u, 0u, 0u};
-        if (h0 + h < a.heads) {
-            if (c < a.rank_ld) v = *reinterpret_cast<const ls_u32x4_t*>(a.qa + ((size_t)r * a.heads + h0 + h) * a.rank_ld + c);
-            else if (c < a.ldc) {
-                const uint16_t* q = a.q + (size_t)r * a.ldq + (size_t)(h0 + h) * a.hs + a.dim_ld;
-                float e[8];
-#pragma unroll
-                for (uint32_t u = 0; u < 8; ++u) {
-                    const uint32_t d = c - a.rank_ld + u;
-                    float x = d < a.rot ? act_load(q + d) : 0.f;
-                    if (a.freq && d < a.rot_dims) {
-                        const uint32_t f = d < half ? d : d - half;
-                        const float o = act_load(q + (d < half ? d + half : d - half));
-                        x = d < half ? x * cs[2 * f] - o * cs[2 * f + 1] : x * cs[2 * f] + o * cs[2 * f + 1];
-                    }
-                    e[u] = x;
-                }
-                v = ls_u32x4_t{pack_bf16(e[0], e[1]), pack_bf16(e[2], e[3]), pack_bf16(e[4], e[5]), pack_bf16(e[6], e[7])};
-            }
-        }
+        if (h0 + h < a.heads && c < a.ldc)
+            v = c < a.rank_ld ? *reinterpret_cast<const ls_u32x4_t*>(a.qa + ((size_t)r * a.heads + h0 + h) * a.rank_ld + c)
+                              : *reinterpret_cast<const ls_u32x4_t*>(a.q + (size_t)r * a.ldq + (size_t)(h0 + h) * a.hs + a.dim_ld + c - a.rank_ld);
         *reinterpret_cast<ls_u32x4_t*>(qs + h * QS + c) = v;
     }
     __syncthreads();
+    if (a.tab) {   // the queries arrive unrotated
+        const uint32_t half = a.rot_dims / 2u;
+        for (uint32_t i = tid; i < 16u * half; i += 256u) {
+            const uint32_t h = i / half, d = i - h * half;
+            uint16_t* q = qs + h * QS + a.rank_ld + d;
+            const float u = act_load(q), v = act_load(q + half), cs = a.tab[2 * d], sn = a.tab[2 * d + 1];
+            act_store(q, u * cs - v * sn);
+            act_store(q + half, v * cs + u * sn);
+        }
+        __syncthreads();
+    }
 
     const float scale2 = a.scale * 1.4426950408889634f;
     float m_run = -INFINITY, l_run = 0.f;
@@ -115,7 +104,7 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const LatentSplitArgs
                 const ls_u32x4_t v = k[f * 8 + i < S ? f * 8 + i : 0];
                 ls_u32x4_t w;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) w[e] = (uint32_t)__shfl_xor((int)v[e], 1, kWave);
+                for (int e = 0; e < 4; ++e) w[e] = (uint32_t)__builtin_amdgcn_update_dpp(0, (int)v[e], 0xB1, 0xF, 0xF, true);   // lane ^ 1
                 const bool odd = l16 & 1u;
                 const uint32_t a0 = odd ? w[2] : v[0], a1 = odd ? w[3] : v[1], b0 = odd ? v[2] : w[0], b1 = odd ? v[3] : w[1];
                 uint16_t* q = ct + (i * 32u + kq * 8u + (odd ? 4u : 0u)) * kLsCs + wave * 16u + (l16 & ~1u);
@@ -192,25 +181,21 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const LatentSplitArgs
 
 // Partial rows -> the latent sum of one (head, row), with the sink in the denominator.
 __global__ __launch_bounds__(256) void latent_combine_kernel(const LatentSplitArgs a) {
+    __shared__ float w[kMaxSplits];
     const uint32_t h = blockIdx.x, r = blockIdx.y, pl = a.rank_ld + 2u;
     const float* p = a.part + ((size_t)r * a.splits * a.heads + h) * pl;
     const size_t ss = (size_t)a.heads * pl;
-    const float sink = bf16_bits_to_f32(a.sink[h]);
-    float top = sink;
-    for (uint32_t s = 0; s < a.splits; ++s) top = fmaxf(top, p[s * ss + a.rank_ld]);
-    float l = expf(sink - top);
-    for (uint32_t s = 0; s < a.splits; ++s) l += expf(p[s * ss + a.rank_ld] - top) * p[s * ss + a.rank_ld + 1u];
+    split_weights(p + a.rank_ld, ss, a.splits, bf16_bits_to_f32(a.sink[h]), w);
+    __syncthreads();
     for (uint32_t c = threadIdx.x * 2u; c < a.rank_ld; c += 512u) {
         float v0 = 0.f, v1 = 0.f;
+#pragma unroll 8
         for (uint32_t s = 0; s < a.splits; ++s) {
-            const float e = expf(p[s * ss + a.rank_ld] - top);
-            if (e != 0.f) {
-                const float2 q = *reinterpret_cast<const float2*>(p + s * ss + c);
-                v0 = fmaf(e, q.x, v0);
-                v1 = fmaf(e, q.y, v1);
-            }
+            const float2 q = *reinterpret_cast<const float2*>(p + s * ss + c);
+            v0 = fmaf(w[s], q.x, v0);
+            v1 = fmaf(w[s], q.y, v1);
         }
-        *reinterpret_cast<uint32_t*>(a.out + ((size_t)r * a.heads + h) * a.rank_ld + c) = pack_bf16(v0 / l, v1 / l);
+        *reinterpret_cast<uint32_t*>(a.out + ((size_t)r * a.heads + h) * a.rank_ld + c) = pack_bf16(v0, v1);
     }
 }
 
@@ -223,8 +208,8 @@ const LsForm kLsForms[] = {{4 * 32, 256, (const void*)&latent_split_kernel<4, 1>
 
 }  // namespace
 
-bool latent_split_supported(uint32_t rank_ld, uint32_t ldc, uint32_t rot_dims) {
-    if (rot_dims > 2 * kMaxSplitRot || rank_ld % 32 || ldc % 32) return false;
+bool latent_split_supported(uint32_t rank_ld, uint32_t ldc) {
+    if (rank_ld % 32 || ldc % 32) return false;
     for (const LsForm& f : kLsForms)
         if (ldc <= f.ldc && rank_ld <= f.rank) return true;
     return false;
@@ -236,8 +221,8 @@ fk_status plan_latent_split(LatentSplitArgs& a, bool combine, Launch* out) {
     if (!a.ring || (a.ring & (a.ring - 1)) || (uint64_t)a.window + a.rows - 1u > a.ring) return set_error(FK_ERR_INVALID, "latent split: ring too small");
     if (!a.splits || !a.span || a.span % kLsTile || (uint64_t)a.splits * a.span < a.window) return set_error(FK_ERR_INVALID, "latent split: the splits must cover the window in whole tiles");
     if (a.rot_dims % 2 || a.rot_dims > a.rot || a.rank_ld + a.rot > a.ldc) return set_error(FK_ERR_INVALID, "latent split: bad row layout");
-    if (!latent_split_supported(a.rank_ld, a.ldc, a.rot_dims)) return set_error(FK_ERR_UNSUPPORTED, "latent split: cache rows of at most 512 + 64 elements");
-    if (a.rows > 65535 || a.splits > 65535) return set_error(FK_ERR_UNSUPPORTED, "latent split: too many rows or splits");
+    if (!latent_split_supported(a.rank_ld, a.ldc)) return set_error(FK_ERR_UNSUPPORTED, "latent split: cache rows of at most 512 + 64 elements");
+    if (a.rows > 65535 || a.splits > kMaxSplits) return set_error(FK_ERR_UNSUPPORTED, "latent split: too many rows or splits");
     for (const LsForm& f : kLsForms)
         if (a.ldc <= f.ldc && a.rank_ld <= f.rank) {
             out->func = f.f;

@@ -14,6 +14,7 @@
 // into the latent space, gate / up | attention | W_uv | output), a state-space layer four.
 #include "act_device.hpp"
 #include "layer_decode.hpp"
+#include "split_device.hpp"
 
 namespace fk {
 
@@ -22,6 +23,7 @@ namespace {
 typedef uint32_t ld_u32x4_t __attribute__((ext_vector_type(4)));
 
 constexpr int kJobBlock = 256;
+static_assert(kMaxSplits <= kMaxGateGroups, "both lists share the LDS behind the reduction words");
 constexpr uint32_t kAhead = 4;   // pieces of two rows in flight per wave: a piece is 64 lanes x 16 bytes = 512 elements
 
 __device__ __forceinline__ float dot8(ld_u32x4_t a, ld_u32x4_t b, float s) {
@@ -182,23 +184,18 @@ __device__ void stage_row(const GemvJob& j, uint32_t head, uint32_t first_block,
     } else {   // kRowCombine: the partial rows of one head, [splits][heads][pl] = latent sums | maximum | sum
         const float* p = reinterpret_cast<const float*>(j.x) + (size_t)head * j.pl;
         const size_t ss = (size_t)j.heads * j.pl;
-        float top = bf16_bits_to_f32(j.nw[head]);   // the sink
-        const float sink = top;
-        for (uint32_t s = 0; s < j.splits; ++s) top = fmaxf(top, p[s * ss + j.k]);
-        float l = expf(sink - top);
-        for (uint32_t s = 0; s < j.splits; ++s) l += expf(p[s * ss + j.k] - top) * p[s * ss + j.k + 1u];
-        const float inv = 1.0f / l;
+        float* w = red + 8;
+        split_weights(p + j.k, ss, j.splits, bf16_bits_to_f32(j.nw[head]), w);   // nw: the sinks
+        __syncthreads();
         for (uint32_t c = tid * 2u; c < j.k; c += kJobBlock * 2u) {
             float v0 = 0.f, v1 = 0.f;
+#pragma unroll 8
             for (uint32_t s = 0; s < j.splits; ++s) {
-                const float e = expf(p[s * ss + j.k] - top);
-                if (e != 0.f) {
-                    const float2 q = *reinterpret_cast<const float2*>(p + s * ss + c);
-                    v0 = fmaf(e, q.x, v0);
-                    v1 = fmaf(e, q.y, v1);
-                }
+                const float2 q = *reinterpret_cast<const float2*>(p + s * ss + c);
+                v0 = fmaf(w[s], q.x, v0);
+                v1 = fmaf(w[s], q.y, v1);
             }
-            *reinterpret_cast<uint32_t*>(xs + c) = pack_bf16(v0 * inv, v1 * inv);
+            *reinterpret_cast<uint32_t*>(xs + c) = pack_bf16(v0, v1);
         }
     }
 }
@@ -265,7 +262,11 @@ __device__ void route_wave(const RouteJob& a, uint32_t lane) {
 __device__ void store_row(const StoreJob& a, float* red, float* cs) {
     const uint32_t tid = threadIdx.x, pos = *a.offset, half = a.rot_dims / 2u;
     uint16_t* row = a.cache + (size_t)(pos & (a.ring - 1u)) * a.ldc;
-    for (uint32_t i = tid; i < half; i += kJobBlock) position_cos_sin(pos, a.freq[i], cs[2 * i], cs[2 * i + 1]);
+    for (uint32_t i = tid; i < half; i += kJobBlock) {
+        position_cos_sin(pos, a.freq[i], cs[2 * i], cs[2 * i + 1]);
+        a.tab[2 * i] = cs[2 * i];
+        a.tab[2 * i + 1] = cs[2 * i + 1];
+    }
     float ss = 0.f;
     for (uint32_t c = tid; c < a.rank; c += kJobBlock) ss = fmaf(a.kv[c], a.kv[c], ss);
     ss = block_sum<kJobBlock>(ss, red);
@@ -537,7 +538,7 @@ fk_status plan_layer_jobs(LayerJobsArgs& a, Launch* out) {
         if (!j.w) continue;
         if (j.k % kRowPad || j.ldw < j.k || j.ldw % 8 || j.width > j.k || !j.n) return set_error(FK_ERR_INVALID, "layer jobs: product shape");
         if (j.mode == kRowGated && (!j.groups || j.groups > kMaxGateGroups || j.width % j.groups)) return set_error(FK_ERR_UNSUPPORTED, "layer jobs: at most 64 norm groups");
-        if (j.mode == kRowCombine && (!j.rows_per_head || !j.splits)) return set_error(FK_ERR_INVALID, "layer jobs: combination of what");
+        if (j.mode == kRowCombine && (!j.rows_per_head || !j.splits || j.splits > kMaxSplits)) return set_error(FK_ERR_INVALID, "layer jobs: combination of what");
         if (j.rows_per_head && j.n % j.rows_per_head) return set_error(FK_ERR_INVALID, "layer jobs: rows per head");
         if (!j.rows_per_head) j.y_head = 0;
         else if (j.y_head < j.rows_per_head) return set_error(FK_ERR_INVALID, "layer jobs: outputs per head");

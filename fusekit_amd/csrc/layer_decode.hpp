@@ -52,6 +52,7 @@ struct StoreJob {
     const uint16_t* norm;
     const double* freq;
     uint16_t* cache;
+    float* tab;           // [rot_dims] the rotation of this position (cos, sin per pair), for the queries
     const uint32_t* offset;
     uint32_t rank, rank_ld, ldc, ring, rot, rot_dims;
     float eps;

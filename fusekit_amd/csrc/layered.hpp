@@ -133,13 +133,13 @@ struct LatentSplitArgs {
     const uint16_t* sink;
     uint16_t* out;          // [rows, heads, rank_ld] when combined here
     float* part;
-    const double* freq;     // rotates q while it is read; null: q is rotated already
+    const float* tab;       // [rot_dims] cos, sin per pair: rotates q while it is read; null: q is rotated already
     const uint32_t* offset;
     uint32_t rows, heads, hs, dim_ld, rot, rot_dims, rank_ld, ldc, ldq, ring, window, splits, span;
     float scale;
 };
-constexpr uint32_t kMaxSplitRot = 64;   // rotated pairs
-bool latent_split_supported(uint32_t rank_ld, uint32_t ldc, uint32_t rot_dims);
+constexpr uint32_t kMaxSplits = 64;
+bool latent_split_supported(uint32_t rank_ld, uint32_t ldc);
 fk_status plan_latent_split(LatentSplitArgs& a, bool combine, Launch* out);
 
 // Attention of a pass with keys and values formed from the latents (bf16): row 0 of k / column 0 of vt is position

@@ -10,6 +10,53 @@ namespace fk {
 
 namespace {
 
+// A thread owns one column and walks kConvRows rows, its window of inputs and its weights in registers (up to kConvTaps).
+constexpr uint32_t kConvRows = 16, kConvTaps = 4;
+template <typename T>
+__global__ __launch_bounds__(256) void ssm_conv_rows_kernel(const SsmConvArgs a) {
+    const uint32_t c = (blockIdx.x * 256u + threadIdx.x) * 4u, r0 = blockIdx.y * kConvRows;
+    if (c >= a.channels) return;
+    const uint32_t pos0 = *a.offset;
+    const T* u = reinterpret_cast<const T*>(a.u) + c;
+    const T* hist = reinterpret_cast<const T*>(a.hist) + c;
+    float w[kConvTaps][4], x[kConvTaps][4], b[4];
+#pragma unroll
+    for (uint32_t k = 0; k < kConvTaps; ++k)   // right-aligned: the last entry meets the current row
+#pragma unroll
+        for (uint32_t e = 0; e < 4; ++e) w[k][e] = k + a.taps >= kConvTaps ? bf16_bits_to_f32(a.w[(size_t)(c + e) * a.taps + k + a.taps - kConvTaps]) : 0.f;
+#pragma unroll
+    for (uint32_t e = 0; e < 4; ++e) b[e] = bf16_bits_to_f32(a.b[c + e]);
+    auto input = [&](int32_t r) __attribute__((always_inline)) {   // row r of the pass; before it: the history, zeros before the start
+        if (r >= 0) return act_load4(u + (size_t)r * a.ldu);
+        const int32_t p = (int32_t)pos0 + r;
+        if (p < 0 || -r >= (int32_t)a.taps) return make_float4(0.f, 0.f, 0.f, 0.f);
+        return act_load4(hist + (size_t)((uint32_t)p % a.taps) * a.ldh);
+    };
+    auto put = [&](float (&d)[4], float4 v) __attribute__((always_inline)) { d[0] = v.x; d[1] = v.y; d[2] = v.z; d[3] = v.w; };
+#pragma unroll
+    for (uint32_t k = 0; k + 1u < kConvTaps; ++k) put(x[k + 1], input((int32_t)(r0 + k) - (int32_t)(kConvTaps - 1u)));
+    T* y = reinterpret_cast<T*>(a.y) + c;
+#pragma unroll
+    for (uint32_t i = 0; i < kConvRows; ++i) {
+        const uint32_t r = r0 + i;
+        if (r >= a.rows) break;
+#pragma unroll
+        for (uint32_t k = 0; k + 1u < kConvTaps; ++k)
+#pragma unroll
+            for (uint32_t e = 0; e < 4; ++e) x[k][e] = x[k + 1][e];
+        put(x[kConvTaps - 1], act_load4(u + (size_t)r * a.ldu));
+        float s[4];
+#pragma unroll
+        for (uint32_t e = 0; e < 4; ++e) {
+            s[e] = b[e];
+#pragma unroll
+            for (uint32_t k = 0; k < kConvTaps; ++k) s[e] = fmaf(w[k][e], x[k][e], s[e]);
+            s[e] = silu(s[e]);
+        }
+        act_store4(y + (size_t)r * a.ldy, make_float4(s[0], s[1], s[2], s[3]));
+    }
+}
+
 template <typename T>
 __global__ __launch_bounds__(256) void ssm_conv_kernel(const SsmConvArgs a) {
     const uint32_t c = blockIdx.x * 256u + threadIdx.x, r = blockIdx.y;
@@ -113,8 +160,15 @@ fk_status plan_ssm_conv(const SsmConvArgs& a, uint32_t act, Launch* out) {
     if (act != 16 && act != 32) return set_error(FK_ERR_INVALID, "ssm conv: act must be 16 or 32");
     if (!a.u || !a.w || !a.b || !a.hist || !a.y || !a.offset || !a.rows || !a.channels || !a.taps) return set_error(FK_ERR_INVALID, "ssm conv: bad arguments");
     if (a.rows > 65535) return set_error(FK_ERR_UNSUPPORTED, "ssm conv: at most 65535 rows");
-    out->func = act == 16 ? (const void*)&ssm_conv_kernel<uint16_t> : (const void*)&ssm_conv_kernel<float>;
-    out->grid = dim3((a.channels + 255u) / 256u, a.rows);
+    const uintptr_t align = act == 16 ? 7 : 15;   // four elements per access
+    if (a.rows >= kConvRows && a.taps <= kConvTaps && a.channels % 4 == 0 && a.ldu % 4 == 0 && a.ldy % 4 == 0 && a.ldh % 4 == 0 &&
+        (((uintptr_t)a.u | (uintptr_t)a.hist | (uintptr_t)a.y) & align) == 0) {
+        out->func = act == 16 ? (const void*)&ssm_conv_rows_kernel<uint16_t> : (const void*)&ssm_conv_rows_kernel<float>;
+        out->grid = dim3((a.channels / 4u + 255u) / 256u, (a.rows + kConvRows - 1u) / kConvRows);
+    } else {
+        out->func = act == 16 ? (const void*)&ssm_conv_kernel<uint16_t> : (const void*)&ssm_conv_kernel<float>;
+        out->grid = dim3((a.channels + 255u) / 256u, a.rows);
+    }
     out->block = dim3(256, 1, 1);
     out->shmem = 0;
     out->set_args(a);

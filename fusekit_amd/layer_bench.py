@@ -48,7 +48,13 @@ def _family(kernel: str) -> str:
 def label(t) -> str:
     p = t.params
     f = _family(t.kernel)
-    if f in ("dense", "experts", "layer_in", "layer_out", "head_dense"):
+    if f == "layer_jobs":
+        parts = [f"{int(p[f'g{i}_n'])}x{int(p[f'g{i}_k'])}" for i in (0, 1) if f"g{i}_n" in p]
+        parts += [n for n, k in (("gate/up", "pair_n"), ("choice", "route_outputs"), ("cache row", "store_rank"), ("state step", "scan_heads")) if p.get(k)]
+        return "jobs: " + " | ".join(parts)
+    if f == "layer_out":
+        return "layer out" + (" (o + down)" if p.get("ko") else " (down)")
+    if f in ("dense", "experts"):
         extra = " x%d heads" % p["batch"] if p.get("batch", 1) > 1 else ""
         return f"{f} {int(p['n'])}x{int(p['k'])}{extra}" + (" pair" if p.get("pair") else "")
     return f
@@ -90,9 +96,12 @@ def layer_work(c, rows: int, ctx: int):
             w = {"dense": lambda: p["n"] * p["k"] * p.get("batch", 1) * 2,
                  "experts": lambda: real * p["n"] * p["k"] * 2 * (2 if p.get("pair") else 1),
                  "latent_attn": lambda: min(ctx, lat.window) * lat.ldc * 2,
+                 "latent_split": lambda: min(ctx, lat.window) * lat.ldc * 2,
+                 "layer_out": lambda: p["n"] * (p.get("ko", 0) + real * p.get("kf", 0)) * 2,
+                 "layer_jobs": lambda: sum(p[f"g{i}_n"] * p[f"g{i}_k"] * 2 for i in (0, 1) if f"g{i}_n" in p)
+                 + (2 * real * p["pair_n"] * p["pair_k"] * 2 if p.get("pair_n") else 0)
+                 + (2 * ssm.heads * ssm.vdim * ssm.state * 4 if p.get("scan_heads") else 0),
                  "ssm_scan": lambda: 2 * ssm.heads * ssm.vdim * ssm.state * 4}.get(f)
-            if w is None and "bytes" in p:
-                w = lambda: p["bytes"]
             return (w() if w else 0), 0
         seen = sum(min(i + 1, lat.window) for i in range(rows))
         fl = {"dense": lambda: 2.0 * p["rows"] * p["n"] * p["k"] * p.get("batch", 1),

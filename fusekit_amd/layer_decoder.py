@@ -487,6 +487,7 @@ class LayerRuntime:
                 want("qa", R * m.heads * m.rank_ld * e)
                 want("ol", R * m.heads * m.rank_ld * e)
                 want("att", R * pad(m.heads * m.vdim_ld) * e)
+                want("rot", m.rot_dims * 4)
                 if self._split_latent(m):
                     most = max(rows * self._splits(m, rows)[0] for rows in range(1, R + 1) if not self._long_latent(m, rows))
                     want("part", most * m.heads * (m.rank_ld + 2) * 4)
@@ -521,7 +522,7 @@ class LayerRuntime:
 
     def _split_latent(self, m: LatentAttention) -> bool:
         """The window of a few query rows split over workgroups on the matrix cores (instead of a workgroup per head)."""
-        return self.cfg.act == 16 and self.cfg.tiled and native.latent_split_supported(m.rank_ld, m.ldc, m.rot_dims)
+        return self.cfg.act == 16 and self.cfg.tiled and native.latent_split_supported(m.rank_ld, m.ldc)
 
     def _splits(self, m: LatentAttention, rows: int) -> Tuple[int, int]:
         """(splits, positions per split): whole 64-position tiles, fewer and longer splits as rows fill the device."""
@@ -629,7 +630,7 @@ class LayerRuntime:
         w, b = self.w, self.buf
         splits, span = self._splits(m, rows)
         cache = self.state.entries[run]["cache"]
-        a = [arg(b["qa"]), arg(b["q"]), arg(cache), off] + ([arg(w.vecs[p + "rot_freq"])] if rotate else []) + [arg(b["part"])]
+        a = [arg(b["qa"]), arg(b["q"]), arg(cache), off] + ([arg(b["rot"])] if rotate else []) + [arg(b["part"])]
         a += [] if rotate else [arg(w.vecs[p + "sink"]), arg(b["ol"])]
         return Dispatch(self._name("latent_split"), a,
                         dict(rows=rows, heads=m.heads, hs=m.hs, dim_ld=m.dim_ld, rot=m.rot_dim, rot_dims=m.rot_dims, rank_ld=m.rank_ld,
@@ -697,7 +698,7 @@ class LayerRuntime:
                 # 2: queries, the cache row, the choice of experts
                 Wq, Wk, Wv = w.mats[q + "uq"], w.mats[q + "uk_t"], w.mats[q + "uv"]
                 a = [arg(b["low"]), arg(w.vecs[q + "dq.norm"]), arg(Wq.w), arg(b["q"])] + route
-                a += [arg(b["low"], None, m.q_rank * 4), arg(w.vecs[q + "dkv.norm"]), arg(w.vecs[q + "rot_freq"]), off, arg(st["cache"])]
+                a += [arg(b["low"], None, m.q_rank * 4), arg(w.vecs[q + "dkv.norm"]), arg(w.vecs[q + "rot_freq"]), off, arg(st["cache"]), arg(b["rot"])]
                 self._jobs(t, a, **self._product(0, Wq, Wq.n, mode=1, width=m.q_rank, eps=c.eps), **prm_route, store_rank=m.kv_rank,
                            store_rank_ld=m.rank_ld, store_ldc=m.ldc, store_ring=self.state.rings[run], store_rot=m.rot_dim,
                            store_rot_dims=m.rot_dims, store_eps=c.eps)
@@ -925,7 +926,7 @@ class LayerRuntime:
         out = {n: (getattr(self, n), "uint32", True) for n in ("token", "step_counter", "offset", "kv_len", "hist_counter", "history", "argmax_ws")}
         out["logits"] = (self.logits, "float32", True)
         for n, b in self.buf.items():
-            out[n] = (b, "uint32" if n == "ridx" else "float32" if n in ("x", "mix", "low", "dt", "rl", "rwt") else act, True)
+            out[n] = (b, "uint32" if n in ("ridx", "perm", "tiles", "tile_count") else "float32" if n in ("x", "mix", "low", "dt", "rl", "rwt", "rot", "part", "chunks", "decay") else act, True)
         for r, e in enumerate(self.state.entries):
             for n, b in e.items():
                 out[f"state.{n}.{r}"] = (b, "float32" if n == "state" else act, True)

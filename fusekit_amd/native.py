@@ -645,9 +645,9 @@ def latent_prefill_supported(dim_ld: int, rot_ld: int, vdim_ld: int) -> bool:
     return bool(lib.fk_latent_prefill_supported(C.c_uint32(dim_ld), C.c_uint32(rot_ld), C.c_uint32(vdim_ld)))
 
 
-def latent_split_supported(rank_ld: int, ldc: int, rot_dims: int) -> bool:
+def latent_split_supported(rank_ld: int, ldc: int) -> bool:
     """Whether a latent cache row has the matrix-core form of attention for a few query rows."""
-    return bool(lib.fk_latent_split_supported(C.c_uint32(rank_ld), C.c_uint32(ldc), C.c_uint32(rot_dims)))
+    return bool(lib.fk_latent_split_supported(C.c_uint32(rank_ld), C.c_uint32(ldc)))
 
 
 def ssm_chunk_supported(heads: int, vdim: int, state: int) -> bool:

@@ -657,8 +657,8 @@ fk_status fk_xcd_check(void *workspace, fk_stream s);
  * fusekit_latent_prefill and fusekit_ssm_chunk are the matrix-core forms of attention and recurrence for portions of
  * many rows, fusekit_latent_split the attention of a few rows, fusekit_layer_jobs and fusekit_layer_out the fused
  * launches of one decoded token (all bf16).  These answer whether a shape has such a form (padded head widths; heads,
- * head width, state width; padded latent width, cache row, rotated dimensions). */
-int fk_latent_split_supported(uint32_t rank_ld, uint32_t ldc, uint32_t rot_dims);
+ * head width, state width; padded latent width, cache row). */
+int fk_latent_split_supported(uint32_t rank_ld, uint32_t ldc);
 int fk_latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld);
 int fk_ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n);
 
