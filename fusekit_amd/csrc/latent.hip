@@ -4,7 +4,7 @@
 //     latents and the weighted sum of latents is left to W_uv (decoding and short portions: nothing is formed per key);
 //   * with keys and values formed from the latents for the positions a pass can see (long portions: the pass shares
 //     them, latent_prefill.hip).
-// The window is a parameter: position i sees j with 0 <= i - j < window.  The softmax has a sink, a per-head score
+// `window` counts the positions a query can attend to, its own among them.  The softmax has a sink, a per-head score
 // that enters the denominator only.
 #include "act_device.hpp"
 #include "layered.hpp"

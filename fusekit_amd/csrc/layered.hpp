@@ -32,7 +32,7 @@ struct ResidualNormArgs {
 };
 fk_status plan_residual_norm(const ResidualNormArgs& a, uint32_t act, Launch* out);
 
-// y[r] = x[r] / rms(x[r]) * w in `groups` equal parts, optionally of x * silu(z) (the gate comes before the norm).
+// y[r] = x[r] / rms(x[r]) * w in `groups` equal parts, optionally of the gated row x * silu(z).
 struct GroupNormArgs {
     const void* x;      // [rows, ldx]; fp32 when x32, else act
     const void* z;      // [rows, ldz] (act) or null

@@ -1,6 +1,6 @@
 // State-space mixer with one scalar decay per head (Mamba-2): the short causal convolution and the recurrence
-//     S_t = exp(-exp(a_log) dt_t) S_(t-1) + dt_t B_t x_t^T,   y_t = S_t^T C_t + D x_t
-// with S in fp32.  The state of a head is stored as [vdim][state, padded]: sixteen lanes share one value column and
+//     S <- a S + d (B (x) x),   y = C . S + D x,   d = softplus(dt + bias), a = exp(-d exp(a_log))
+// per token, with S in fp32.  The state of a head is stored as [vdim][state, padded]: sixteen lanes share one value column and
 // hold four adjacent state rows each, so a step's reduction stays inside a row of sixteen lanes and the state of a
 // column moves as whole 16-byte words.
 #include "act_device.hpp"

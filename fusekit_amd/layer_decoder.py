@@ -1,8 +1,8 @@
 """Layer-list decoder on the MI355X backend: a model whose layers are described one by one.
 
 Every layer has a mixer (latent attention over a sliding window, or a Mamba-2 state-space mixer) and optionally a
-mixture-of-experts feed-forward, both reading norms of the same input and added to a 32-bit residual stream together:
-    x <- x + (mixer(norm1(x)) + ff(norm2(x)))
+mixture-of-experts feed-forward.  The two run side by side: each reads its own norm of the layer's input, and their
+outputs join a 32-bit residual stream together.
 A range of layers may run several times in a row with the same weights (`loop`), each pass with its own cache or state
 and a learned vector added before it.  The design that uses it today is Pusavik.
 
