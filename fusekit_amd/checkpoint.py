@@ -335,17 +335,46 @@ def load_moe_checkpoint(model_dir: str, capacity: int = 1024):
     return cfg, w
 
 
-# ---------------------------------------------------------------- layer-list decoders (architecture "Pusavik")
+# ---------------------------------------------------------------- layer-list decoders (architecture "Pusavik", "Fumotar")
 #
-# config.json lists the layers (`layers`: type, mixer, mlp), the looped range (`loop`), `embedding.scale`, `norm.eps`,
-# `vocab` and `width`; tensors are bf16, [out, in].  The low-rank width of the queries may be left to the tensor's shape.
+# config.json lists the layers (`layers`: type, mixer, mlp), the looped range (`loop`), `embedding`, `norm.eps`,
+# `vocab` and `width`; tensors are bf16, [out, in].  Low-rank widths may be left to the tensors' shapes.
 
-def layer_config_from_json(c: dict, shapes: Dict[str, Tuple[int, ...]], act: int = 16):
+LAYER_DESIGNS = {"Pusavik": {}, "Fumotar": dict(layer_norm=True, tied=True, join=True)}
+
+
+def _joint_mixer(i: int, kind: str, m: dict, shapes: Dict[str, Tuple[int, ...]]):
+    from .joint_layers import CausalAttention, ChannelDelta, RgLru, RotaryScaling
+    if kind == "attention":
+        rot = m.get("rot") or {}
+        s = rot.get("scaling")
+        if int(m.get("vdim") or m["dim"]) != int(m["dim"]):
+            raise ValueError(f"layer {i}: values are keys, their widths must agree")
+        return CausalAttention(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), scale=float(m["scale"]),
+                               rot_base=float(rot.get("base", 1.0)), rot_dims=int(rot.get("dims", m["dim"]) if rot else 0),
+                               rot_scaling=RotaryScaling(*(float(s[k]) for k in ("factor", "original", "fast", "slow"))) if s else None)
+    if kind == "channel_delta":
+        return ChannelDelta(heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m["vdim"]), conv=int(m["conv"]),
+                            decay_rank=int(m.get("decay_rank") or shapes[f"l{i}.mix.a1"][0]), gate_rank=int(m.get("gate_rank") or shapes[f"l{i}.mix.g1"][0]))
+    if int(m["width"]) % int(m["blocks"]):
+        raise ValueError(f"layer {i}: width is not a multiple of blocks")
+    return RgLru(width=int(m["width"]), blocks=int(m["blocks"]), conv=int(m["conv"]))
+
+
+def layer_config_from_json(c: dict, shapes: Dict[str, Tuple[int, ...]], act: int = 16, capacity: int = 4096):
     """LayerConfig of a parsed config.json; `shapes` are the checkpoint's tensor shapes."""
-    from .layer_decoder import Experts, Layer, LatentAttention, LayerConfig, Mamba2
+    from .joint_layers import JOINT, DenseMlp
+    from .layer_decoder import Experts, Layer, LatentAttention, LayerConfig, Mamba2, PairTable
+    if c["architecture"] not in LAYER_DESIGNS:
+        raise ValueError(f"unknown architecture {c['architecture']!r}")
     layers = []
     for i, l in enumerate(c["layers"]):
         m, f = l["mixer"], l.get("mlp")
+        if l["type"] in JOINT:
+            if f is not None and f.get("kind", "dense") != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward kind {f['kind']!r}")
+            layers.append(Layer(_joint_mixer(i, l["type"], m, shapes), DenseMlp(int(f["ff"])) if f else None))
+            continue
         if l["type"] == "latent_attention":
             rot = m["rot"]
             mixer = LatentAttention(heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
@@ -364,16 +393,34 @@ def layer_config_from_json(c: dict, shapes: Dict[str, Tuple[int, ...]], act: int
             r = f["router"]
             mlp = Experts(experts=int(r["experts"]), identity=int(r.get("identity") or 0), top=int(r["top"]), ff=int(f["expert"]["ff"]))
         layers.append(Layer(mixer, mlp))
-    loop = c.get("loop") or {}
+    loop, emb = c.get("loop") or {}, c.get("embedding") or {}
+    pairs = emb.get("bigram")
     return LayerConfig(width=int(c["width"]), vocab=int(c["vocab"]), layers=layers, eps=float(c["norm"]["eps"]),
-                       embed_scale=float((c.get("embedding") or {}).get("scale", 1.0)), loop_start=int(loop.get("start", 0)),
-                       loop_stop=int(loop.get("stop", 0)), loop_times=int(loop.get("times", 1)), act=act)
+                       embed_scale=float(emb.get("scale", 1.0)), loop_start=int(loop.get("start", 0)),
+                       loop_stop=int(loop.get("stop", 0)), loop_times=int(loop.get("times", 1)), act=act, capacity=capacity,
+                       design=c["architecture"], pairs=PairTable(*(int(pairs[k]) for k in ("buckets", "mul_prev", "mul_cur"))) if pairs else None,
+                       **LAYER_DESIGNS[c["architecture"]])
+
+
+def _joint_mixer_json(m) -> dict:
+    if m.kind == "attention":
+        rot = dict(base=m.rot_base, dims=m.rot_dims)
+        if m.rot_scaling:
+            s = m.rot_scaling
+            rot["scaling"] = dict(factor=s.factor, original=s.original, fast=s.fast, slow=s.slow)
+        return dict(heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.dim, scale=m.scale, rot=rot)
+    if m.kind == "channel_delta":
+        return dict(heads=m.heads, kv_heads=m.kv_heads, dim=m.dim, vdim=m.vdim, conv=m.conv, decay_rank=m.decay_rank, gate_rank=m.gate_rank)
+    return dict(width=m.width, blocks=m.blocks, conv=m.conv)
 
 
 def layer_config_to_json(cfg) -> dict:
     layers = []
     for l in cfg.layers:
         m, f = l.mixer, l.mlp
+        if l.joint:
+            layers.append(dict(type=m.kind, mixer=_joint_mixer_json(m), mlp=None if f is None else dict(kind="dense", ff=f.ff)))
+            continue
         if m.kind == "latent_attention":
             mixer = dict(heads=m.heads, dim=m.dim, rot_dim=m.rot_dim, vdim=m.vdim, kv_rank=m.kv_rank, q_rank=m.q_rank,
                          mask=dict(size=m.window), scale=m.scale, rot=dict(base=m.rot_base, dims=m.rot_dims))
@@ -381,8 +428,10 @@ def layer_config_to_json(cfg) -> dict:
             mixer = dict(heads=m.heads, vdim=m.vdim, state=m.state, groups=m.groups, conv=m.conv, norm_groups=m.norm_groups)
         mlp = None if f is None else dict(kind="moe", expert=dict(ff=f.ff), router=dict(experts=f.experts, identity=f.identity, top=f.top))
         layers.append(dict(type=m.kind, mixer=mixer, mlp=mlp))
-    out = dict(architecture="Pusavik", vocab=cfg.vocab, width=cfg.width, norm=dict(eps=cfg.eps),
-               embedding=dict(scale=cfg.embed_scale), layers=layers)
+    emb = dict(scale=cfg.embed_scale) if cfg.embed_scale != 1.0 or not cfg.pairs else {}
+    if cfg.pairs:
+        emb["bigram"] = dict(buckets=cfg.pairs.buckets, mul_prev=cfg.pairs.mul_prev, mul_cur=cfg.pairs.mul_cur)
+    out = dict(architecture=cfg.design, vocab=cfg.vocab, width=cfg.width, norm=dict(eps=cfg.eps), embedding=emb, layers=layers)
     if cfg.looped:
         out["loop"] = dict(start=cfg.loop_start, stop=cfg.loop_stop, times=cfg.loop_times)
     return out
@@ -395,7 +444,7 @@ def save_layer_checkpoint(model_dir: str, cfg, tensors: Dict[str, np.ndarray]) -
     json.dump(layer_config_to_json(cfg), open(os.path.join(model_dir, "config.json"), "w"), indent=1)
 
 
-def load_layer_checkpoint(model_dir: str, act: int = 16):
+def load_layer_checkpoint(model_dir: str, act: int = 16, capacity: int = 4096):
     """(LayerConfig, LayerWeights) of a layer-list model; every tensor's dtype and shape is checked against the config."""
     from .layer_decoder import LayerWeights, tensor_shapes
     files = [SafetensorsFile(os.path.join(model_dir, f)) for f in sorted(os.listdir(model_dir)) if f.endswith(".safetensors")]
@@ -403,7 +452,7 @@ def load_layer_checkpoint(model_dir: str, act: int = 16):
         raise FileNotFoundError(f"no .safetensors file in {model_dir}")
     where = {name: f for f in files for name in f.tensors}
     cfg = layer_config_from_json(json.load(open(os.path.join(model_dir, "config.json"))),
-                                 {n: tuple(f.tensors[n]["shape"]) for n, f in where.items()}, act)
+                                 {n: tuple(f.tensors[n]["shape"]) for n, f in where.items()}, act, capacity)
     for name, shape in tensor_shapes(cfg).items():
         if name not in where:
             raise KeyError(f"checkpoint has no tensor {name}")

@@ -20,9 +20,16 @@ __device__ __forceinline__ void act_store4(uint16_t* p, float4 v) {
 }
 __device__ __forceinline__ void act_store4(float* p, float4 v) { *reinterpret_cast<float4*>(p) = v; }
 
+__device__ __forceinline__ float sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
 __device__ __forceinline__ float silu(float z) { return z / (1.0f + expf(-z)); }
 // log(1 + exp(z)) without overflow and without losing small results.
 __device__ __forceinline__ float softplus(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
+
+// 0.5 z (1 + tanh(t)) = z sigmoid(2 t), t = sqrt(2 / pi) (z + 0.044715 z^3)
+__device__ __forceinline__ float gelu_tanh(float z) {
+    const float t = 0.7978845608028654f * fmaf(0.044715f * z * z, z, z);
+    return z * sigmoid(2.0f * t);
+}
 
 // cos / sin of position * freq.  The angle is formed and reduced in double, so its error does not grow with the
 // position; the evaluation is fp32.

@@ -41,7 +41,19 @@ struct TileArgs {
     uint32_t ring, row_back;
     uint32_t m, n, k, ldx, ldw, ldy, x_div, tiles_m, tiles_n;
     uint64_t xb, wstride, yb;   // batch strides; wstride: per batch or per expert
+    ColumnOut out;
 };
+
+// What becomes of one column's sum before it is stored.
+__device__ __forceinline__ float column_value(const ColumnOut& o, uint32_t n, float v) {
+    if (o.bias) v += bf16_bits_to_f32(o.bias[n]);
+    const uint32_t fn = n >= o.begin && n < o.end ? o.fn : n >= o.begin2 ? o.fn2 : (uint32_t)kFnNone;
+    if (fn == kFnRelu2) {
+        v = fmaxf(v, 0.f);
+        return v * v;
+    }
+    return fn == kFnGelu ? gelu_tanh(v) : v;
+}
 
 __device__ __forceinline__ dm_u32x4_t lds_piece(const uint16_t* tile, uint32_t row, uint32_t piece) {
     return *reinterpret_cast<const dm_u32x4_t*>(tile + row * kBK + ((piece ^ (row & 7u)) << 3));
@@ -49,6 +61,7 @@ __device__ __forceinline__ dm_u32x4_t lds_piece(const uint16_t* tile, uint32_t r
 
 template <int BM, int BN, int WM, int WN, int NB, int OUT, bool GROUPED>
 __global__ __launch_bounds__(kTileThreads) void dense_tile_kernel(const TileArgs a) {
+    constexpr bool PLAIN_OUT = OUT != kOutT && NB == 1 && !GROUPED;
     constexpr int TM = BM / WM / 16, TN = BN / WN / 16;   // 16 x 16 tiles per wave
     constexpr int LA = BM / 32, LB = BN / 32;             // 16-byte pieces per thread and staged tile
     static_assert(WM * WN == 4 && BM % 32 == 0 && BN % 32 == 0, "tile shape");
@@ -228,6 +241,16 @@ __global__ __launch_bounds__(kTileThreads) void dense_tile_kernel(const TileArgs
                 const uint32_t mr = mb + l16, n = nb + kq * 4u;
                 if (mr >= live || n >= a.n) continue;
                 const size_t row = GROUPED ? (size_t)a.perm[m0 + mr] : (size_t)(m0 + mr);
+                if (PLAIN_OUT) {
+#pragma unroll
+                    for (int r = 0; r < 4; ++r)
+                        if (n + (uint32_t)r < a.n) v[r] = column_value(a.out, n + (uint32_t)r, v[r]);
+                    if (a.out.tail && n >= a.out.tail_begin) {
+                        for (uint32_t r = 0; r < 4; ++r)
+                            if (n + r < a.n) a.out.tail[row * a.out.ldt + n + r - a.out.tail_begin] = v[r];
+                        continue;
+                    }
+                }
                 const size_t off = (size_t)blockIdx.y * a.yb + row * a.ldy + n;
                 const bool whole = n + 4u <= a.n && (a.ldy & 3u) == 0 && (a.yb & 3u) == 0;
                 if (OUT == kOut32) {
@@ -273,10 +296,11 @@ __global__ __launch_bounds__(256) void dense_few_kernel(const DenseArgs a) {
     }
 #pragma unroll
     for (uint32_t r = 0; r < 8; ++r) {
-        const float v = wave_sum(acc[r]);
+        const float v = column_value(a.out, n, wave_sum(acc[r]));
         if (lane == 0 && r < rows) {
             const size_t off = (size_t)blockIdx.z * a.yb + (size_t)(r0 + r) * a.ldy + n;
-            if (a.y32) reinterpret_cast<float*>(a.y)[off] = v;
+            if (a.out.tail && n >= a.out.tail_begin) a.out.tail[(size_t)(r0 + r) * a.out.ldt + n - a.out.tail_begin] = v;
+            else if (a.y32) reinterpret_cast<float*>(a.y)[off] = v;
             else act_store(reinterpret_cast<T*>(a.y) + off, v);
         }
     }
@@ -315,7 +339,10 @@ __global__ __launch_bounds__(256) void dense_f32_kernel(const DenseArgs a) {
     for (uint32_t i = 0; i < 4; ++i)
         for (uint32_t j = 0; j < 4; ++j) {
             const uint32_t m = m0 + ty * 4u + i, n = n0 + tx * 4u + j;
-            if (m < a.m && n < a.n) y[(size_t)m * a.ldy + n] = acc[i][j];
+            if (m >= a.m || n >= a.n) continue;
+            const float v = column_value(a.out, n, acc[i][j]);
+            if (a.out.tail && n >= a.out.tail_begin) a.out.tail[(size_t)m * a.out.ldt + n - a.out.tail_begin] = v;
+            else y[(size_t)m * a.ldy + n] = v;
         }
 }
 
@@ -336,6 +363,12 @@ fk_status plan_dense(const DenseArgs& a, uint32_t act, Launch* out) {
     if (a.ring && ((a.ring & (a.ring - 1)) || !a.row_base || a.m > a.ring)) return set_error(FK_ERR_INVALID, "dense: the ring must be a power of two of at least m rows");
     if (a.batch > 65535) return set_error(FK_ERR_UNSUPPORTED, "dense: at most 65535 batches");
     if (a.transposed && (act != 16 || a.y32)) return set_error(FK_ERR_UNSUPPORTED, "dense: transposed outputs are bf16");
+    const ColumnOut& o = a.out;
+    if (o.bias || o.tail || o.fn || o.fn2) {
+        if (a.transposed || a.batch != 1) return set_error(FK_ERR_UNSUPPORTED, "dense: column functions go with one row-major product");
+        if (o.fn > kFnMax || o.fn2 > kFnMax || o.begin % 4 || o.end % 4 || o.begin2 % 4 || (o.tail && (o.tail_begin % 4 || o.tail_begin > a.n || o.ldt < a.n - o.tail_begin)))
+            return set_error(FK_ERR_INVALID, "dense: column functions start at multiples of four columns");
+    }
     out->shmem = 0;
     out->block = dim3(256, 1, 1);
     if (act == 32 || (a.m <= 8 && !a.transposed)) {
@@ -356,12 +389,13 @@ fk_status plan_dense(const DenseArgs& a, uint32_t act, Launch* out) {
     t.x = (const uint16_t*)a.x; t.wa = a.w; t.y = a.y; t.row_base = a.row_base; t.ring = a.ring; t.row_back = a.row_back;
     t.m = a.m; t.n = a.n; t.k = a.k; t.ldx = a.ldx; t.ldw = a.ldw; t.ldy = a.ldy;
     t.xb = a.xb; t.wstride = a.wb; t.yb = a.yb;
-    const int o = a.transposed ? kOutT : (a.y32 ? kOut32 : kOutAct);
+    t.out = a.out;
+    const int kind = a.transposed ? kOutT : (a.y32 ? kOut32 : kOutAct);
     auto blocks = [&](uint32_t bm, uint32_t bn) { return (uint64_t)((a.m + bm - 1) / bm) * ((a.n + bn - 1) / bn) * a.batch; };
     uint32_t bm, bn;
-    if (a.m <= 32 || blocks(64, 64) < 128) { bm = 32; bn = 64; out->func = tile_func<32, 64, 1, 4, 1, false>(o); }
-    else if (blocks(128, 128) >= 192) { bm = 128; bn = 128; out->func = tile_func<128, 128, 2, 2, 1, false>(o); }
-    else { bm = 64; bn = 64; out->func = tile_func<64, 64, 2, 2, 1, false>(o); }
+    if (a.m <= 32 || blocks(64, 64) < 128) { bm = 32; bn = 64; out->func = tile_func<32, 64, 1, 4, 1, false>(kind); }
+    else if (blocks(128, 128) >= 192) { bm = 128; bn = 128; out->func = tile_func<128, 128, 2, 2, 1, false>(kind); }
+    else { bm = 64; bn = 64; out->func = tile_func<64, 64, 2, 2, 1, false>(kind); }
     t.tiles_m = (a.m + bm - 1) / bm;
     t.tiles_n = (a.n + bn - 1) / bn;
     const uint64_t g = ((uint64_t)t.tiles_m * t.tiles_n + 7) / 8 * 8;

@@ -619,13 +619,14 @@ fk_status plan_sdpa_prefill_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     FK_TRY(need_bytes(d, 0, (size_t)rows * n_heads * dim * 2));
     FK_TRY(need_bytes(d, 1, (size_t)n_kv * capacity * dim * 2));
     FK_TRY(need_bytes(d, 2, (size_t)n_kv * capacity * dim * 2));
-    FK_TRY(need_bytes(d, out_slot, (size_t)rows * n_heads * dim * 2));
+    const uint32_t ldo = d.u("ldo", n_heads * dim);
+    FK_TRY(need_bytes(d, out_slot, ((size_t)(rows - 1) * ldo + (size_t)n_heads * dim) * 2));
     rw->reads = {0, 1, 2};
     if (dev_len) rw->reads.push_back(3);
     rw->writes = {(uint32_t)out_slot};
     return plan_sdpa_prefill(arg_ptr<const uint16_t>(d, 0), arg_ptr<const uint16_t>(d, 1), arg_ptr<const uint16_t>(d, 2),
                              arg_ptr<uint16_t>(d, out_slot), rows, kv_len, n_heads, n_kv, dim, capacity, scale, l,
-                             dev_len ? arg_ptr<const uint32_t>(d, 3) : nullptr);
+                             dev_len ? arg_ptr<const uint32_t>(d, 3) : nullptr, ldo);
 }
 
 // x, weight, out: RMSNorm of `rows` rows, T(w * T(x * r)) (the norm stage of the reference's multi-row
@@ -1561,6 +1562,13 @@ const Family kFamilies[] = {
     {"fusekit_latent_attn", plan_latent_attn_d},
     {"fusekit_ssm_conv", plan_ssm_conv_d},
     {"fusekit_ssm_scan", plan_ssm_scan_d},
+    {"fusekit_embed_rows", plan_embed_rows_d},
+    {"fusekit_head_norm", plan_head_norm_d},
+    {"fusekit_qk_store", plan_qk_store_d},
+    {"fusekit_gqa_rows", plan_gqa_rows_d},
+    {"fusekit_delta_prep", plan_delta_prep_d},
+    {"fusekit_delta_scan", plan_delta_scan_d},
+    {"fusekit_lru_scan", plan_lru_scan_d},
     {"fusekit_latent_prefill", plan_latent_prefill_d},
     {"fusekit_ssm_chunk", plan_ssm_chunk_d},
     {"fusekit_latent_split", plan_latent_split_d},

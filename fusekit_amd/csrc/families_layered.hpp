@@ -43,8 +43,9 @@ uint64_t act_bytes(uint32_t act) { return act == 32 ? 4 : 2; }
 // Bytes from the first element of row 0 to the last valid one of row rows - 1.
 uint64_t rows_bytes(uint64_t rows, uint64_t ld, uint64_t width, uint64_t elem) { return ((rows - 1) * ld + width) * elem; }
 
-// x, [mix: has_mix], [routes, weight, index, prev: top > 0], [step: has_step], [w1, h1: has_h1], [w2, h2: has_h2]
-//   {rows, width, ld, act, eps, top, experts}
+// x, [mix: has_mix], [routes, weight, index, prev: top > 0], [step: has_step], [copy: ldcopy > 0], [w1, [b1: layer_norm], h1:
+// has_h1], [w2, h2: has_h2]
+//   {rows, width, ld, ldcopy, act, eps, top, experts}
 fk_status plan_residual_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     ResidualNormArgs a;
     memset(&a, 0, sizeof(a));
@@ -63,7 +64,13 @@ fk_status plan_residual_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
         a.prev = s.in(xa);
     }
     if (d.u("has_step")) a.step = s.in<uint16_t>((uint64_t)a.ldx * 2);
-    if (d.u("has_h1")) { a.w1 = s.in<uint16_t>((uint64_t)a.ldx * 2); a.h1 = s.out(xa); }
+    a.ldcopy = d.u("ldcopy");
+    if (a.ldcopy) a.copy = s.out(rows_bytes(a.rows, a.ldcopy, a.ldx, act_bytes(act)));
+    if (d.u("has_h1")) {
+        a.w1 = s.in<uint16_t>((uint64_t)a.ldx * 2);
+        if (d.u("layer_norm")) a.b1 = s.in<uint16_t>((uint64_t)a.ldx * 2);
+        a.h1 = s.out(xa);
+    }
     if (d.u("has_h2")) { a.w2 = s.in<uint16_t>((uint64_t)a.ldx * 2); a.h2 = s.out(xa); }
     FK_TRY(s.end());
     return plan_residual_norm(a, act, l);
@@ -86,7 +93,9 @@ fk_status plan_group_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     return plan_group_norm(a, act, l);
 }
 
-// x, w, [row_base: ring > 0], y   {rows, n, k, ldx, ldw, ldy, batch=1, xb, wb, yb, y32, transposed, ring, row_back, act}
+// x, w, [row_base: ring > 0], [bias: has_bias], y, [tail: ldt > 0]
+//   {rows, n, k, ldx, ldw, ldy, batch=1, xb, wb, yb, y32, transposed, ring, row_back, act,
+//    fn, fn_begin, fn_end, fn2, fn2_begin (ColumnFn), tail_begin, ldt}
 fk_status plan_dense_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     DenseArgs a;
     memset(&a, 0, sizeof(a));
@@ -101,11 +110,159 @@ fk_status plan_dense_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     a.x = s.in(((a.batch - 1) * a.xb + (uint64_t)((a.ring ? a.ring : a.m) - 1) * a.ldx + a.k) * e);
     a.w = s.in<uint16_t>(((a.batch - 1) * a.wb + (uint64_t)(a.n - 1) * a.ldw + a.k) * 2);
     if (a.ring) a.row_base = s.in<uint32_t>(4);
-    const uint64_t rows = a.transposed ? a.n : a.m, cols = a.transposed ? a.m : a.n;
+    a.out.fn = d.u("fn"); a.out.begin = d.u("fn_begin"); a.out.end = d.u("fn_end"); a.out.fn2 = d.u("fn2"); a.out.begin2 = d.u("fn2_begin");
+    a.out.ldt = d.u("ldt"); a.out.tail_begin = a.out.ldt ? d.u("tail_begin") : a.n;
+    if (a.out.tail_begin > a.n) return set_error(FK_ERR_INVALID, d.kernel + ": tail_begin past the columns");
+    if (d.u("has_bias")) a.out.bias = s.in<uint16_t>((uint64_t)a.n * 2);
+    const uint64_t rows = a.transposed ? a.n : a.m, cols = a.transposed ? a.m : a.out.tail_begin;
     if (a.ldy < cols && rows > 1) return set_error(FK_ERR_INVALID, d.kernel + ": ldy below the output width");
     a.y = s.out(((a.batch - 1) * a.yb + (rows - 1) * a.ldy + cols) * ye);
+    if (a.out.ldt && a.out.tail_begin < a.n) a.out.tail = s.out<float>(rows_bytes(a.m, a.out.ldt, a.n - a.out.tail_begin, 4));
     FK_TRY(s.end());
     return plan_dense(a, act, l);
+}
+
+// tokens, table, [pairs, prev, offset: buckets > 0], x, [copy: ldcopy > 0]
+//   {rows, width, vocab, ldw, ld, ldcopy, buckets, mul_prev, mul_cur, scale=1, act}
+fk_status plan_embed_rows_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    EmbedRowsArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.width = d.u("width"); a.vocab = d.u("vocab"); a.ldw = d.u("ldw", a.width); a.ldx = d.u("ld", a.width); a.ldcopy = d.u("ldcopy");
+    a.buckets = d.u("buckets"); a.mul_prev = d.u("mul_prev"); a.mul_cur = d.u("mul_cur"); a.scale = (float)d.param("scale", 1.0);
+    if (!a.rows || !a.width || !a.vocab) return set_error(FK_ERR_INVALID, d.kernel + ": rows / width / vocab parameters missing");
+    SlotCursor s{d, rw};
+    a.tokens = s.in<uint32_t>((uint64_t)a.rows * 4);
+    a.table = s.in<uint16_t>((uint64_t)a.vocab * a.ldw * 2);
+    if (a.buckets) {
+        a.pairs = s.in<uint16_t>(((uint64_t)a.buckets + 1) * a.ldw * 2);
+        a.prev = s.inout<uint32_t>(4);
+        a.offset = s.in<uint32_t>(4);
+    }
+    a.x = s.out<float>((uint64_t)a.rows * a.ldx * 4);
+    if (a.ldcopy) a.copy = s.out(rows_bytes(a.rows, a.ldcopy, a.ldx, act_bytes(act)));
+    FK_TRY(s.end());
+    return plan_embed_rows(a, act, l);
+}
+
+// x, z, w, y   {rows, heads, dim, ld, ldx, ldz, ldy, eps, act}
+fk_status plan_head_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    HeadNormArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.dim = d.u("dim"); a.ld = d.u("ld", a.dim); a.eps = (float)d.param("eps", 1e-6);
+    const uint32_t n = a.heads * a.ld;
+    a.ldx = d.u("ldx", n); a.ldz = d.u("ldz", n); a.ldy = d.u("ldy", n);
+    if (!a.rows || !n || a.ldx < n || a.ldz < n || a.ldy < n) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.x = s.in<float>(rows_bytes(a.rows, a.ldx, n, 4));
+    a.z = s.in(rows_bytes(a.rows, a.ldz, n, act_bytes(act)));
+    a.w = s.in<uint16_t>((uint64_t)a.ld * 2);
+    a.y = s.out(rows_bytes(a.rows, a.ldy, n, act_bytes(act)));
+    FK_TRY(s.end());
+    return plan_head_norm(a, act, l);
+}
+
+// u, q norm, k norm, freq, offset, q, cache_k, cache_v
+//   {rows, heads, kv_heads, dim, dim_ld, rot_dims, ldu, k0, q0, capacity, mag=1, eps, act}
+fk_status plan_qk_store_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    QkStoreArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.kv_heads = d.u("kv_heads"); a.dim = d.u("dim"); a.dim_ld = d.u("dim_ld", a.dim); a.rot_dims = d.u("rot_dims");
+    a.ldu = d.u("ldu"); a.k0 = d.u("k0"); a.q0 = d.u("q0"); a.capacity = d.u("capacity"); a.eps = (float)d.param("eps", 1e-6); a.mag = (float)d.param("mag", 1.0);
+    if (!a.rows || !a.heads || !a.kv_heads || !a.dim || !a.capacity) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    const uint64_t e = act_bytes(act), nq = (uint64_t)a.heads * a.dim_ld, nk = (uint64_t)a.kv_heads * a.dim_ld;
+    SlotCursor s{d, rw};
+    a.u = s.in(rows_bytes(a.rows, a.ldu, std::max(a.k0 + nk, a.q0 + nq), e));
+    a.wq = s.in<uint16_t>(nq * 2);
+    a.wk = s.in<uint16_t>(nk * 2);
+    a.freq = s.in<double>(a.rot_dims >= 2 ? (uint64_t)(a.rot_dims / 2) * 8 : 1);
+    a.offset = s.in<uint32_t>(4);
+    a.q = s.out(a.rows * nq * e);
+    a.cache_k = s.inout(nk * a.capacity * e);
+    a.cache_v = s.inout(nk * a.capacity * e);
+    FK_TRY(s.end());
+    return plan_qk_store(a, act, l);
+}
+
+// q, cache_k, cache_v, offset, out   {rows, heads, kv_heads, dim_ld, capacity, ldo, scale, act}
+fk_status plan_gqa_rows_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    GqaRowsArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.kv_heads = d.u("kv_heads"); a.dim_ld = d.u("dim_ld"); a.capacity = d.u("capacity");
+    const uint64_t e = act_bytes(act), nq = (uint64_t)a.heads * a.dim_ld, nk = (uint64_t)a.kv_heads * a.dim_ld;
+    a.ldo = d.u("ldo", (uint32_t)nq); a.scale = (float)d.param("scale", 1.0);
+    if (!a.rows || !nq || !nk || !a.capacity) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.q = s.in(a.rows * nq * e);
+    a.cache_k = s.in(nk * a.capacity * e);
+    a.cache_v = s.in(nk * a.capacity * e);
+    a.offset = s.in<uint32_t>(4);
+    a.out = s.out(rows_bytes(a.rows, a.ldo, nq, e));
+    FK_TRY(s.end());
+    return plan_gqa_rows(a, act, l);
+}
+
+// xc, dt_bias, a_log, decay, beta, qk   {rows, heads, kv_heads, dim, dim_ld, ldx, ldb, act}
+fk_status plan_delta_prep_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    DeltaPrepArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.kv_heads = d.u("kv_heads"); a.dim = d.u("dim"); a.dim_ld = d.u("dim_ld", a.dim); a.ldx = d.u("ldx"); a.ldb = d.u("ldb", a.heads);
+    const uint64_t nk = (uint64_t)a.kv_heads * a.dim_ld, nd = (uint64_t)a.heads * a.dim_ld;
+    if (!a.rows || !nk || !nd || a.ldx < 2 * nk) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.xc = s.in(rows_bytes(a.rows, a.ldx, 2 * nk, act_bytes(act)));
+    a.dt_bias = s.in<uint16_t>(nd * 2);
+    a.a_log = s.in<uint16_t>((uint64_t)a.heads * 2);
+    a.decay = s.inout<float>(a.rows * nd * 4);
+    a.beta = s.inout<float>(rows_bytes(a.rows, a.ldb, a.heads, 4));
+    a.qk = s.out<float>(a.rows * nk * 8);
+    FK_TRY(s.end());
+    return plan_delta_prep(a, act, l);
+}
+
+// qk, decay, beta, v, state, o   {rows, heads, kv_heads, dim_ld, vdim_ld, state_ld, ldx, ldb, act}
+fk_status plan_delta_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    DeltaScanArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.kv_heads = d.u("kv_heads"); a.dim_ld = d.u("dim_ld"); a.vdim_ld = d.u("vdim_ld"); a.state_ld = d.u("state_ld");
+    a.ldx = d.u("ldx"); a.ldb = d.u("ldb", a.heads);
+    const uint64_t nk = (uint64_t)a.kv_heads * a.dim_ld, nd = (uint64_t)a.heads * a.dim_ld, nv = (uint64_t)a.heads * a.vdim_ld;
+    if (!a.rows || !nk || !nv || !a.state_ld || a.ldx < nv) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.qk = s.in<float>(a.rows * nk * 8);
+    a.decay = s.in<float>(a.rows * nd * 4);
+    a.beta = s.in<float>(rows_bytes(a.rows, a.ldb, a.heads, 4));
+    a.v = s.in(rows_bytes(a.rows, a.ldx, nv, act_bytes(act)));
+    a.state = s.inout<float>(nv * a.state_ld * 4);
+    a.o = s.out<float>(a.rows * nv * 4);
+    FK_TRY(s.end());
+    return plan_delta_scan(a, act, l);
+}
+
+// u, gates, r bias, i bias, lam, state, y, carry   {rows, width, block, ldx, ldy, act}; carry holds 2 * width words per 32 rows
+fk_status plan_lru_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    LruScanArgs a;
+    memset(&a, 0, sizeof(a));
+    const uint32_t act = d.u("act", 16);
+    a.rows = d.u("rows", 1); a.width = d.u("width"); a.block = d.u("block", a.width); a.ldx = d.u("ldx", a.width); a.ldy = d.u("ldy", a.width);
+    if (!a.rows || !a.width || a.ldx < a.width || a.ldy < a.width) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    const uint64_t e = act_bytes(act), w2 = (uint64_t)a.width * 2;
+    SlotCursor s{d, rw};
+    a.u = s.in(rows_bytes(a.rows, a.ldx, a.width, e));
+    a.gates = s.in<float>(a.rows * w2 * 4);
+    a.rb = s.in<uint16_t>(w2);
+    a.ib = s.in<uint16_t>(w2);
+    a.lam = s.in<uint16_t>(w2);
+    a.state = s.inout<float>(w2 * 2);
+    a.y = s.inout(rows_bytes(a.rows, a.ldy, a.width, e));
+    a.carry = s.inout<float>((a.rows + kLruChunk - 1) / kLruChunk * w2 * 4);
+    FK_TRY(s.end());
+    return plan_lru_scan(a, act, l);
 }
 
 // logits, correction, index, weight   {rows, outputs, top, ld}
@@ -206,7 +363,7 @@ fk_status plan_latent_attn_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     return plan_latent_attn(a, act, l);
 }
 
-// u, w, b, hist, offset, y   {rows, channels, taps, ldu, ldy, ldh, act}
+// u, w, [b: has_bias=1], hist, offset, y   {rows, channels, taps, ldu, ldy, ldh, linear, update, act}
 fk_status plan_ssm_conv_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     SsmConvArgs a;
     memset(&a, 0, sizeof(a));
@@ -217,8 +374,9 @@ fk_status plan_ssm_conv_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     SlotCursor s{d, rw};
     a.u = s.in(rows_bytes(a.rows, a.ldu, a.channels, e));
     a.w = s.in<uint16_t>((uint64_t)a.channels * a.taps * 2);
-    a.b = s.in<uint16_t>((uint64_t)a.channels * 2);
-    a.hist = s.in((uint64_t)a.taps * a.ldh * e);
+    if (d.u("has_bias", 1)) a.b = s.in<uint16_t>((uint64_t)a.channels * 2);
+    a.linear = d.u("linear"); a.update = d.u("update");
+    a.hist = a.update ? s.inout((uint64_t)a.taps * a.ldh * e) : const_cast<void*>(s.in((uint64_t)a.taps * a.ldh * e));
     a.offset = s.in<uint32_t>(4);
     a.y = s.out(rows_bytes(a.rows, a.ldy, a.channels, e));
     FK_TRY(s.end());

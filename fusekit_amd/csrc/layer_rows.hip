@@ -18,7 +18,8 @@ __global__ __launch_bounds__(kRowBlock) void residual_norm_kernel(const Residual
     const float* mix = a.mix ? a.mix + (size_t)r * a.ldx : nullptr;
     const T* prev = a.prev ? reinterpret_cast<const T*>(a.prev) + (size_t)r * a.ldx : nullptr;
     const T* routes = a.routes ? reinterpret_cast<const T*>(a.routes) + (size_t)r * a.top * a.ldx : nullptr;
-    float ss = 0.f;
+    T* copy = a.copy ? reinterpret_cast<T*>(a.copy) + (size_t)r * a.ldcopy : nullptr;
+    float ss = 0.f, sum = 0.f;
     for (uint32_t c = threadIdx.x * 4u; c < a.ldx; c += kRowBlock * 4u) {
         float4 v = *reinterpret_cast<const float4*>(x + c);
         float4 add = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -38,9 +39,30 @@ __global__ __launch_bounds__(kRowBlock) void residual_norm_kernel(const Residual
             v.x += s.x; v.y += s.y; v.z += s.z; v.w += s.w;
         }
         *reinterpret_cast<float4*>(x + c) = v;
+        if (copy) act_store4(copy + c, v);
+        sum += (v.x + v.y) + (v.z + v.w);
         ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
     }
     if (!a.w1 && !a.w2) return;
+    if (a.b1) {   // layer norm: the padding is outside the mean of the squared deviations, and its weight and bias are zero
+        const float mean = block_sum<kRowBlock>(sum, red) / (float)a.width;
+        __syncthreads();
+        float dev = 0.f;
+        for (uint32_t c = threadIdx.x * 4u; c < a.ldx; c += kRowBlock * 4u) {
+            const float4 v = *reinterpret_cast<const float4*>(x + c);
+            const float d[4] = {v.x - mean, v.y - mean, v.z - mean, v.w - mean};
+#pragma unroll
+            for (uint32_t e = 0; e < 4; ++e)
+                if (c + e < a.width) dev = fmaf(d[e], d[e], dev);
+        }
+        const float k = 1.0f / sqrtf(block_sum<kRowBlock>(dev, red) / (float)a.width + a.eps);
+        for (uint32_t c = threadIdx.x * 4u; c < a.ldx; c += kRowBlock * 4u) {
+            const float4 v = *reinterpret_cast<const float4*>(x + c), w = act_load4(a.w1 + c), b = act_load4(a.b1 + c);
+            act_store4(reinterpret_cast<T*>(a.h1) + (size_t)r * a.ldx + c,
+                       make_float4(fmaf((v.x - mean) * k, w.x, b.x), fmaf((v.y - mean) * k, w.y, b.y), fmaf((v.z - mean) * k, w.z, b.z), fmaf((v.w - mean) * k, w.w, b.w)));
+        }
+        return;
+    }
     ss = block_sum<kRowBlock>(ss, red);
     const float k = 1.0f / sqrtf(ss / (float)a.width + a.eps);
     for (uint32_t c = threadIdx.x * 4u; c < a.ldx; c += kRowBlock * 4u) {
@@ -77,6 +99,59 @@ __global__ __launch_bounds__(kRowBlock) void group_norm_kernel(const GroupNormAr
     const float k = 1.0f / sqrtf(ss / (float)part + a.eps);
     T* y = reinterpret_cast<T*>(a.y) + (size_t)r * a.ldy;
     for (uint32_t c = c0 + threadIdx.x; c < c0 + part; c += kRowBlock) act_store(y + c, value(c) * k * bf16_bits_to_f32(a.w[c]));
+}
+
+// One block per row.  The block of row 0 is the only one that needs the token before the pass: it reads that word, then
+// leaves the pass's last token in its place.
+template <typename T>
+__global__ __launch_bounds__(kRowBlock) void embed_rows_kernel(const EmbedRowsArgs a) {
+    const uint32_t r = blockIdx.x;
+    const uint32_t raw = a.tokens[r], tok = raw < a.vocab ? raw : a.vocab - 1u;
+    const uint16_t* second = nullptr;
+    if (a.pairs) {
+        uint32_t row = a.buckets;
+        if (*a.offset + r > 0u) {
+            const uint32_t before = r ? a.tokens[r - 1u] : *a.prev;
+            row = (uint32_t)(((uint64_t)before * a.mul_prev + (uint64_t)tok * a.mul_cur) % a.buckets);
+        }
+        second = a.pairs + (size_t)row * a.ldw;
+        if (r == 0) {
+            __syncthreads();
+            if (threadIdx.x == 0) *a.prev = a.tokens[a.rows - 1u];
+        }
+    }
+    const uint16_t* first = a.table + (size_t)tok * a.ldw;
+    for (uint32_t c = threadIdx.x * 4u; c < a.ldx; c += kRowBlock * 4u) {
+        float4 v = act_load4(first + c);
+        v.x *= a.scale; v.y *= a.scale; v.z *= a.scale; v.w *= a.scale;
+        if (second) {
+            const float4 p = act_load4(second + c);
+            v.x += p.x; v.y += p.y; v.z += p.z; v.w += p.w;
+        }
+        *reinterpret_cast<float4*>(a.x + (size_t)r * a.ldx + c) = v;
+        if (a.copy) act_store4(reinterpret_cast<T*>(a.copy) + (size_t)r * a.ldcopy + c, v);
+    }
+}
+
+// A wave per (row, head).
+template <typename T>
+__global__ __launch_bounds__(kRowBlock) void head_norm_kernel(const HeadNormArgs a) {
+    const uint32_t lane = threadIdx.x & (kWave - 1u), i = blockIdx.x * (kRowBlock / kWave) + threadIdx.x / kWave;
+    if (i >= a.rows * a.heads) return;
+    const uint32_t r = i / a.heads, h = i - r * a.heads;
+    const float* x = a.x + (size_t)r * a.ldx + (size_t)h * a.ld;
+    const T* z = reinterpret_cast<const T*>(a.z) + (size_t)r * a.ldz + (size_t)h * a.ld;
+    T* y = reinterpret_cast<T*>(a.y) + (size_t)r * a.ldy + (size_t)h * a.ld;
+    float ss = 0.f;
+    for (uint32_t c = lane * 4u; c < a.ld; c += kWave * 4u) {
+        const float4 v = *reinterpret_cast<const float4*>(x + c);
+        ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
+    }
+    const float k = 1.0f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps);
+    for (uint32_t c = lane * 4u; c < a.ld; c += kWave * 4u) {
+        const float4 v = *reinterpret_cast<const float4*>(x + c), w = act_load4(a.w + c), g = act_load4(z + c);
+        act_store4(y + c, make_float4(v.x * k * w.x * sigmoid(g.x), v.y * k * w.y * sigmoid(g.y), v.z * k * w.z * sigmoid(g.z), v.w * k * w.w * sigmoid(g.w)));
+    }
 }
 
 // One wave per token.  The scores stay in registers, lane l holding outputs l, l + 64, ...; a selection round is a
@@ -229,6 +304,8 @@ fk_status plan_experts_grouped(const ExpertArgs& a, Launch* out);   // dense_mfm
 fk_status plan_residual_norm(const ResidualNormArgs& a, uint32_t act, Launch* out) {
     FK_TRY(check_act(act, "residual norm"));
     if (!a.x || !a.rows || !a.width || a.ldx % kRowPad || a.ldx < a.width) return set_error(FK_ERR_INVALID, "residual norm: bad shape");
+    if (a.b1 && (!a.w1 || a.w2)) return set_error(FK_ERR_INVALID, "residual norm: a layer norm is the only norm");
+    if (a.copy && (a.ldcopy % 4 || a.ldcopy < a.ldx)) return set_error(FK_ERR_INVALID, "residual norm: copies go to padded rows");
     if ((a.w1 && !a.h1) || (a.w2 && !a.h2)) return set_error(FK_ERR_INVALID, "residual norm: a norm without an output");
     if (a.routes && (!a.weight || !a.index || !a.prev || !a.top)) return set_error(FK_ERR_INVALID, "residual norm: incomplete routes");
     fill(out, act == 16 ? (const void*)&residual_norm_kernel<uint16_t> : (const void*)&residual_norm_kernel<float>, dim3(a.rows), kRowBlock, 0, a);
@@ -240,6 +317,25 @@ fk_status plan_group_norm(const GroupNormArgs& a, uint32_t act, Launch* out) {
     if (!a.x || !a.w || !a.y || !a.rows || !a.groups || a.width % a.groups || !a.width) return set_error(FK_ERR_INVALID, "group norm: bad shape");
     if (a.groups > 65535) return set_error(FK_ERR_UNSUPPORTED, "group norm: too many groups");
     fill(out, act == 16 ? (const void*)&group_norm_kernel<uint16_t> : (const void*)&group_norm_kernel<float>, dim3(a.rows, a.groups), kRowBlock, 0, a);
+    return FK_OK;
+}
+
+fk_status plan_embed_rows(const EmbedRowsArgs& a, uint32_t act, Launch* out) {
+    FK_TRY(check_act(act, "embedding rows"));
+    if (!a.tokens || !a.table || !a.x || !a.rows || !a.vocab || a.ldx % kRowPad || a.ldx < a.width || a.ldw % 4 || a.ldw < a.ldx)
+        return set_error(FK_ERR_INVALID, "embedding rows: bad shape");
+    if (a.pairs && (!a.buckets || !a.prev || !a.offset)) return set_error(FK_ERR_INVALID, "embedding rows: incomplete second table");
+    if (a.copy && (a.ldcopy % 4 || a.ldcopy < a.ldx)) return set_error(FK_ERR_INVALID, "embedding rows: copies go to padded rows");
+    fill(out, act == 16 ? (const void*)&embed_rows_kernel<uint16_t> : (const void*)&embed_rows_kernel<float>, dim3(a.rows), kRowBlock, 0, a);
+    return FK_OK;
+}
+
+fk_status plan_head_norm(const HeadNormArgs& a, uint32_t act, Launch* out) {
+    FK_TRY(check_act(act, "head norm"));
+    if (!a.x || !a.z || !a.w || !a.y || !a.rows || !a.heads || !a.dim || a.ld < a.dim || a.ld % 4 || a.ldx % 4 || a.ldz % 4 || a.ldy % 4)
+        return set_error(FK_ERR_INVALID, "head norm: bad shape");
+    fill(out, act == 16 ? (const void*)&head_norm_kernel<uint16_t> : (const void*)&head_norm_kernel<float>,
+         dim3((uint32_t)(((uint64_t)a.rows * a.heads + 3u) / 4u)), kRowBlock, 0, a);
     return FK_OK;
 }
 

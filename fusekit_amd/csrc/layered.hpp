@@ -14,7 +14,8 @@ namespace fk {
 
 constexpr uint32_t kRowPad = 64;
 
-// x += mixer output + feed-forward output (+ a constant vector), then up to two RMS norms of the new x.
+// x += mixer output + feed-forward output (+ a constant vector), then up to two norms of the new x: RMS norms, or layer
+// norms where a bias is given.
 struct ResidualNormArgs {
     float* x;               // [rows, ldx]
     const float* mix;       // [rows, ldx] or null
@@ -25,9 +26,11 @@ struct ResidualNormArgs {
     const uint16_t* step;   // [width] added as well, or null
     const uint16_t* w1;     // norm weights [ldx] or null
     const uint16_t* w2;
+    const uint16_t* b1;     // layer norm's bias [ldx], or null: RMS norm (the second norm is always one)
     void* h1;               // [rows, ldx] (act)
     void* h2;
-    uint32_t rows, width, ldx, top, experts;
+    void* copy;             // [rows, ldcopy] (act): the new x itself, or null
+    uint32_t rows, width, ldx, top, experts, ldcopy;
     float eps;
 };
 fk_status plan_residual_norm(const ResidualNormArgs& a, uint32_t act, Launch* out);
@@ -43,6 +46,46 @@ struct GroupNormArgs {
 };
 fk_status plan_group_norm(const GroupNormArgs& a, uint32_t act, Launch* out);
 
+// What becomes of a product's columns before they are stored.  All bounds are multiples of four columns.
+enum ColumnFn : uint32_t {
+    kFnNone = 0,
+    kFnRelu2 = 1,   // the square of relu
+    kFnGelu = 2,    // gelu, tanh form
+    kFnMax = 2,
+};
+struct ColumnOut {
+    const uint16_t* bias;       // [n] added first, or null
+    float* tail;                // columns tail_begin .. are stored here as fp32 instead, or null
+    uint32_t fn, begin, end;    // function of columns begin .. end - 1
+    uint32_t fn2, begin2;       // function of columns begin2 ..
+    uint32_t tail_begin, ldt;
+};
+
+// Token rows: x = scale * table[token] (+ a row of a second table, chosen by a hash of the token and the one before it).
+struct EmbedRowsArgs {
+    const uint32_t* tokens;   // [rows]
+    const uint16_t* table;    // [vocab, ldw]
+    const uint16_t* pairs;    // [buckets + 1, ldw] or null; the last row is for the first token of a sequence
+    uint32_t* prev;           // the token before the pass; becomes the last one of it
+    const uint32_t* offset;
+    float* x;                 // [rows, ldx]
+    void* copy;               // [rows, ldcopy] (act) or null
+    uint32_t rows, width, vocab, buckets, mul_prev, mul_cur, ldw, ldx, ldcopy;
+    float scale;
+};
+fk_status plan_embed_rows(const EmbedRowsArgs& a, uint32_t act, Launch* out);
+
+// y[r, h] = x[r, h] / rms(x[r, h]) * w * sigmoid(z[r, h]) per head of `dim` elements (`ld` padded).
+struct HeadNormArgs {
+    const float* x;      // [rows, ldx]
+    const void* z;       // [rows, ldz] (act)
+    const uint16_t* w;   // [ld], shared by the heads
+    void* y;             // [rows, ldy] (act)
+    uint32_t rows, heads, dim, ld, ldx, ldz, ldy;
+    float eps;
+};
+fk_status plan_head_norm(const HeadNormArgs& a, uint32_t act, Launch* out);
+
 // y[b][m, n] = x[b][m, k] . w[b][n, k]^T.
 struct DenseArgs {
     const void* x;
@@ -54,6 +97,7 @@ struct DenseArgs {
     uint32_t ldx, ldw, ldy, batch;
     uint64_t xb, wb, yb;       // elements between batches
     uint32_t y32, transposed;  // transposed: y[b][n, m] (bf16 matrix-core form only)
+    ColumnOut out;             // row-major outputs of plain rows only
 };
 fk_status plan_dense(const DenseArgs& a, uint32_t act, Launch* out);
 
@@ -159,16 +203,17 @@ bool latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld
 fk_status plan_latent_prefill(const LatentPrefillArgs& a, Launch* out);
 
 // ---- state-space mixer ----
-// conv: y[r, c] = silu(b[c] + sum_k w[c, k] u[r - taps + 1 + k, c]); rows before the pass come from `hist`
-// [taps, ldh], where position p lies in row p % taps.
+// conv: y[r, c] = f(b[c] + sum_k w[c, k] u[r - taps + 1 + k, c]), f = silu or nothing; rows before the pass come from
+// `hist` [taps, ldh], where position p lies in row p % taps.
 struct SsmConvArgs {
     const void* u;      // [rows, ldu] (act), at the first convolved column
     const uint16_t* w;  // [channels, taps]
-    const uint16_t* b;  // [channels]
-    const void* hist;   // (act)
+    const uint16_t* b;  // [channels] or null
+    void* hist;         // (act)
     void* y;            // [rows, ldy] (act)
     const uint32_t* offset;
     uint32_t rows, channels, taps, ldu, ldy, ldh;
+    uint32_t linear, update;   // linear: no silu; update: the history takes the rows of this pass (else the scan does it)
 };
 fk_status plan_ssm_conv(const SsmConvArgs& a, uint32_t act, Launch* out);
 
@@ -208,5 +253,81 @@ struct SsmChunkArgs {
 constexpr uint32_t kSsmChunk = 64;
 bool ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n);
 fk_status plan_ssm_chunk(const SsmChunkArgs& a, Launch* out);
+
+// ---- grouped-query attention ----
+// One launch between the joint input projection and the attention of a pass: RMS norm of the whole query row and of the
+// whole key row (all heads at once), rotation, the new cache rows.  The values are the keys as they were projected.
+// Heads are padded to dim_ld elements; caches are [kv_heads][capacity][dim_ld].
+struct QkStoreArgs {
+    const void* u;            // [rows, ldu] (act): keys at column k0, queries at column q0
+    const uint16_t* wq;       // [heads * dim_ld] norm weights
+    const uint16_t* wk;       // [kv_heads * dim_ld]
+    const double* freq;       // [rot_dims / 2] radians per position
+    void* q;                  // [rows, heads * dim_ld] (act)
+    void* cache_k;
+    void* cache_v;
+    const uint32_t* offset;
+    uint32_t rows, heads, kv_heads, dim, dim_ld, rot_dims, ldu, k0, q0, capacity;
+    float eps, mag;           // mag: factor of cos and sin
+};
+fk_status plan_qk_store(const QkStoreArgs& a, uint32_t act, Launch* out);
+
+// Causal attention of the rows of a pass, any head width, one workgroup per (head, row).
+struct GqaRowsArgs {
+    const void* q;            // [rows, heads * dim_ld] (act)
+    const void* cache_k;
+    const void* cache_v;
+    const uint32_t* offset;
+    void* out;                // [rows, ldo] (act)
+    uint32_t rows, heads, kv_heads, dim_ld, capacity, ldo;
+    float scale;
+};
+constexpr uint32_t kMaxGqaDim = 512;
+fk_status plan_gqa_rows(const GqaRowsArgs& a, uint32_t act, Launch* out);
+
+// ---- gated delta rule with one decay per key channel ----
+// Head h of `heads` has its own state, values and decays and shares queries and keys of head h / (heads / kv_heads).
+// Head widths are padded to whole 32s (dim_ld, vdim_ld); the padding holds zeros.
+//
+// prep: unit vectors of the convolved queries (times dim^-1/2) and keys, log2 of the decays, step sizes.
+struct DeltaPrepArgs {
+    const void* xc;           // [rows, ldx] (act) after the convolution: q | k | v
+    const uint16_t* dt_bias;  // [heads * dim_ld]
+    const uint16_t* a_log;    // [heads]
+    float* decay;             // [rows, heads * dim_ld]: the projection before bias and softplus; becomes log2 of the decay
+    float* beta;              // [rows, ldb]: before the sigmoid; becomes the step size
+    float* qk;                // [rows, 2 * kv_heads * dim_ld]
+    uint32_t rows, heads, kv_heads, dim, dim_ld, ldx, ldb;
+};
+fk_status plan_delta_prep(const DeltaPrepArgs& a, uint32_t act, Launch* out);
+
+// The recurrence over the rows of a pass, row after row.
+struct DeltaScanArgs {
+    const float* qk;
+    const float* decay;
+    const float* beta;
+    const void* v;            // [rows, ldx] (act), at the first value column
+    float* state;             // [heads][vdim_ld][state_ld]
+    float* o;                 // [rows, heads * vdim_ld]
+    uint32_t rows, heads, kv_heads, dim_ld, vdim_ld, state_ld, ldx, ldb;
+};
+fk_status plan_delta_scan(const DeltaScanArgs& a, uint32_t act, Launch* out);
+
+// ---- real-gated linear recurrent unit ----
+// S <- a S + sqrt(1 - a^2) i u, log a = -8 r softplus(lam), r and i sigmoids of block-diagonal products; the output is
+// S times the gate branch, in its place.  `width` counts padded channels.
+struct LruScanArgs {
+    const void* u;            // [rows, ldx] (act) after the convolution
+    const float* gates;       // [rows, 2 * width]: per block of `block` channels its r, then its i, before bias and sigmoid
+    const uint16_t* rb;       // [width]
+    const uint16_t* ib;
+    const uint16_t* lam;
+    float* state;             // [width]
+    void* y;                  // [rows, ldy] (act): the gate branch in, the output out
+    float* carry;             // [chunks][2][width]: product of decays and end of every chunk
+    uint32_t rows, width, block, ldx, ldy;
+};
+constexpr uint32_t kLruChunk = 32;
+fk_status plan_lru_scan(const LruScanArgs& a, uint32_t act, Launch* out);
 
 }  // namespace fk

@@ -54,10 +54,11 @@ struct SdpaPrefillArgs {
     const uint16_t* q;    // [rows, n_heads, D]
     const uint16_t* k;    // [n_kv, capacity, D]
     const uint16_t* v;
-    uint16_t* out;        // [rows, n_heads, D]
+    uint16_t* out;        // rows of ldo elements: [n_heads, D]
     uint32_t rows, kv_len, n_heads, heads_per_kv, capacity, row_tiles;
     float scale2;         // softmax scale times log2(e)
     const uint32_t* kv_len_ptr;  // optional: the count on the device (a replayed graph), instead of kv_len
+    uint32_t ldo;                // elements between output rows
 };
 
 // Positions in the cache including the group's rows.  A device value is clamped to what the
@@ -304,7 +305,7 @@ __global__ __launch_bounds__(kPrefillBlock) void sdpa_prefill_kernel(const SdpaP
             o[0] += lo.x; o[1] += lo.y; o[2] += lo.z; o[3] += lo.w;
             o[4] += hi.x; o[5] += hi.y; o[6] += hi.z; o[7] += hi.w;
         }
-        *reinterpret_cast<uint4*>(a.out + ((size_t)(r0 + row) * a.n_heads + head) * D + piece * 8u) =
+        *reinterpret_cast<uint4*>(a.out + (size_t)(r0 + row) * a.ldo + head * D + piece * 8u) =
             make_uint4(pack_bf16(o[0], o[1]), pack_bf16(o[2], o[3]), pack_bf16(o[4], o[5]), pack_bf16(o[6], o[7]));
     }
 }
@@ -520,14 +521,14 @@ __global__ __launch_bounds__(kPrefillBlock) void sdpa_prefill_tile_kernel(const 
         if (row >= live) continue;
         const float4 lo = *reinterpret_cast<const float4*>(ob + row * OS + pc * 8u);
         const float4 hi = *reinterpret_cast<const float4*>(ob + row * OS + pc * 8u + 4u);
-        *reinterpret_cast<uint4*>(a.out + ((size_t)(r0 + row) * a.n_heads + head) * D + pc * 8u) =
+        *reinterpret_cast<uint4*>(a.out + (size_t)(r0 + row) * a.ldo + head * D + pc * 8u) =
             make_uint4(pack_bf16(lo.x, lo.y), pack_bf16(lo.z, lo.w), pack_bf16(hi.x, hi.y), pack_bf16(hi.z, hi.w));
     }
 }
 
 fk_status plan_sdpa_prefill(const uint16_t* q, const uint16_t* cache_k, const uint16_t* cache_v, uint16_t* out,
                             uint32_t rows, uint32_t kv_len, uint32_t n_heads, uint32_t n_kv, uint32_t head_dim,
-                            uint32_t capacity, float scale, Launch* l, const uint32_t* kv_len_ptr) {
+                            uint32_t capacity, float scale, Launch* l, const uint32_t* kv_len_ptr, uint32_t ldo) {
     const DeviceFacts* dev;
     FK_TRY(device_facts(&dev));
     if (!q || !cache_k || !cache_v || !out) return set_error(FK_ERR_INVALID, "sdpa_prefill: null pointer");
@@ -542,6 +543,8 @@ fk_status plan_sdpa_prefill(const uint16_t* q, const uint16_t* cache_k, const ui
     memset(&a, 0, sizeof(a));
     a.q = q; a.k = cache_k; a.v = cache_v; a.out = out;
     a.kv_len_ptr = kv_len_ptr;
+    a.ldo = ldo ? ldo : n_heads * head_dim;
+    if (a.ldo < n_heads * head_dim || a.ldo % 8) return set_error(FK_ERR_INVALID, "sdpa_prefill: output rows below the heads' width or not 16-byte aligned");
     if (rows > capacity) return set_error(FK_ERR_INVALID, "sdpa_prefill: more rows than the cache holds");
     a.rows = rows; a.kv_len = kv_len; a.n_heads = n_heads; a.heads_per_kv = n_heads / n_kv; a.capacity = capacity;
     a.scale2 = scale * 1.4426950408889634f;

@@ -25,7 +25,7 @@ __global__ __launch_bounds__(256) void ssm_conv_rows_kernel(const SsmConvArgs a)
 #pragma unroll
         for (uint32_t e = 0; e < 4; ++e) w[k][e] = k + a.taps >= kConvTaps ? bf16_bits_to_f32(a.w[(size_t)(c + e) * a.taps + k + a.taps - kConvTaps]) : 0.f;
 #pragma unroll
-    for (uint32_t e = 0; e < 4; ++e) b[e] = bf16_bits_to_f32(a.b[c + e]);
+    for (uint32_t e = 0; e < 4; ++e) b[e] = a.b ? bf16_bits_to_f32(a.b[c + e]) : 0.f;
     auto input = [&](int32_t r) __attribute__((always_inline)) {   // row r of the pass; before it: the history, zeros before the start
         if (r >= 0) return act_load4(u + (size_t)r * a.ldu);
         const int32_t p = (int32_t)pos0 + r;
@@ -35,6 +35,10 @@ __global__ __launch_bounds__(256) void ssm_conv_rows_kernel(const SsmConvArgs a)
     auto put = [&](float (&d)[4], float4 v) __attribute__((always_inline)) { d[0] = v.x; d[1] = v.y; d[2] = v.z; d[3] = v.w; };
 #pragma unroll
     for (uint32_t k = 0; k + 1u < kConvTaps; ++k) put(x[k + 1], input((int32_t)(r0 + k) - (int32_t)(kConvTaps - 1u)));
+    if (a.update && r0 == 0u) {   // these threads alone read the history of their columns, and have done so
+        for (uint32_t t = a.rows - (a.taps - 1u); t < a.rows; ++t)
+            act_store4(reinterpret_cast<T*>(a.hist) + (size_t)((pos0 + t) % a.taps) * a.ldh + c, act_load4(u + (size_t)t * a.ldu));
+    }
     T* y = reinterpret_cast<T*>(a.y) + c;
 #pragma unroll
     for (uint32_t i = 0; i < kConvRows; ++i) {
@@ -51,7 +55,7 @@ __global__ __launch_bounds__(256) void ssm_conv_rows_kernel(const SsmConvArgs a)
             s[e] = b[e];
 #pragma unroll
             for (uint32_t k = 0; k < kConvTaps; ++k) s[e] = fmaf(w[k][e], x[k][e], s[e]);
-            s[e] = silu(s[e]);
+            if (!a.linear) s[e] = silu(s[e]);
         }
         act_store4(y + (size_t)r * a.ldy, make_float4(s[0], s[1], s[2], s[3]));
     }
@@ -64,14 +68,26 @@ __global__ __launch_bounds__(256) void ssm_conv_kernel(const SsmConvArgs a) {
     const uint32_t pos = *a.offset + r;
     const T* u = reinterpret_cast<const T*>(a.u);
     const T* hist = reinterpret_cast<const T*>(a.hist);
-    float s = bf16_bits_to_f32(a.b[c]);
+    float s = a.b ? bf16_bits_to_f32(a.b[c]) : 0.f;
     for (uint32_t k = 0; k < a.taps; ++k) {
         const uint32_t back = a.taps - 1u - k;
         if (back > pos) continue;   // before the first token: zero
         const float v = back <= r ? act_load(u + (size_t)(r - back) * a.ldu + c) : act_load(hist + (size_t)((pos - back) % a.taps) * a.ldh + c);
         s = fmaf(bf16_bits_to_f32(a.w[(size_t)c * a.taps + k]), v, s);
     }
-    act_store(reinterpret_cast<T*>(a.y) + (size_t)r * a.ldy + c, silu(s));
+    act_store(reinterpret_cast<T*>(a.y) + (size_t)r * a.ldy + c, a.linear ? s : silu(s));
+    // a single row takes the place of the one that has left the convolution, which nobody reads
+    if (a.update && a.rows == 1u) reinterpret_cast<T*>(a.hist)[(size_t)(pos % a.taps) * a.ldh + c] = u[c];
+}
+
+// The history after a pass of several rows: its last taps - 1 rows.
+template <typename T>
+__global__ __launch_bounds__(256) void ssm_conv_history_kernel(const SsmConvArgs a) {
+    const uint32_t c = blockIdx.x * 256u + threadIdx.x, pos = *a.offset;
+    if (c >= a.channels) return;
+    const uint32_t keep = a.rows < a.taps - 1u ? a.rows : a.taps - 1u;
+    for (uint32_t t = a.rows - keep; t < a.rows; ++t)
+        reinterpret_cast<T*>(a.hist)[(size_t)((pos + t) % a.taps) * a.ldh + c] = reinterpret_cast<const T*>(a.u)[(size_t)t * a.ldu + c];
 }
 
 // Four adjacent values of a row of `n`, zeros past its end.
@@ -158,7 +174,7 @@ const void* scan_func(uint32_t ni) {
 
 fk_status plan_ssm_conv(const SsmConvArgs& a, uint32_t act, Launch* out) {
     if (act != 16 && act != 32) return set_error(FK_ERR_INVALID, "ssm conv: act must be 16 or 32");
-    if (!a.u || !a.w || !a.b || !a.hist || !a.y || !a.offset || !a.rows || !a.channels || !a.taps) return set_error(FK_ERR_INVALID, "ssm conv: bad arguments");
+    if (!a.u || !a.w || !a.hist || !a.y || !a.offset || !a.rows || !a.channels || !a.taps) return set_error(FK_ERR_INVALID, "ssm conv: bad arguments");
     if (a.rows > 65535) return set_error(FK_ERR_UNSUPPORTED, "ssm conv: at most 65535 rows");
     const uintptr_t align = act == 16 ? 7 : 15;   // four elements per access
     if (a.rows >= kConvRows && a.taps <= kConvTaps && a.channels % 4 == 0 && a.ldu % 4 == 0 && a.ldy % 4 == 0 && a.ldh % 4 == 0 &&
@@ -168,6 +184,14 @@ fk_status plan_ssm_conv(const SsmConvArgs& a, uint32_t act, Launch* out) {
     } else {
         out->func = act == 16 ? (const void*)&ssm_conv_kernel<uint16_t> : (const void*)&ssm_conv_kernel<float>;
         out->grid = dim3((a.channels + 255u) / 256u, a.rows);
+        if (a.update && a.rows > 1u && a.taps > 1u) {
+            Launch h;
+            h.func = act == 16 ? (const void*)&ssm_conv_history_kernel<uint16_t> : (const void*)&ssm_conv_history_kernel<float>;
+            h.grid = dim3((a.channels + 255u) / 256u, 1, 1);
+            h.block = dim3(256, 1, 1);
+            h.set_args(a);
+            out->then.push_back(h);
+        }
     }
     out->block = dim3(256, 1, 1);
     out->shmem = 0;

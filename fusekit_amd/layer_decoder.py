@@ -1,14 +1,16 @@
 """Layer-list decoder on the MI355X backend: a model whose layers are described one by one.
 
-Every layer has a mixer (latent attention over a sliding window, or a Mamba-2 state-space mixer) and optionally a
-mixture-of-experts feed-forward.  The two run side by side: each reads its own norm of the layer's input, and their
-outputs join a 32-bit residual stream together.
-A range of layers may run several times in a row with the same weights (`loop`), each pass with its own cache or state
-and a learned vector added before it.  The design that uses it today is Pusavik.
+Every layer has a mixer and optionally a feed-forward.  The two run side by side and their outputs join a 32-bit residual
+stream together.  Either each reads its own norm of the layer's input (latent attention over a sliding window, Mamba-2
+state-space mixers, mixtures of experts: this module; the design is Pusavik), or both read one norm (joint layers with
+causal attention, gated delta rules, gated linear recurrences and dense feed-forwards: joint_layers.py; the design is
+Fumotar).
+A range of layers may run several times in a row with the same weights (`loop`), each pass with its own cache or state.
+Ahead of a pass a learned vector is added, or the stream is projected together with the embedding output (`join`).
 
 What a sequence leaves behind is held by `LayerState`: per layer RUN (a looped layer has several) a ring of latent rows
-just long enough for the window, or a recurrent state and the convolution's last inputs.  Its size does not grow with
-the sequence.
+just long enough for the window, a key / value cache of `capacity` positions, or a recurrent state and the convolution's
+last inputs.
 
 Two task lists share the kernels' families: the decode list (one token, captured as one hipGraph and replayed) and the
 rows list (a portion of a prompt of any length).  `act` 32 runs everything in fp32 through the same families.
@@ -22,15 +24,11 @@ from typing import Callable, Dict, List, Optional, Sequence, Tuple
 
 import numpy as np
 
-from . import native
+from . import joint_layers, native
 from .decoder import _synth
+from .joint_layers import JOINT, CausalAttention, ChannelDelta, DenseMlp, JointTasks, RgLru, RotaryScaling, pad
 from .native import DeviceBuffer, DeviceWeight
 from .runtime import FK_CHUNK, Dispatch, Dispatcher, arg, make_uniforms
-
-
-def pad(n: int, to: int = 64) -> int:
-    """Padded length of a row (kernels walk rows in whole blocks; the padding holds zeros)."""
-    return -(-n // to) * to
 
 
 # ---------------------------------------------------------------- configuration
@@ -120,7 +118,27 @@ class Experts:
 @dataclass
 class Layer:
     mixer: object
-    mlp: Optional[Experts] = None
+    mlp: object = None           # Experts, DenseMlp (joint layers) or None
+
+    @property
+    def joint(self) -> bool:
+        return self.mixer.kind in JOINT
+
+    @property
+    def experts(self) -> Optional[Experts]:
+        return self.mlp if isinstance(self.mlp, Experts) else None
+
+    def __post_init__(self):
+        if self.mlp is not None and isinstance(self.mlp, DenseMlp) != self.joint:
+            raise ValueError("dense feed-forwards go with joint mixers, experts with the others")
+
+
+@dataclass
+class PairTable:
+    """A second embedding table, its rows chosen by a hash of a token and the one before it (row `buckets`: no token before)."""
+    buckets: int
+    mul_prev: int
+    mul_cur: int
 
 
 @dataclass
@@ -133,6 +151,12 @@ class LayerConfig:
     loop_start: int = 0
     loop_stop: int = 0
     loop_times: int = 1
+    design: str = "Pusavik"
+    layer_norm: bool = False     # norms: x - mean over the standard deviation, with a bias; else RMS norms
+    tied: bool = False           # the embedding table is the head
+    pairs: Optional[PairTable] = None
+    join: bool = False           # ahead of a loop pass: x <- W [x; embedding output]; else a learned vector is added
+    capacity: int = 4096         # positions of a key / value cache
     act: int = 16                # 16: bf16 matrices and activations, 32-bit residual, norms, router, softmax and state; 32: all fp32
     rows_per_pass: int = 2048    # most tokens of one rows pass
     artifact_type = "layer-list-decoder"
@@ -154,6 +178,11 @@ class LayerConfig:
     @property
     def head_dim(self) -> int:
         return max((l.mixer.vdim for l in self.layers), default=0)
+
+    @property
+    def max_positions(self) -> Optional[int]:
+        """Longest sequence the state holds, None without a limit."""
+        return self.capacity if any(l.mixer.kind == "attention" for l in self.layers) else None
 
     @property
     def looped(self) -> bool:
@@ -180,16 +209,41 @@ def small_config(width: int = 256, vocab: int = 1000, heads: int = 4, ff: int = 
                        loop_start=1, loop_stop=3, loop_times=2, **more)
 
 
+def small_joint_config(width: int = 256, vocab: int = 1000, heads: int = 4, ff: int = 96, **more) -> LayerConfig:
+    """A four-layer model of the three joint mixers with a loop, for examples and tests."""
+    att = CausalAttention(heads=heads, kv_heads=max(1, heads // 2), dim=40, scale=40 ** -0.5, rot_base=5000.0, rot_dims=24,
+                          rot_scaling=RotaryScaling(factor=3.0, original=512, fast=16.0, slow=1.5))
+    dlt = ChannelDelta(heads=heads, kv_heads=max(1, heads // 2), dim=24, vdim=40, conv=3, decay_rank=20, gate_rank=28)
+    lru = RgLru(width=3 * 40, blocks=3, conv=4)
+    mlp = DenseMlp(ff)
+    return LayerConfig(width=width, vocab=vocab, layers=[Layer(lru, mlp), Layer(att, mlp), Layer(dlt), Layer(att, mlp)], loop_start=1, loop_stop=3,
+                       loop_times=2, design="Fumotar", layer_norm=True, tied=True, pairs=PairTable(buckets=211, mul_prev=13, mul_cur=7), join=True, **more)
+
+
 def tensor_shapes(cfg: LayerConfig) -> Dict[str, Tuple[int, ...]]:
     """Names and shapes of a checkpoint's tensors."""
     D = cfg.width
     s: Dict[str, Tuple[int, ...]] = {"embed": (cfg.vocab, D)}
-    if cfg.looped:
+    if cfg.pairs:
+        s["bigram"] = (cfg.pairs.buckets + 1, D)
+    if cfg.looped and cfg.join:
+        s["loop.in"] = (D, 2 * D)
+    elif cfg.looped:
         s["loop.step"] = (cfg.loop_times, D)
+
+    def norm(name: str) -> None:
+        s[name] = (D,)
+        if cfg.layer_norm:
+            s[name + ".b"] = (D,)
+
     for i, l in enumerate(cfg.layers):
-        p, m, f = f"l{i}.", l.mixer, l.mlp
-        s[p + "norm1"] = (D,)
-        if m.kind == "latent_attention":
+        p, m, f = f"l{i}.", l.mixer, l.experts
+        norm(p + "norm1")
+        if l.joint:
+            s.update(joint_layers.mixer_shapes(m, p + "mix.", D))
+            if l.mlp:
+                s.update(joint_layers.mlp_shapes(l.mlp, p + "mlp.", D))
+        elif m.kind == "latent_attention":
             s[p + "mix.dq"], s[p + "mix.dq.norm"] = (m.q_rank, D), (m.q_rank,)
             s[p + "mix.uq"] = (m.heads * (m.dim + m.rot_dim), m.q_rank)
             s[p + "mix.dkv"], s[p + "mix.dkv.norm"] = (m.kv_rank + m.rot_dim, D), (m.kv_rank,)
@@ -206,7 +260,9 @@ def tensor_shapes(cfg: LayerConfig) -> Dict[str, Tuple[int, ...]]:
             for e in range(f.experts):
                 s[p + f"mlp.e{e}.gate"], s[p + f"mlp.e{e}.up"], s[p + f"mlp.e{e}.down"] = (f.ff, D), (f.ff, D), (D, f.ff)
             s[p + "mlp.router"], s[p + "mlp.correction"] = (f.outputs, D), (f.outputs,)
-    s["final.norm"], s["head"] = (D,), (cfg.vocab, D)
+    norm("final.norm")
+    if not cfg.tied:
+        s["head"] = (cfg.vocab, D)
     return s
 
 
@@ -218,7 +274,9 @@ def random_tensors(cfg: LayerConfig, seed: int = 0, std: float = 0.05) -> Dict[s
     for name, shape in tensor_shapes(cfg).items():
         leaf = name.rsplit(".", 1)[-1]
         v = rng.standard_normal(shape)
-        if leaf in ("norm1", "norm2", "norm"):
+        if leaf == "lam":
+            v = -3.0 + v
+        elif leaf in ("norm1", "norm2", "norm"):
             v = 1.0 + 0.1 * v
         elif leaf == "A_log":
             v = np.log(1.0 + 7.0 * rng.random(shape))
@@ -226,7 +284,7 @@ def random_tensors(cfg: LayerConfig, seed: int = 0, std: float = 0.05) -> Dict[s
             v = -2.0 + 0.5 * v
         elif leaf in ("D", "sink"):
             v = 1.0 + 0.5 * v
-        elif leaf in ("embed", "head"):
+        elif leaf in ("embed", "head", "bigram"):
             v = v * 0.5
         elif leaf == "router":
             v = v * 0.3
@@ -295,16 +353,35 @@ class LayerWeights:
     def from_tensors(cls, cfg: LayerConfig, get: Callable[[str], np.ndarray]) -> "LayerWeights":
         """`get(name)` returns a tensor's bf16 bit patterns in its own shape."""
         self, c = cls(cfg), cfg
-        self._dense("embed", DeviceBuffer.from_numpy(get("embed")), c.vocab, c.width)
-        self._matrix("head", get("head"))
-        self._vector("final.norm", get("final.norm"), True)
-        if c.looped:
+        if c.tied:
+            self._matrix("head", get("embed"))
+            self.mats["embed"] = self.mats["head"]
+        else:
+            self._dense("embed", DeviceBuffer.from_numpy(get("embed")), c.vocab, c.width)
+            self._matrix("head", get("head"))
+        if c.pairs:
+            self._matrix("bigram", get("bigram"))
+
+        def norm(name: str) -> None:
+            self._vector(name, get(name), True)
+            if c.layer_norm:
+                self._vector(name + ".b", get(name + ".b"), True)
+
+        norm("final.norm")
+        if c.looped and c.join:
+            W, D = get("loop.in"), pad(c.width)
+            both = np.zeros((c.width, 2 * D), np.uint16)
+            both[:, :c.width], both[:, D:D + c.width] = W[:, :c.width], W[:, c.width:]
+            self._matrix("loop.in", both)
+        elif c.looped:
             self._vector("loop.step", get("loop.step"), True)
         for i, l in enumerate(c.layers):
-            p, m, f = f"l{i}.", l.mixer, l.mlp
-            self._vector(p + "norm1", get(p + "norm1"), True)
+            p, m, f = f"l{i}.", l.mixer, l.experts
+            norm(p + "norm1")
             q = p + "mix."
-            if m.kind == "latent_attention":
+            if l.joint:
+                joint_layers.load_layer(self, p, l, c.width, get)
+            elif m.kind == "latent_attention":
                 self._matrix(q + "down", np.concatenate([get(q + "dq"), get(q + "dkv")], 0))
                 self._vector(q + "dq.norm", get(q + "dq.norm"), True)
                 self._vector(q + "dkv.norm", get(q + "dkv.norm"), True)
@@ -358,16 +435,31 @@ class LayerWeights:
                 raise ValueError(f"{name}: random_init takes widths that need no padding")
             self._dense(name, fill(n * k * max(experts, 1), 0.0, sd), n, k, experts)
 
-        matrix("embed", c.vocab, c.width, sd=0.5)
-        matrix("head", c.vocab, c.width)
-        self.vecs["final.norm"] = fill(pad(c.width), 1.0, 0.1)
-        if c.looped:
+        matrix("embed", c.vocab, c.width, sd=std if c.tied else 0.5)
+        if c.tied:
+            self.mats["head"] = self.mats["embed"]
+        else:
+            matrix("head", c.vocab, c.width)
+        if c.pairs:
+            matrix("bigram", c.pairs.buckets + 1, c.width, sd=0.5)
+
+        def norm(name: str) -> None:
+            self.vecs[name] = fill(pad(c.width), 1.0, 0.1)
+            if c.layer_norm:
+                self.vecs[name + ".b"] = fill(pad(c.width), 0.0, 0.1)
+
+        norm("final.norm")
+        if c.looped and c.join:
+            matrix("loop.in", c.width, 2 * c.width)
+        elif c.looped:
             self.vecs["loop.step"] = fill(c.loop_times * pad(c.width), 0.0, 0.1)
         for i, l in enumerate(c.layers):
-            p, m, f = f"l{i}.", l.mixer, l.mlp
-            self.vecs[p + "norm1"] = fill(c.width, 1.0, 0.1)
+            p, m, f = f"l{i}.", l.mixer, l.experts
+            norm(p + "norm1")
             q = p + "mix."
-            if m.kind == "latent_attention":
+            if l.joint:
+                joint_layers.random_layer(self, p, l, c.width, fill, matrix)
+            elif m.kind == "latent_attention":
                 if m.dim % 32 or m.rot_dim % 32 or m.vdim % 32:
                     raise ValueError("random_init takes head widths that need no padding")
                 matrix(q + "down", m.low_rows, c.width)
@@ -397,23 +489,29 @@ class LayerWeights:
         return self
 
     def nbytes(self) -> int:
-        return sum(m.nbytes for m in self.mats.values()) + sum(v.nbytes for v in self.vecs.values())
+        mats = {id(m): m for m in self.mats.values()}   # a tied head is one matrix under two names
+        return sum(m.nbytes for m in mats.values()) + sum(v.nbytes for v in self.vecs.values())
 
 
 # ---------------------------------------------------------------- what a sequence leaves behind
 
 class LayerState:
-    """Caches and states of one sequence, one entry per layer run.  Position p of an attention run lies in row
-    p % ring of its ring of latent rows (rows a window can no longer see are overwritten); a state-space run holds its
-    fp32 state and the last convolution inputs (position p in row p % taps)."""
+    """Caches and states of one sequence, one entry per layer run.  Position p of a windowed attention run lies in row
+    p % ring of its ring of latent rows (rows a window can no longer see are overwritten), of a causal one in row p of its
+    key and value caches; a recurrent run holds its fp32 state and the last convolution inputs (position p in row
+    p % taps).  `prev` is the last token, where a table of token pairs needs it."""
 
     def __init__(self, cfg: LayerConfig, rows: int):
         e = cfg.act // 8
         self.entries: List[Dict[str, DeviceBuffer]] = []
         self.rings: List[int] = []
+        self.prev = native.zeros(4)
         for i, _ in cfg.runs():
             m = cfg.layers[i].mixer
-            if m.kind == "latent_attention":
+            if cfg.layers[i].joint:
+                self.rings.append(0)
+                self.entries.append(joint_layers.state_entry(m, cfg.act, cfg.capacity))
+            elif m.kind == "latent_attention":
                 ring = 1 << (m.window + rows - 2).bit_length()
                 self.rings.append(ring)
                 # a product that walks padded rows may read up to one padding block past the last row
@@ -424,8 +522,8 @@ class LayerState:
                                          hist=native.zeros(m.conv * pad(m.channels) * e)))
 
     def reset(self) -> None:
-        """A new sequence: recurrent states start at zero.  Latent rows need no clearing: a window sees only rows that
-        the sequence itself has written."""
+        """A new sequence: recurrent states start at zero.  Cache rows need no clearing: a position sees only rows that the
+        sequence itself has written, and the first one looks at no token before it."""
         for e in self.entries:
             for name in ("state", "hist"):
                 if name in e:
@@ -438,7 +536,7 @@ class LayerState:
 
 # ---------------------------------------------------------------- runtime
 
-class LayerRuntime:
+class LayerRuntime(JointTasks):
     """Scratch arena, sequence state, decode graph and rows passes of one model."""
 
     HEAD_ROWS = 64      # logits rows formed at once for a portion that asks for them
@@ -448,14 +546,14 @@ class LayerRuntime:
         self.cfg, self.w = cfg, weights
         self.d = dispatcher or Dispatcher()
         self.runs = c.runs()
-        tops = [l.mlp.top for l in c.layers if l.mlp]
-        self.R = max(1, min(c.rows_per_pass, 65535 // max(tops, default=1)))
+        tops = [l.experts.top for l in c.layers if l.experts]
+        self.R = max(1, min(c.rows_per_pass, 65535 // max(tops, default=1), c.max_positions or c.rows_per_pass))
         self.position = 0
         self.state = LayerState(c, self.R)
         z = native.zeros
         self.token, self.step_counter, self.offset, self.kv_len, self.hist_counter = (z(4) for _ in range(5))
         self.history = z(4 * hist_capacity)
-        self.row_offset, self.tokens = z(4), z(4 * self.R)
+        self.row_offset, self.row_kv, self.tokens = z(4), z(4), z(4 * self.R)
         self.argmax_ws = z(native.ARGMAX_WORKSPACE_BYTES)
         self.buf: Dict[str, DeviceBuffer] = {}
         self._alloc_rows()
@@ -478,9 +576,13 @@ class LayerRuntime:
         D = pad(c.width)
         for n, b in (("x", 4), ("mix", 4), ("h1", e), ("h2", e)):
             want(n, R * D * b)
+        if c.looped and c.join:
+            want("cat", R * 2 * D * e)
         for l in c.layers:
-            m, f = l.mixer, l.mlp
-            if m.kind == "latent_attention":
+            m, f = l.mixer, l.experts
+            if l.joint:
+                joint_layers.scratch(m, l.mlp, R, c.act, c.capacity, want)
+            elif m.kind == "latent_attention":
                 want("low", R * pad(m.low_rows) * 4)
                 want("cq", R * pad(m.q_rank) * e)
                 want("q", R * pad(m.heads * m.hs) * e)
@@ -554,7 +656,7 @@ class LayerRuntime:
                y32: bool = False, **more) -> None:
         """y = x . W[n0 : n0 + n]^T."""
         n = W.n - n0 if n is None else n
-        t.append(Dispatch(self._name("dense"), [x, arg(W.w, (W.w.nbytes // (2 * W.k) - n0) * W.k * 2, n0 * W.k * 2)] + more.pop("base", []) + [y],
+        t.append(Dispatch(self._name("dense"), [x, arg(W.w, (W.w.nbytes // (2 * W.k) - n0) * W.k * 2, n0 * W.k * 2)] + more.pop("base", []) + [y] + more.pop("tail", []),
                           dict(rows=rows, n=n, k=W.k, ldx=ldx, ldw=W.k, ldy=ldy, y32=int(y32), act=self.cfg.act, **more)))
 
     def _norm_tasks(self, t, run: int, rows: int, first: bool) -> None:
@@ -562,26 +664,39 @@ class LayerRuntime:
         that run `run` (or the head) reads."""
         c, w, b = self.cfg, self.w, self.buf
         D = pad(c.width)
-        p = dict(rows=rows, width=c.width, ld=D, act=c.act, eps=c.eps)
-        a = [arg(b["x"])]
+        shape = dict(rows=rows, width=c.width, ld=D, act=c.act, eps=c.eps)
+        p, a = dict(shape), [arg(b["x"])]
+
+        def norm(name: str) -> None:
+            a.append(arg(w.vecs[name]))
+            if c.layer_norm:
+                a.append(arg(w.vecs[name + ".b"]))
+                p["layer_norm"] = 1
+            a.append(arg(b["h1"]))
+            p["has_h1"] = 1
+
         if not first:
             a.append(arg(b["mix"]))
             p["has_mix"] = 1
-            f = c.layers[self.runs[run - 1][0]].mlp
+            f = c.layers[self.runs[run - 1][0]].experts
             if f:
                 a += [arg(b["eo"]), arg(b["rwt"]), arg(b["ridx"]), arg(b["h2"])]
                 p.update(top=f.top, experts=f.experts)
         if run == len(self.runs):
-            a += [arg(w.vecs["final.norm"]), arg(b["h1"])]
-            p["has_h1"] = 1
+            norm("final.norm")
         else:
             i, step = self.runs[run]
-            if step is not None:
+            if step is not None and c.join:   # the stream beside the embedding output, their product is the new stream
+                a.append(arg(b["cat"]))
+                p["ldcopy"] = 2 * D
+                t.append(Dispatch(self._name("residual_norm"), list(a), dict(p)))
+                self._dense(t, arg(b["cat"]), w.mats["loop.in"], arg(b["x"]), rows, 2 * D, D, y32=True)
+                a[:], p = [arg(b["x"])], dict(shape)
+            elif step is not None:
                 a.append(arg(w.vecs["loop.step"], D * 2, step * D * 2))
                 p["has_step"] = 1
-            a += [arg(w.vecs[f"l{i}.norm1"]), arg(b["h1"])]
-            p["has_h1"] = 1
-            if c.layers[i].mlp:
+            norm(f"l{i}.norm1")
+            if c.layers[i].experts:
                 a += [arg(w.vecs[f"l{i}.norm2"]), arg(b["h2"])]
                 p["has_h2"] = 1
         t.append(Dispatch(self._name("residual_norm"), a, p))
@@ -641,7 +756,7 @@ class LayerRuntime:
     def _fused(self) -> bool:
         """Whether every layer has the fused decode launches."""
         c = self.cfg
-        if c.act != 16 or not c.fuse or not c.tiled or pad(c.width) > 30720:
+        if c.act != 16 or not c.fuse or not c.tiled or pad(c.width) > 30720 or any(l.joint for l in c.layers):
             return False
         for l in c.layers:
             m, f = l.mixer, l.mlp
@@ -783,19 +898,36 @@ class LayerRuntime:
         t.append(Dispatch(self._name("experts"), [arg(b["eh"]), arg(w.mats[p + "down"].w), arg(b["ridx"])] + groups + [arg(b["eo"])],
                           dict(q, n=c.width, k=F, ldx=F, ldw=F, ldy=D, x_div=1)))
 
-    def _body_tasks(self, t, tokens, off, rows: int) -> None:
+    def _embed_task(self, tokens, off, rows: int) -> Dispatch:
+        """Embedding rows; with a join their copies beside the place of the stream."""
+        c, b, W, D = self.cfg, self.buf, self.w.mats["embed"], pad(self.cfg.width)
+        if not c.pairs and not c.tied and not (c.looped and c.join):
+            return Dispatch(self._name("embed_lookup_decode"), [tokens, arg(W.w), arg(b["x"])],
+                            dict(bits=16, hidden=c.width, vocab=c.vocab, output_scale=c.embed_scale, rows=rows, out_bits=32, x_row_stride=D))
+        a, p = [tokens, arg(W.w)], dict(rows=rows, width=c.width, vocab=c.vocab, ldw=W.k, ld=D, scale=c.embed_scale, act=c.act)
+        if c.pairs:
+            n = c.pairs.buckets
+            a += [arg(self.w.mats["bigram"].w), arg(self.state.prev), off]
+            p.update(buckets=n, mul_prev=c.pairs.mul_prev % n, mul_cur=c.pairs.mul_cur % n)
+        a.append(arg(b["x"]))
+        if c.looped and c.join:
+            a.append(arg(b["cat"], None, D * (c.act // 8)))
+            p["ldcopy"] = 2 * D
+        return Dispatch(self._name("embed_rows"), a, p)
+
+    def _body_tasks(self, t, tokens, off, kv_len, rows: int) -> None:
         """Embedding to the final norm of `rows` tokens; h1 holds the head's input rows."""
         c, b = self.cfg, self.buf
-        t.append(Dispatch(self._name("embed_lookup_decode"), [tokens, arg(self.w.mats["embed"].w), arg(b["x"])],
-                          dict(bits=16, hidden=c.width, vocab=c.vocab, output_scale=c.embed_scale, rows=rows, out_bits=32,
-                               x_row_stride=pad(c.width))))
+        t.append(self._embed_task(tokens, off, rows))
         self._norm_tasks(t, 0, rows, True)
         for run, (i, _) in enumerate(self.runs):
-            if c.layers[i].mixer.kind == "latent_attention":
+            if c.layers[i].joint:
+                self._joint_tasks(t, run, rows, off, kv_len)
+            elif c.layers[i].mixer.kind == "latent_attention":
                 self._latent_tasks(t, run, rows, off)
             else:
                 self._ssm_tasks(t, run, rows, off)
-            if c.layers[i].mlp:
+            if c.layers[i].experts:
                 self._expert_tasks(t, run, rows)
             self._norm_tasks(t, run + 1, rows, False)
 
@@ -812,16 +944,16 @@ class LayerRuntime:
         if self.fused:
             self._fused_tasks(t)
         else:
-            self._body_tasks(t, arg(self.token), arg(self.offset), 1)
+            self._body_tasks(t, arg(self.token), arg(self.offset), arg(self.kv_len), 1)
             self._dense(t, arg(self.buf["h1"]), self.w.mats["head"], arg(self.logits), 1, pad(c.width), pad(c.vocab), y32=True)
         t.append(self._argmax_task())
         return t
 
     def rows_tasks(self, rows: int) -> List[Dispatch]:
-        """The task list of a portion of `rows` tokens at positions *row_offset .. (tokens and row_offset are device words)."""
+        """The task list of a portion of `rows` tokens at positions *row_offset .. *row_kv - 1 (device words, as are the tokens)."""
         self._fid = 0
         t: List[Dispatch] = []
-        self._body_tasks(t, arg(self.tokens, rows * 4), arg(self.row_offset), rows)
+        self._body_tasks(t, arg(self.tokens, rows * 4), arg(self.row_offset), arg(self.row_kv), rows)
         return t
 
     # -- running
@@ -835,6 +967,7 @@ class LayerRuntime:
         m = len(tokens)
         self.tokens.upload(tokens)
         self.row_offset.upload(np.array([self.position], np.uint32))
+        self.row_kv.upload(np.array([self.position + m], np.uint32))
         if m == self.R:                      # whole passes are replayed; odd portions are launched as they come
             if self._full_pass is None:
                 self._full_pass = self.d.build_decode_graph(self.rows_tasks(m), False)
@@ -868,7 +1001,13 @@ class LayerRuntime:
         t = np.asarray(tokens, np.int64)
         if t.ndim != 1 or t.size == 0 or t.min() < 0 or t.max() >= self.cfg.vocab:
             raise ValueError("token ids must lie in 0 .. vocab - 1, at least one")
+        self._check_room(t.size)
         return t.astype(np.uint32)
+
+    def _check_room(self, n: int) -> None:
+        limit = self.cfg.max_positions
+        if limit is not None and self.position + n > limit:
+            raise ValueError(f"the sequence would exceed the cache's {limit} positions")
 
     def step(self, tokens: Sequence[int], want: Sequence[int] = ()) -> np.ndarray:
         """Runs the sequence's next tokens from the state earlier calls left; logits [len(want), vocab] at the wanted
@@ -913,6 +1052,7 @@ class LayerRuntime:
         gpu_s, steps = 0.0, 0
         while len(out) < max_tokens:
             n = min(FK_CHUNK, max_tokens - len(out), self.uniforms.hist_capacity)
+            self._check_room(n)
             toks, sec = self.d.decode_chunk(self.graph, self.uniforms, self.position, out[-1], n)
             self.position += n
             out += toks
@@ -925,8 +1065,11 @@ class LayerRuntime:
         act = "float32" if self.cfg.act == 32 else "bfloat16"
         out = {n: (getattr(self, n), "uint32", True) for n in ("token", "step_counter", "offset", "kv_len", "hist_counter", "history", "argmax_ws")}
         out["logits"] = (self.logits, "float32", True)
+        words = ("ridx", "perm", "tiles", "tile_count", "counters")
+        floats = ("x", "x2", "mix", "low", "dt", "rl", "rwt", "rot", "part", "chunks", "decay", "beta", "decays", "qk", "o", "gates", "carry")
         for n, b in self.buf.items():
-            out[n] = (b, "uint32" if n in ("ridx", "perm", "tiles", "tile_count") else "float32" if n in ("x", "mix", "low", "dt", "rl", "rwt", "rot", "part", "chunks", "decay") else act, True)
+            out[n] = (b, "uint32" if n in words else "float32" if n in floats else act, True)
+        out["state.prev"] = (self.state.prev, "uint32", True)
         for r, e in enumerate(self.state.entries):
             for n, b in e.items():
                 out[f"state.{n}.{r}"] = (b, "float32" if n == "state" else act, True)

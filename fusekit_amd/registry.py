@@ -24,7 +24,7 @@ class Family:
 
 def _load_layer(model_dir, capacity, act):
     from .checkpoint import load_layer_checkpoint
-    return load_layer_checkpoint(model_dir, act)
+    return load_layer_checkpoint(model_dir, act, capacity)
 
 
 def _layer_runtime(cfg, w):
@@ -53,7 +53,7 @@ def _dense_runtime(cfg, w):
 
 
 FAMILIES = [
-    Family("layer-list", lambda c: c.get("architecture") == "Pusavik", _load_layer, _layer_runtime, acts=(16, 32)),
+    Family("layer-list", lambda c: c.get("architecture") in ("Pusavik", "Fumotar"), _load_layer, _layer_runtime, acts=(16, 32)),
     Family("moe", lambda c: c.get("model_type", "").startswith("deepseek"), _load_moe, _moe_runtime),
     Family("dense", lambda c: "hidden_size" in c.get("text_config", c), _load_dense, _dense_runtime, kv_bits=True),
 ]
