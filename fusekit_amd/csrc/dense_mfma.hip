@@ -13,8 +13,7 @@
 //
 // Expert products take the same tile: the tile table of fusekit_route_group names the expert and the routes, rows are
 // gathered through the route list, and a gate / up pair is one launch (NB = 2) whose epilogue is silu(gate) * up.
-#include "act_device.hpp"
-#include "layered.hpp"
+#include "column_device.hpp"
 
 namespace fk {
 
@@ -43,17 +42,6 @@ struct TileArgs {
     uint64_t xb, wstride, yb;   // batch strides; wstride: per batch or per expert
     ColumnOut out;
 };
-
-// What becomes of one column's sum before it is stored.
-__device__ __forceinline__ float column_value(const ColumnOut& o, uint32_t n, float v) {
-    if (o.bias) v += bf16_bits_to_f32(o.bias[n]);
-    const uint32_t fn = n >= o.begin && n < o.end ? o.fn : n >= o.begin2 ? o.fn2 : (uint32_t)kFnNone;
-    if (fn == kFnRelu2) {
-        v = fmaxf(v, 0.f);
-        return v * v;
-    }
-    return fn == kFnGelu ? gelu_tanh(v) : v;
-}
 
 __device__ __forceinline__ dm_u32x4_t lds_piece(const uint16_t* tile, uint32_t row, uint32_t piece) {
     return *reinterpret_cast<const dm_u32x4_t*>(tile + row * kBK + ((piece ^ (row & 7u)) << 3));

@@ -484,14 +484,19 @@ fk_status plan_latent_split_d(const Dispatch& d, Launch* l, SlotRW* rw) {
 }
 
 // Jobs side by side; every part is announced by a parameter, slots in this order:
-//   products i = 0, 1 (g<i>): g<i>_mode 0: x | 1: x, [step: g<i>_step], norm weights, [kept row: g<i>_keep] | 2: x, z, norm
-//     weights | 3: partial rows, sinks; then w, [y: n_act > 0], [y32: n_act < n]
-//     {g<i>_n, _k, _ldw, _width, _n_act, _rows_per_head, _x_head, _y_head, _groups, _splits, _heads, _eps}
+//   products i = 0, 1 (g<i>): g<i>_mode 0: x | 1: x, [step: g<i>_step], norm weights, [norm bias: g<i>_layer_norm], [kept row:
+//     g<i>_keep] | 2: x, z, norm weights | 3: partial rows, sinks | 4: x, second row; then w, [bias: g<i>_has_bias], [y:
+//     n_act > 0], [y32: n_act < n]
+//     {g<i>_n, _k, _ldw, _width, _n_act, _rows_per_head, _x_head, _y_head, _groups, _splits, _heads, _eps, _fn, _fn_begin,
+//      _fn_end, _fn2, _fn2_begin}
 //   pair: x, gate, up, index, y                     {pair_n, _k, _ldw, _ldy, _top, _experts}
 //   route: logits, correction, index, weight        {route_outputs, _top}
 //   store: kv, norm, freq, offset, cache, tab            {store_rank, _rank_ld, _ldc, _ring, _rot, _rot_dims, _eps}
 //   scan: u, dt, conv, conv bias, dt_bias, a_log, d, offset, state, hist, y
 //                                                   {scan_heads, _groups, _n, _p, _state_ld, _ldh, _taps}
+//   delta: u, a1, beta, conv, a2, dt_bias, a_log, offset, state, hist, o
+//                                                   {delta_heads, _kv_heads, _dim, _dim_ld, _vdim_ld, _state_ld, _rank_ld, _ldh, _taps}
+//   lru: u, conv, conv bias, gates, r bias, i bias, lam, offset, state, hist, y    {lru_width, _block, _ldh, _taps}
 fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     LayerJobsArgs a;
     memset(&a, 0, sizeof(a));
@@ -504,7 +509,7 @@ fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
         j.mode = u("mode"); j.n = u("n"); j.k = u("k"); j.ldw = u("ldw", j.k); j.width = u("width", j.k); j.n_act = u("n_act");
         j.rows_per_head = u("rows_per_head"); j.x_head = u("x_head"); j.y_head = u("y_head", j.rows_per_head);
         j.groups = u("groups", 1); j.splits = u("splits"); j.heads = u("heads"); j.eps = (float)d.param((g + "eps").c_str(), 1e-6);
-        if (!j.n || !j.k || !j.width || j.mode > kRowCombine) return set_error(FK_ERR_INVALID, d.kernel + ": product parameters missing");
+        if (!j.n || !j.k || !j.width || j.mode > kRowJoin) return set_error(FK_ERR_INVALID, d.kernel + ": product parameters missing");
         const uint64_t nh = j.rows_per_head ? j.n / j.rows_per_head : 1;
         if (nh == 0) return set_error(FK_ERR_INVALID, d.kernel + ": rows per head");
         if (j.mode == kRowPlain) j.x = s.in(((nh - 1) * j.x_head + j.k) * 2);
@@ -513,11 +518,15 @@ fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
             j.vec = ((uintptr_t)j.x & 15u) == 0;
             if (u("step")) j.x2 = s.in((uint64_t)j.k * 2);
             j.nw = s.in<uint16_t>((uint64_t)j.k * 2);
+            if (u("layer_norm")) j.nb = s.in<uint16_t>((uint64_t)j.k * 2);
             if (u("keep")) j.keep = s.out<uint16_t>((uint64_t)j.k * 2);
         } else if (j.mode == kRowGated) {
             j.x = s.in((uint64_t)j.width * 2);
             j.x2 = s.in((uint64_t)j.width * 2);
             j.nw = s.in<uint16_t>((uint64_t)j.width * 2);
+        } else if (j.mode == kRowJoin) {
+            j.x = s.in((uint64_t)j.width * 4);
+            j.x2 = s.in((uint64_t)j.k);
         } else {
             j.pl = j.k + 2;
             if (j.heads != nh) return set_error(FK_ERR_INVALID, d.kernel + ": heads of the partial rows");
@@ -525,6 +534,8 @@ fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
             j.nw = s.in<uint16_t>((uint64_t)j.heads * 2);
         }
         j.w = s.in<uint16_t>(((uint64_t)(j.n - 1) * j.ldw + j.k) * 2);
+        j.out.fn = u("fn"); j.out.begin = u("fn_begin"); j.out.end = u("fn_end"); j.out.fn2 = u("fn2"); j.out.begin2 = u("fn2_begin");
+        if (u("has_bias")) j.out.bias = s.in<uint16_t>((uint64_t)j.n * 2);
         const uint64_t outs = (nh - 1) * j.y_head + (j.rows_per_head ? j.rows_per_head : j.n);
         if (j.n_act && j.n_act < j.n && j.rows_per_head) return set_error(FK_ERR_UNSUPPORTED, d.kernel + ": per-head products have one kind of output");
         if (j.n_act) j.y = s.out((j.n_act < j.n ? j.n_act : outs) * 2);
@@ -577,12 +588,48 @@ fk_status plan_layer_jobs_d(const Dispatch& d, Launch* l, SlotRW* rw) {
         j.hist = s.inout<uint16_t>((uint64_t)j.taps * j.ldh * 2);
         j.y = s.out<uint16_t>((uint64_t)j.heads * j.p * 2);
     }
+    if (d.u("delta_heads")) {
+        DeltaJob& j = a.delta;
+        j.heads = d.u("delta_heads"); j.kv_heads = d.u("delta_kv_heads"); j.dim = d.u("delta_dim"); j.dim_ld = d.u("delta_dim_ld"); j.vdim_ld = d.u("delta_vdim_ld");
+        j.state_ld = d.u("delta_state_ld"); j.rank_ld = d.u("delta_rank_ld"); j.ldh = d.u("delta_ldh"); j.taps = d.u("delta_taps");
+        const uint64_t nd = (uint64_t)j.heads * j.dim_ld, nv = (uint64_t)j.heads * j.vdim_ld, ch = 2ull * j.kv_heads * j.dim_ld + nv;
+        if (!j.kv_heads || !j.dim || !nd || !nv || !j.taps || j.ldh < ch) return set_error(FK_ERR_INVALID, d.kernel + ": delta rule parameters missing");
+        j.u = s.in<uint16_t>(ch * 2);
+        j.a1 = s.in<uint16_t>((uint64_t)j.rank_ld * 2);
+        j.beta = s.in<float>((uint64_t)j.heads * 4);
+        j.w = s.in<uint16_t>(ch * j.taps * 2);
+        j.a2 = s.in<uint16_t>(nd * j.rank_ld * 2);
+        j.dt_bias = s.in<uint16_t>(nd * 2);
+        j.a_log = s.in<uint16_t>((uint64_t)j.heads * 2);
+        j.offset = s.in<uint32_t>(4);
+        j.state = s.inout<float>(nv * j.state_ld * 4);
+        j.hist = s.inout<uint16_t>((uint64_t)j.taps * j.ldh * 2);
+        j.o = s.out<float>(nv * 4);
+    }
+    if (d.u("lru_width")) {
+        LruJob& j = a.lru;
+        j.width = d.u("lru_width"); j.block = d.u("lru_block"); j.ldh = d.u("lru_ldh"); j.taps = d.u("lru_taps");
+        if (!j.block || !j.taps || j.ldh < j.width) return set_error(FK_ERR_INVALID, d.kernel + ": linear recurrence parameters missing");
+        const uint64_t w2 = (uint64_t)j.width * 2;
+        j.u = s.in<uint16_t>(w2);
+        j.w = s.in<uint16_t>(w2 * j.taps);
+        j.b = s.in<uint16_t>(w2);
+        j.gates = s.in<uint16_t>(w2 * 2 * j.block);
+        j.rb = s.in<uint16_t>(w2);
+        j.ib = s.in<uint16_t>(w2);
+        j.lam = s.in<uint16_t>(w2);
+        j.offset = s.in<uint32_t>(4);
+        j.state = s.inout<float>(w2 * 2);
+        j.hist = s.inout<uint16_t>((uint64_t)j.taps * j.ldh * 2);
+        j.y = s.inout<uint16_t>(w2);
+    }
     FK_TRY(s.end());
     return plan_layer_jobs(a, l);
 }
 
-// x, [mix: has_mix], [att, w: ko > 0], [expert rows, down, index, weight, h2: top > 0], [step: has_step]
-//   {n, ko, ldo, kf, top, experts}
+// x, [mix: has_mix], [att, w: ko > 0], [expert rows, down, index, weight, h2: top > 0], [step: has_step],
+// [o, z, norm weights: norm_heads > 0]
+//   {n, ko, ldo, kf, top, experts, norm_heads, norm_dim, norm_ld, norm_eps}
 fk_status plan_layer_out_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     LayerOutArgs a;
     memset(&a, 0, sizeof(a));
@@ -603,6 +650,13 @@ fk_status plan_layer_out_d(const Dispatch& d, Launch* l, SlotRW* rw) {
         a.h2 = s.in<uint16_t>((uint64_t)a.n * 2);
     }
     if (d.u("has_step")) a.step = s.in<uint16_t>((uint64_t)a.n * 2);
+    a.heads = d.u("norm_heads"); a.hdim = d.u("norm_dim"); a.hld = d.u("norm_ld", a.hdim); a.heps = (float)d.param("norm_eps", 1e-6);
+    if (a.heads) {
+        const uint64_t nv = (uint64_t)a.heads * a.hld;
+        a.ho = s.in<float>(nv * 4);
+        a.hz = s.in<uint16_t>(nv * 2);
+        a.hw = s.in<uint16_t>((uint64_t)a.hld * 2);
+    }
     FK_TRY(s.end());
     return plan_layer_out(a, l);
 }

@@ -6,14 +6,17 @@
 //     row, a gated norm in groups, the combination of the attention's partial rows -- with the first weight rows
 //     already requested;
 //   * the gate / up pair of the chosen experts;
-//   * the router's softmax and choice, the latent cache row, a state-space step with its convolution.
+//   * the router's softmax and choice, the latent cache row;
+//   * a step of a state-space mixer, a gated delta rule or a gated linear recurrence, with its convolution and gates.
 // `layer_out_kernel` closes a layer: per element of the residual row the mixer's output projection, the weighted down
 // projections of the chosen experts and the identities' share, added to the row in fp32.
 //
 // A latent-attention layer is six launches (norms + down projections + router | queries, cache row, choice | queries
-// into the latent space, gate / up | attention | W_uv | output), a state-space layer four.
-#include "act_device.hpp"
+// into the latent space, gate / up | attention | W_uv | output), a state-space layer four.  A joint layer is the norm with
+// the joint input projection, the recurrence's step (or the cache rows and the attention), the joint output projection.
+#include "column_device.hpp"
 #include "layer_decode.hpp"
+#include "lru_device.hpp"
 #include "split_device.hpp"
 
 namespace fk {
@@ -133,11 +136,32 @@ __device__ void stage_row(const GemvJob& j, uint32_t head, uint32_t first_block,
             const float4 v = load(c);
             ss = fmaf(v.x, v.x, ss); ss = fmaf(v.y, v.y, ss); ss = fmaf(v.z, v.z, ss); ss = fmaf(v.w, v.w, ss);
         }
+        float mean = 0.f;
+        if (j.nb) {   // layer norm: ss becomes the sum of the squared deviations
+            float sum = 0.f;
+#pragma unroll
+            for (uint32_t i = 0; i < kHold; ++i) sum += (held[i].x + held[i].y) + (held[i].z + held[i].w);
+            for (uint32_t c = (tid + kHold * kJobBlock) * 4u; c < j.k; c += kJobBlock * 4u) {
+                const float4 v = load(c);
+                sum += (v.x + v.y) + (v.z + v.w);
+            }
+            mean = block_sum<kJobBlock>(sum, red + 4) / (float)j.width;
+            ss = 0.f;
+            auto dev = [&](uint32_t c, float4 v) __attribute__((always_inline)) {
+                const float d[4] = {v.x - mean, v.y - mean, v.z - mean, v.w - mean};
+#pragma unroll
+                for (uint32_t e = 0; e < 4; ++e) ss = c + e < j.width ? fmaf(d[e], d[e], ss) : ss;
+            };
+#pragma unroll
+            for (uint32_t i = 0; i < kHold; ++i) dev((tid + i * kJobBlock) * 4u, held[i]);
+            for (uint32_t c = (tid + kHold * kJobBlock) * 4u; c < j.k; c += kJobBlock * 4u) dev(c, load(c));
+        }
         ss = block_sum<kJobBlock>(ss, red);
         const float r = 1.0f / sqrtf(ss / (float)j.width + j.eps);
         auto put = [&](uint32_t c, float4 v) __attribute__((always_inline)) {
-            const float4 w = act_load4(j.nw + c);
-            const uint2 o = make_uint2(pack_bf16(v.x * r * w.x, v.y * r * w.y), pack_bf16(v.z * r * w.z, v.w * r * w.w));
+            const float4 w = act_load4(j.nw + c), b = j.nb ? act_load4(j.nb + c) : make_float4(0.f, 0.f, 0.f, 0.f);
+            v.x = (v.x - mean) * r; v.y = (v.y - mean) * r; v.z = (v.z - mean) * r; v.w = (v.w - mean) * r;
+            const uint2 o = make_uint2(pack_bf16(fmaf(v.x, w.x, b.x), fmaf(v.y, w.y, b.y)), pack_bf16(fmaf(v.z, w.z, b.z), fmaf(v.w, w.w, b.w)));
             *reinterpret_cast<uint2*>(xs + c) = o;
             if (j.keep && first_block) *reinterpret_cast<uint2*>(j.keep + c) = o;
         };
@@ -180,6 +204,17 @@ __device__ void stage_row(const GemvJob& j, uint32_t head, uint32_t first_block,
             float v = 0.f;
             if (c < j.width) v = act_load(y + c) * silu(act_load(z + c)) * sums[c / part] * bf16_bits_to_f32(j.nw[c]);
             act_store(xs + c, v);
+        }
+    } else if (j.mode == kRowJoin) {
+        const float* x = reinterpret_cast<const float*>(j.x);
+        const uint16_t* second = reinterpret_cast<const uint16_t*>(j.x2);
+        const uint32_t half = j.k / 2u;
+        for (uint32_t c = tid * 4u; c < half; c += kJobBlock * 4u) {
+            float v[4];
+#pragma unroll
+            for (uint32_t e = 0; e < 4; ++e) v[e] = c + e < j.width ? x[c + e] : 0.f;
+            *reinterpret_cast<uint2*>(xs + c) = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+            *reinterpret_cast<uint2*>(xs + half + c) = *reinterpret_cast<const uint2*>(second + c);
         }
     } else {   // kRowCombine: the partial rows of one head, [splits][heads][pl] = latent sums | maximum | sum
         const float* p = reinterpret_cast<const float*>(j.x) + (size_t)head * j.pl;
@@ -340,6 +375,121 @@ __device__ void scan_step(const ScanJob& a, uint32_t h, uint32_t pt, float* sm) 
     if (live && nl == 0) act_store(a.y + (size_t)h * a.p + p, fmaf(bf16_bits_to_f32(a.d[h]), x, out));
 }
 
+// The convolution of one channel for the token at `pos`; its raw input takes the ring row of the one that has left.
+__device__ __forceinline__ float conv_token(const uint16_t* u, const uint16_t* w, const uint16_t* b, uint16_t* hist, uint32_t ch, uint32_t taps, uint32_t ldh,
+                                            uint32_t pos, bool write) {
+    const uint16_t raw = u[ch];
+    const uint16_t* k = w + (size_t)ch * taps;
+    float v = b ? bf16_bits_to_f32(b[ch]) : 0.f;
+    for (uint32_t i = 0; i + 1u < taps; ++i) {
+        const uint32_t back = taps - 1u - i;
+        if (back <= pos) v = fmaf(bf16_bits_to_f32(k[i]), bf16_bits_to_f32(hist[(size_t)((pos - back) % taps) * ldh + ch]), v);
+    }
+    v = fmaf(bf16_bits_to_f32(k[taps - 1u]), bf16_bits_to_f32(raw), v);
+    if (write) hist[(size_t)(pos % taps) * ldh + ch] = raw;
+    return v;
+}
+
+// One token of one head and sixteen value columns of a gated delta rule (the layout of delta.hip).  Every workgroup of a
+// head forms its unit vectors and decays itself: the second decay projection is dim x rank, out of the L2 for all but one.
+__device__ void delta_step(const DeltaJob& a, uint32_t h, uint32_t pt, float* sm) {
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, pos = *a.offset;
+    const uint32_t per = a.heads / a.kv_heads, g = h / per, nk = a.kv_heads * a.dim_ld, p0 = pt * 16u;
+    float *qs = sm, *ks = qs + a.state_ld, *gs = ks + a.state_ld, *vs = gs + a.state_ld;
+    const uint32_t pl = wave * 4u + (lane >> 4), nl = (lane & 15u) * 4u, ni = a.state_ld / 64u;
+    float* state = a.state + ((size_t)h * a.vdim_ld + p0 + pl) * a.state_ld + nl;
+    float4 S[4];
+#pragma unroll
+    for (uint32_t i = 0; i < 4; ++i)
+        if (i < ni) S[i] = *reinterpret_cast<const float4*>(state + 64u * i);
+    // decays: four lanes per row of the projection
+    for (uint32_t d = tid >> 2; d < a.state_ld; d += kJobBlock / 4u) {
+        float z = 0.f;
+        if (d < a.dim_ld) {
+            const uint16_t* row = a.a2 + ((size_t)h * a.dim_ld + d) * a.rank_ld;
+            for (uint32_t c = (tid & 3u) * 8u; c < a.rank_ld; c += 32u)
+                z = dot8(*reinterpret_cast<const ld_u32x4_t*>(row + c), *reinterpret_cast<const ld_u32x4_t*>(a.a1 + c), z);
+        }
+        z = group_sum(z, 4);
+        if ((tid & 3u) == 0)
+            gs[d] = d < a.dim_ld ? expf(-expf(bf16_bits_to_f32(a.a_log[h])) * softplus(z + bf16_bits_to_f32(a.dt_bias[(size_t)h * a.dim_ld + d]))) : 0.f;
+    }
+    for (uint32_t i = tid; i < 2u * a.state_ld + 16u; i += kJobBlock) {
+        uint32_t ch = 0xffffffffu, at = i;
+        bool write = h % per == 0u && pt == 0u;
+        if (i < a.state_ld) {
+            if (i < a.dim_ld) ch = g * a.dim_ld + i;
+        } else if (i < 2u * a.state_ld) {
+            if (i - a.state_ld < a.dim_ld) ch = nk + g * a.dim_ld + i - a.state_ld;
+        } else {
+            ch = 2u * nk + h * a.vdim_ld + p0 + i - 2u * a.state_ld;
+            at = i + a.state_ld;   // behind the decays
+            write = true;
+        }
+        sm[at] = ch != 0xffffffffu ? round_bf16(silu(conv_token(a.u, a.w, nullptr, a.hist, ch, a.taps, a.ldh, pos, write))) : 0.f;
+    }
+    const float beta = sigmoid(a.beta[h]);
+    __syncthreads();
+    float qq = 0.f, kk = 0.f;
+    for (uint32_t c = lane; c < a.state_ld; c += 64u) {
+        qq = fmaf(qs[c], qs[c], qq);
+        kk = fmaf(ks[c], ks[c], kk);
+    }
+    const float fq = 1.0f / (sqrtf(wave_sum(qq) + 1e-6f) * sqrtf((float)a.dim)), fk = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
+    float sk = 0.f, sq = 0.f, kq = 0.f;
+#pragma unroll
+    for (uint32_t i = 0; i < 4; ++i) {
+        if (i >= ni) break;
+        const float4 k = *reinterpret_cast<const float4*>(ks + nl + 64u * i), q = *reinterpret_cast<const float4*>(qs + nl + 64u * i);
+        const float4 d = *reinterpret_cast<const float4*>(gs + nl + 64u * i);
+        S[i].x *= d.x; S[i].y *= d.y; S[i].z *= d.z; S[i].w *= d.w;
+        sk = fmaf(S[i].x, k.x, sk); sk = fmaf(S[i].y, k.y, sk); sk = fmaf(S[i].z, k.z, sk); sk = fmaf(S[i].w, k.w, sk);
+        sq = fmaf(S[i].x, q.x, sq); sq = fmaf(S[i].y, q.y, sq); sq = fmaf(S[i].z, q.z, sq); sq = fmaf(S[i].w, q.w, sq);
+        kq = fmaf(k.x, q.x, kq); kq = fmaf(k.y, q.y, kq); kq = fmaf(k.z, q.z, kq); kq = fmaf(k.w, q.w, kq);
+    }
+    sk = group_sum(sk, 16) * fk;
+    sq = group_sum(sq, 16) * fq;
+    kq = group_sum(kq, 16) * fk * fq;
+    const float u = beta * (vs[pl] - sk), uk = u * fk;
+#pragma unroll
+    for (uint32_t i = 0; i < 4; ++i) {
+        if (i >= ni) break;
+        const float4 k = *reinterpret_cast<const float4*>(ks + nl + 64u * i);
+        S[i].x = fmaf(k.x, uk, S[i].x); S[i].y = fmaf(k.y, uk, S[i].y); S[i].z = fmaf(k.z, uk, S[i].z); S[i].w = fmaf(k.w, uk, S[i].w);
+        *reinterpret_cast<float4*>(state + 64u * i) = S[i];
+    }
+    if (nl == 0) a.o[(size_t)h * a.vdim_ld + p0 + pl] = fmaf(kq, u, sq);
+}
+
+// One token of some channels of one diagonal block: the convolution of the whole block, then per channel its two gates.
+__device__ void lru_token(const LruJob& a, uint32_t part, uint32_t sub, uint16_t* xs) {
+    const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, pos = *a.offset;
+    const uint32_t c0 = sub * kLruRows, count = a.block - c0 < kLruRows ? a.block - c0 : kLruRows;
+    const uint32_t turns = wave < count ? (count - wave + 3u) / 4u : 0u;
+    const uint16_t *wr = a.gates + (size_t)part * 2u * a.block * a.block, *wi = wr + (size_t)a.block * a.block;
+    auto rows = [&](uint32_t t, const uint16_t*& w0, const uint16_t*& w1) __attribute__((always_inline)) {
+        const uint32_t r = wave + t * 4u, rr = c0 + (r < count ? r : count - 1u);
+        w0 = wr + (size_t)rr * a.block;
+        w1 = wi + (size_t)rr * a.block;
+    };
+    PairStream<decltype(rows)> st(rows, a.block, turns, lane);
+    st.start();
+    for (uint32_t i = tid; i < a.block; i += kJobBlock)
+        act_store(xs + i, conv_token(a.u, a.w, a.b, a.hist, part * a.block + i, a.taps, a.ldh, pos, i - c0 < count));
+    __syncthreads();
+    if (!turns) return;
+    st.run(xs, [&](uint32_t t, float zr, float zi) __attribute__((always_inline)) {
+        const uint32_t r = wave + t * 4u;
+        if (lane != 0 || r >= count) return;
+        const uint32_t c = part * a.block + c0 + r;
+        float decay, add;
+        lru_step(zr + bf16_bits_to_f32(a.rb[c]), zi + bf16_bits_to_f32(a.ib[c]), lru_rate(a.lam[c]), act_load(xs + c0 + r), decay, add);
+        const float S = fmaf(decay, a.state[c], add);
+        a.state[c] = S;
+        act_store(a.y + c, S * act_load(a.y + c));
+    });
+}
+
 __global__ __launch_bounds__(kJobBlock) void layer_jobs_kernel(const LayerJobsArgs a) {
     extern __shared__ __align__(16) uint16_t lds[];
     __shared__ __align__(16) float red[8 + kMaxGateGroups];
@@ -373,7 +523,7 @@ __global__ __launch_bounds__(kJobBlock) void layer_jobs_kernel(const LayerJobsAr
         st.run(lds, [&](uint32_t t, float s0, float s1) __attribute__((always_inline)) {
             const uint32_t r = wave * 2u + t * 8u + lane;
             if (lane < 2u && r < count) {
-                const float v = lane ? s1 : s0;
+                const float v = column_value(j.out, row0 + r, lane ? s1 : s0);
                 if (row0 + r >= j.n_act) j.y32[y0 + r - j.n_act] = v;
                 else reinterpret_cast<uint16_t*>(j.y)[y0 + r] = (uint16_t)f32_to_bf16_bits(v);
             }
@@ -418,6 +568,16 @@ __global__ __launch_bounds__(kJobBlock) void layer_jobs_kernel(const LayerJobsAr
     if (b - a.scan.first < a.scan.blocks) {
         const uint32_t local = b - a.scan.first, pts = (a.scan.p + 15u) / 16u;
         scan_step(a.scan, local / pts, local % pts, reinterpret_cast<float*>(lds));
+        return;
+    }
+    if (b - a.delta.first < a.delta.blocks) {
+        const uint32_t local = b - a.delta.first, pts = a.delta.vdim_ld / 16u;
+        delta_step(a.delta, local / pts, local % pts, reinterpret_cast<float*>(lds));
+        return;
+    }
+    if (b - a.lru.first < a.lru.blocks) {
+        const uint32_t local = b - a.lru.first;
+        lru_token(a.lru, local / a.lru.blocks_per_part, local % a.lru.blocks_per_part, lds);
     }
 }
 
@@ -463,8 +623,27 @@ __global__ __launch_bounds__(kJobBlock) void layer_out_kernel(const LayerOutArgs
         if (lane == 0) { n_items = at; id_scale = idw; }
     }
     const uint32_t base = a.wo ? a.ko : 0u;
+    uint32_t formed = 0;
+    if (a.ho) {
+        formed = a.heads * a.hld;
+        for (uint32_t h = wave; h < a.heads; h += 4u) {
+            const float* o = a.ho + (size_t)h * a.hld;
+            float ss = 0.f;
+            for (uint32_t c = lane * 2u; c < a.hld; c += 128u) {
+                const float2 v = *reinterpret_cast<const float2*>(o + c);
+                ss = fmaf(v.x, v.x, ss);
+                ss = fmaf(v.y, v.y, ss);
+            }
+            const float k = 1.0f / sqrtf(wave_sum(ss) / (float)a.hdim + a.heps);
+            for (uint32_t c = lane * 2u; c < a.hld; c += 128u) {
+                const float2 v = *reinterpret_cast<const float2*>(o + c);
+                const uint32_t w = *reinterpret_cast<const uint32_t*>(a.hw + c), z = *reinterpret_cast<const uint32_t*>(a.hz + (size_t)h * a.hld + c);
+                *reinterpret_cast<uint32_t*>(xs + (size_t)h * a.hld + c) = pack_bf16(v.x * k * bf16_lo(w) * sigmoid(bf16_lo(z)), v.y * k * bf16_hi(w) * sigmoid(bf16_hi(z)));
+            }
+        }
+    }
     if (a.wo)
-        for (uint32_t c = tid * 8u; c < a.ko; c += kJobBlock * 8u) *reinterpret_cast<ld_u32x4_t*>(xs + c) = *reinterpret_cast<const ld_u32x4_t*>(a.att + c);
+        for (uint32_t c = formed + tid * 8u; c < a.ko; c += kJobBlock * 8u) *reinterpret_cast<ld_u32x4_t*>(xs + c) = *reinterpret_cast<const ld_u32x4_t*>(a.att + c);
     for (uint32_t c = tid * 8u; c < a.top * a.kf; c += kJobBlock * 8u) *reinterpret_cast<ld_u32x4_t*>(xs + base + c) = *reinterpret_cast<const ld_u32x4_t*>(a.eh + c);
     __syncthreads();
     const uint32_t n = n_items;
@@ -520,6 +699,23 @@ fk_status plan_layer_jobs(LayerJobsArgs& a, Launch* out) {
         take(j.first, j.blocks);
         lds = std::max(lds, (16u + 2u * j.state_ld) * 4u);
     }
+    if (a.delta.u) {
+        DeltaJob& j = a.delta;
+        if (!j.kv_heads || j.heads % j.kv_heads || j.dim_ld % 32 || j.vdim_ld % 32 || j.state_ld % 64 || j.state_ld < j.dim_ld || j.state_ld > kMaxSsmState ||
+            j.rank_ld % 8 || !j.taps)
+            return set_error(FK_ERR_UNSUPPORTED, "layer jobs: delta rule shape");
+        j.blocks = j.heads * (j.vdim_ld / 16);
+        take(j.first, j.blocks);
+        lds = std::max(lds, (3u * j.state_ld + 16u) * 4u);
+    }
+    if (a.lru.u) {
+        LruJob& j = a.lru;
+        if (!j.block || j.block % kRowPad || j.width % j.block || !j.taps) return set_error(FK_ERR_UNSUPPORTED, "layer jobs: linear recurrence shape");
+        j.blocks_per_part = (j.block + kLruRows - 1) / kLruRows;
+        j.blocks = j.width / j.block * j.blocks_per_part;
+        take(j.first, j.blocks);
+        lds = std::max(lds, j.block * 2u);
+    }
     if (a.route.logits) {
         if (a.route.outputs > kMaxRouterOutputs || a.route.top > kMaxRouterTop || !a.route.top || a.route.top > a.route.outputs) return set_error(FK_ERR_UNSUPPORTED, "layer jobs: router shape");
         a.route.blocks = 1;
@@ -539,6 +735,8 @@ fk_status plan_layer_jobs(LayerJobsArgs& a, Launch* out) {
         if (j.k % kRowPad || j.ldw < j.k || j.ldw % 8 || j.width > j.k || !j.n) return set_error(FK_ERR_INVALID, "layer jobs: product shape");
         if (j.mode == kRowGated && (!j.groups || j.groups > kMaxGateGroups || j.width % j.groups)) return set_error(FK_ERR_UNSUPPORTED, "layer jobs: at most 64 norm groups");
         if (j.mode == kRowCombine && (!j.rows_per_head || !j.splits || j.splits > kMaxSplits)) return set_error(FK_ERR_INVALID, "layer jobs: combination of what");
+        if (j.mode == kRowJoin && (!j.x2 || j.k % (2 * kRowPad) || j.width > j.k / 2)) return set_error(FK_ERR_INVALID, "layer jobs: joined rows");
+        if (j.out.fn > kFnMax || j.out.fn2 > kFnMax) return set_error(FK_ERR_INVALID, "layer jobs: column function");
         if (j.rows_per_head && j.n % j.rows_per_head) return set_error(FK_ERR_INVALID, "layer jobs: rows per head");
         if (!j.rows_per_head) j.y_head = 0;
         else if (j.y_head < j.rows_per_head) return set_error(FK_ERR_INVALID, "layer jobs: outputs per head");
@@ -578,6 +776,7 @@ fk_status plan_layer_jobs(LayerJobsArgs& a, Launch* out) {
 fk_status plan_layer_out(LayerOutArgs& a, Launch* out) {
     if (!a.x || !a.n || (a.wo && (!a.att || a.ko % kRowPad || a.ldo < a.ko)) || (a.top && (!a.eh || !a.wd || !a.index || !a.weight || !a.h2 || a.kf % kRowPad || !a.kf)))
         return set_error(FK_ERR_INVALID, "layer out: bad arguments");
+    if (a.ho && (!a.hz || !a.hw || !a.wo || !a.hdim || a.hld % 8 || a.hld < a.hdim || (uint64_t)a.heads * a.hld > a.ko)) return set_error(FK_ERR_INVALID, "layer out: heads to normalise");
     if (!a.wo) a.ko = 0;
     if (!a.top) a.kf = 0;
     a.max_items = ((a.ko + 511) / 512 + a.top * ((a.kf + 511) / 512) + 2) / 2 * 2;   // even: the inputs behind stay 16-byte aligned

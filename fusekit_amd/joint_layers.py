@@ -333,6 +333,15 @@ def scratch(m, f, R: int, act: int, capacity: int, want: Callable[[str, int], No
         want("carry", -(-R // LRU_CHUNK) * 2 * m.inner * 4)
 
 
+def fusable(m) -> bool:
+    """Whether the mixer has the fused launches of one token."""
+    if m.kind == "attention":
+        return m.dim_ld <= 512
+    if m.kind == "channel_delta":
+        return m.state_ld <= 256
+    return m.block_ld <= 30720
+
+
 class JointTasks:
     """Task lists of joint layers (a part of LayerRuntime)."""
 
@@ -406,3 +415,39 @@ class JointTasks:
         t.append(Dispatch(self._name("lru_scan"),
                           [arg(b["xbc"]), arg(b["gates"]), arg(w.vecs[q + "ra.b"]), arg(w.vecs[q + "ri.b"]), arg(w.vecs[q + "lam"]), arg(st["state"]), u("y"), arg(b["carry"])],
                           dict(rows=rows, width=m.inner, block=n, ldx=m.inner, ldy=col.width, act=c.act)))
+
+    # -- one decoded token in fused launches
+    def _fused_joint_tasks(self, t, run: int, x, step) -> None:
+        """Norm and joint input projection | the recurrence's step (or cache rows | attention) | joint output projection."""
+        c, w, b, st = self.cfg, self.w, self.buf, self.state.entries[run]
+        i = self.runs[run][0]
+        l, p, off = c.layers[i], f"l{i}.", arg(self.offset)
+        m, q = l.mixer, p + "mix."
+        col = Columns(m, l.mlp)
+        u = lambda name: arg(b["u"], None, col.at[name] * 2)
+        more = dict(col.fns, mode=1, width=c.width, eps=c.eps, step=len(step), layer_norm=int(c.layer_norm), has_bias=int(m.kind == "rglru"))
+        norm = [arg(w.vecs[p + "norm1"])] + ([arg(w.vecs[p + "norm1.b"])] if c.layer_norm else [])
+        W = w.mats[q + "in"]
+        self._jobs(t, [x] + step + norm + [arg(W.w)] + ([arg(w.vecs[q + "in.b"])] if m.kind == "rglru" else []) + [arg(b["u"])] + ([arg(b["beta"])] if col.tail else []),
+                   **self._product(0, W, col.width, **more))
+        a, prm = [x, u(m.out_part), arg(w.mats[p + "out"].w)], dict(n=c.width, ko=col.ko, ldo=w.mats[p + "out"].k)
+        after = []
+        if m.kind == "attention":
+            t.append(self._qk_store(m, q, col, run, 1, off))
+            t.append(Dispatch(self._name("sdpa_decode"), [arg(b["q"]), arg(st["k"]), arg(st["v"]), arg(self.kv_len), u("q"), arg(b["part"]), arg(b["counters"])],
+                              dict(n_heads=m.heads, n_kv=m.kv_heads, head_dim=m.dim_ld, capacity=c.capacity, scale=m.scale)))
+        elif m.kind == "channel_delta":
+            A, G = w.mats[q + "a2"], w.mats[q + "g2"]
+            self._jobs(t, [u("g1"), arg(G.w), arg(b["gate"]), u("q"), u("a1"), arg(b["beta"]), arg(w.vecs[q + "conv"]), arg(A.w), arg(w.vecs[q + "dt_bias"]),
+                           arg(w.vecs[q + "A_log"]), off, arg(st["state"]), arg(st["hist"]), arg(b["o"])],
+                       **self._product(0, G, G.n, mode=0), delta_heads=m.heads, delta_kv_heads=m.kv_heads, delta_dim=m.dim, delta_dim_ld=m.dim_ld,
+                       delta_vdim_ld=m.vdim_ld, delta_state_ld=m.state_ld, delta_rank_ld=A.k, delta_ldh=pad(m.channels), delta_taps=m.conv)
+            after = [arg(b["o"]), arg(b["gate"]), arg(w.vecs[q + "norm"])]
+            prm.update(norm_heads=m.heads, norm_dim=m.vdim, norm_ld=m.vdim_ld, norm_eps=c.eps)
+        else:
+            self._jobs(t, [u("x"), arg(w.vecs[q + "conv"]), arg(w.vecs[q + "conv.b"]), arg(w.mats[q + "gates"].w), arg(w.vecs[q + "ra.b"]), arg(w.vecs[q + "ri.b"]),
+                           arg(w.vecs[q + "lam"]), off, arg(st["state"]), arg(st["hist"]), u("y")],
+                       lru_width=m.inner, lru_block=m.block_ld, lru_ldh=m.inner, lru_taps=m.conv)
+        if step:
+            a, prm["has_step"] = a + step, 1
+        t.append(Dispatch(self._name("layer_out"), a + after, prm))

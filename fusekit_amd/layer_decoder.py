@@ -578,6 +578,7 @@ class LayerRuntime(JointTasks):
             want(n, R * D * b)
         if c.looped and c.join:
             want("cat", R * 2 * D * e)
+            want("x2", D * 4)
         for l in c.layers:
             m, f = l.mixer, l.experts
             if l.joint:
@@ -756,12 +757,16 @@ class LayerRuntime(JointTasks):
     def _fused(self) -> bool:
         """Whether every layer has the fused decode launches."""
         c = self.cfg
-        if c.act != 16 or not c.fuse or not c.tiled or pad(c.width) > 30720 or any(l.joint for l in c.layers):
+        if c.act != 16 or not c.fuse or not c.tiled or pad(c.width) * (2 if c.looped and c.join else 1) > 30720:
             return False
         for l in c.layers:
-            m, f = l.mixer, l.mlp
+            m, f = l.mixer, l.experts
             ko = 0
-            if m.kind == "latent_attention":
+            if l.joint:
+                ko = joint_layers.Columns(m, l.mlp).ko
+                if not joint_layers.fusable(m):
+                    return False
+            elif m.kind == "latent_attention":
                 ko = pad(m.heads * m.vdim_ld)
                 if not self._split_latent(m) or max(pad(m.q_rank), m.rank_ld) > 30720:
                     return False
@@ -782,25 +787,35 @@ class LayerRuntime(JointTasks):
     def _fused_tasks(self, t: List[Dispatch]) -> None:
         c, w, b = self.cfg, self.w, self.buf
         off, D = arg(self.offset), pad(c.width)
-        t.append(Dispatch(self._name("embed_lookup_decode"), [arg(self.token), arg(w.mats["embed"].w), arg(b["x"])],
-                          dict(bits=16, hidden=c.width, vocab=c.vocab, output_scale=c.embed_scale, out_bits=32, x_row_stride=D)))
+        t.append(self._embed_task(arg(self.token), off, 1))
+        x, other = arg(b["x"]), arg(b["x2"]) if "x2" in b else None
         for run, (i, first) in enumerate(self.runs):
-            m, f, p = c.layers[i].mixer, c.layers[i].mlp, f"l{i}."
+            m, f, p = c.layers[i].mixer, c.layers[i].experts, f"l{i}."
             q = p + "mix."
             st = self.state.entries[run]
-            step = [] if first is None else [arg(w.vecs["loop.step"], D * 2, first * D * 2)]
-            norm = dict(mode=1, width=c.width, eps=c.eps, step=len(step))
+            step = []
+            if first is not None and c.join:   # a product of the whole row: into the other of two rows
+                W = w.mats["loop.in"]
+                self._jobs(t, [x, arg(b["cat"], None, D * 2), arg(W.w), other], **self._product(0, W, 0, mode=4, width=c.width))
+                x, other = other, x
+            elif first is not None:
+                step = [arg(w.vecs["loop.step"], D * 2, first * D * 2)]
+            if c.layers[i].joint:
+                self._fused_joint_tasks(t, run, x, step)
+                continue
+            norm = dict(mode=1, width=c.width, eps=c.eps, step=len(step), layer_norm=int(c.layer_norm))
+            norm1 = [arg(w.vecs[p + "norm1"])] + ([arg(w.vecs[p + "norm1.b"])] if c.layer_norm else [])
             latent = m.kind == "latent_attention"
             # 1: norms; the mixer's joint down / input projection and the router
             Win = w.mats[q + ("down" if latent else "in")]
             n_act = 0 if latent else m.inner + m.channels
-            a = [arg(b["x"])] + step + [arg(w.vecs[p + "norm1"]), arg(Win.w)]
+            a = [x] + step + norm1 + [arg(Win.w)]
             a += [arg(b["low"])] if latent else [arg(b["u"]), arg(b["dt"])]
             prm = self._product(0, Win, n_act, **norm)
             if f:
                 Wr = w.mats[p + "mlp.router"]
-                a += [arg(b["x"])] + step + [arg(w.vecs[p + "norm2"]), arg(b["h2"]), arg(Wr.w), arg(b["rl"])]
-                prm.update(self._product(1, Wr, 0, keep=1, **norm))
+                a += [x] + step + [arg(w.vecs[p + "norm2"]), arg(b["h2"]), arg(Wr.w), arg(b["rl"])]
+                prm.update(self._product(1, Wr, 0, keep=1, **dict(norm, layer_norm=0)))
             self._jobs(t, a, **prm)
             route = [arg(b["rl"]), arg(w.vecs[p + "mlp.correction"]), arg(b["ridx"]), arg(b["rwt"])] if f else []
             prm_route = dict(route_outputs=f.outputs, route_top=f.top) if f else {}
@@ -836,7 +851,7 @@ class LayerRuntime(JointTasks):
                 self._jobs(t, [arg(b["y"]), arg(b["u"]), arg(w.vecs[q + "norm"]), arg(Wo.w), arg(b["mix"])] + pair,
                            **self._product(0, Wo, 0, mode=2, width=m.inner, groups=m.norm_groups, eps=c.eps), **prm_pair)
             # last: everything into the residual row
-            a, prm = [arg(b["x"])], dict(n=c.width)
+            a, prm = [x], dict(n=c.width)
             if latent:
                 A = pad(m.heads * m.vdim_ld)
                 a += [arg(b["att"]), arg(w.mats[q + "o"].w)]
@@ -852,8 +867,9 @@ class LayerRuntime(JointTasks):
                 prm["has_step"] = 1
             t.append(Dispatch(self._name("layer_out"), a, prm))
         head = w.mats["head"]
-        self._jobs(t, [arg(b["x"]), arg(w.vecs["final.norm"]), arg(head.w), arg(self.logits)],
-                   **self._product(0, head, 0, mode=1, width=c.width, eps=c.eps))
+        norm = [arg(w.vecs["final.norm"])] + ([arg(w.vecs["final.norm.b"])] if c.layer_norm else [])
+        self._jobs(t, [x] + norm + [arg(head.w), arg(self.logits)],
+                   **self._product(0, head, 0, mode=1, width=c.width, eps=c.eps, layer_norm=int(c.layer_norm)))
 
     def _ssm_tasks(self, t, run: int, rows: int, off) -> None:
         c, w, b = self.cfg, self.w, self.buf
