@@ -96,15 +96,15 @@ def main() -> int:
                     help="experiment only: the per-dispatch task list (five launches per layer) instead of the two-launch layer")
     ap.add_argument("--mode", choices=["persistent", "graph"], default="graph",
                     help="persistent: one whole-token kernel per replay; graph: one kernel node per task")
-    ap.add_argument("--workload", choices=["headline", "pusavik"], default="headline",
+    ap.add_argument("--workload", choices=["headline", "pusavik", "fumotar"], default="headline",
                     help="pusavik: prefill and decode of the layer-list decoder at a few sizes beside the mixture-of-experts "
-                         "decoder, instead of the headline benchmark")
-    ap.add_argument("--sizes", default="1k,2k,4k", help="sizes of --workload pusavik")
+                         "decoder, instead of the headline benchmark; fumotar: its joint layers beside the other design")
+    ap.add_argument("--sizes", default="1k,2k,4k", help="sizes of --workload pusavik / fumotar")
     args = ap.parse_args()
-    if args.workload == "pusavik":
+    if args.workload != "headline":
         from fusekit_amd import layer_bench
-        res = layer_bench.run([s for s in args.sizes.split(",") if s], kernels=not args.no_kernels)
-        print(json.dumps({"workload": "pusavik", "data": "synthetic (random-init weights)", "dtype": "bf16", "sizes": res}))
+        res = (layer_bench.run if args.workload == "pusavik" else layer_bench.run_joint)([s for s in args.sizes.split(",") if s], kernels=not args.no_kernels)
+        print(json.dumps({"workload": args.workload, "data": "synthetic (random-init weights)", "dtype": "bf16", "sizes": res}))
         return 0
     if args.gpus != 1:
         print("bench.py: this build runs on ONE GPU; the decode path has no multi-GPU mode (--gpus must be 1)",

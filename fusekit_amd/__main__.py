@@ -4,10 +4,10 @@
   generate --model DIR --ids 1,2,3 [--max-tokens N] [--capacity C] [--dtype float32]
                                          greedy decode of a checkpoint (token ids in, token ids out; no
                                          tokenizer is bundled); config.json chooses the model family
-  export-random --out DIR [--bits 4] [--layers 2] [--moe | --pusavik] ...
+  export-random --out DIR [--bits 4] [--layers 2] [--moe | --pusavik | --fumotar] ...
                                          write a small random-init model in the mlx-lm file layout (--moe: a
-                                         mixture-of-experts model in the deepseek_v2 layout; --pusavik: a
-                                         layer-list model; generate / patch / bench recognise it)
+                                         mixture-of-experts model in the deepseek_v2 layout; --pusavik, --fumotar:
+                                         layer-list models; generate / patch / bench recognise them)
   patch --model DIR [--out DIR/.fusekit] [--prefill-m 32,128] [--capacity C]
                                          the reference's `fusekit patch`: write task_graph.json, manifest.json and
                                          variants/prefill_mN/task_graph.json for a checkpoint
@@ -51,6 +51,7 @@ def main() -> int:
     e.add_argument("--seed", type=int, default=0)
     e.add_argument("--moe", action="store_true", help="a small mixture-of-experts model with low-rank keys (deepseek_v2 layout)")
     e.add_argument("--pusavik", action="store_true", help="a small layer-list model: latent attention and Mamba-2 mixers, routed experts")
+    e.add_argument("--fumotar", action="store_true", help="a small layer-list model: causal attention, delta-rule and linear-recurrence mixers")
     from . import bench_cli
     bench_cli.add_arguments(sub)
     args = ap.parse_args()
@@ -63,12 +64,12 @@ def main() -> int:
         print(json.dumps({f: (getattr(t, f).decode() if isinstance(getattr(t, f), bytes) else getattr(t, f))
                           for f, _ in t._fields_}, indent=1))
         return 0
-    if args.cmd == "export-random" and args.pusavik:
+    if args.cmd == "export-random" and (args.pusavik or args.fumotar):
         from .checkpoint import save_layer_checkpoint
-        from .layer_decoder import random_tensors, small_config
-        lc = small_config(width=args.hidden, vocab=args.vocab, heads=args.heads, ff=args.inter)
+        from .layer_decoder import random_tensors, small_config, small_joint_config
+        lc = (small_joint_config if args.fumotar else small_config)(width=args.hidden, vocab=args.vocab, heads=args.heads, ff=args.inter)
         save_layer_checkpoint(args.out, lc, random_tensors(lc, seed=args.seed))
-        print(f"wrote {args.out}/config.json and model.safetensors (Pusavik)")
+        print(f"wrote {args.out}/config.json and model.safetensors ({lc.design})")
         return 0
     from .decoder import DecoderConfig, DecoderWeights
     if args.cmd == "export-random" and args.moe:

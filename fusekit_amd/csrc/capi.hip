@@ -889,6 +889,10 @@ fk_status fk_xcd_check(void* workspace, fk_stream s) {
 
 int fk_latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld) { return latent_prefill_supported(dim_ld, rot_ld, vdim_ld) ? 1 : 0; }
 int fk_latent_split_supported(uint32_t rank_ld, uint32_t ldc) { return latent_split_supported(rank_ld, ldc) ? 1 : 0; }
+int fk_delta_chunk_supported(uint32_t dim_ld, uint32_t vdim_ld) { return delta_chunk_supported(dim_ld, vdim_ld) ? 1 : 0; }
+uint64_t fk_delta_chunk_work_bytes(uint32_t rows, uint32_t heads, uint32_t dim_ld, uint32_t vdim_ld) {
+    return delta_chunk_work_bytes(rows, heads, dim_ld, vdim_ld);
+}
 int fk_ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n) { return ssm_chunk_supported(heads, p, n) ? 1 : 0; }
 
 }  // extern "C"

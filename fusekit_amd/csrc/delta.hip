@@ -77,12 +77,13 @@ __global__ __launch_bounds__(kDeltaBlock) void delta_scan_kernel(const DeltaScan
         w.v = act_load(reinterpret_cast<const T*>(a.v) + (size_t)r * a.ldx + (size_t)h * a.vdim_ld + p);
         w.beta = a.beta[(size_t)r * a.ldb + h];
     };
-    Row w, n;
-    fetch(0, w);
+    constexpr uint32_t kDeep = NI <= 2 ? 4 : 2;   // rows on their way
+    Row in[kDeep];
+#pragma unroll
+    for (uint32_t e = 0; e < kDeep; ++e) fetch(e < a.rows ? e : a.rows - 1u, in[e]);
     float* o = a.o + (size_t)h * a.vdim_ld + p;
     const size_t ldo = (size_t)a.heads * a.vdim_ld;
-    for (uint32_t r = 0; r < a.rows; ++r) {
-        fetch(r + 1u < a.rows ? r + 1u : r, n);
+    auto step = [&](uint32_t r, const Row& w) __attribute__((always_inline)) {
         float sk = 0.f, sq = 0.f, kq = 0.f;
 #pragma unroll
         for (int i = 0; i < NI; ++i) {
@@ -101,7 +102,13 @@ __global__ __launch_bounds__(kDeltaBlock) void delta_scan_kernel(const DeltaScan
             S[i].z = fmaf(w.k[i].z, u, S[i].z); S[i].w = fmaf(w.k[i].w, u, S[i].w);
         }
         if (nl == 0) o[(size_t)r * ldo] = fmaf(kq, u, sq);
-        w = n;
+    };
+    for (uint32_t r0 = 0; r0 < a.rows; r0 += kDeep) {
+#pragma unroll
+        for (uint32_t e = 0; e < kDeep; ++e) {
+            if (r0 + e < a.rows) step(r0 + e, in[e]);
+            fetch(r0 + e + kDeep < a.rows ? r0 + e + kDeep : a.rows - 1u, in[e]);
+        }
     }
 #pragma unroll
     for (int i = 0; i < NI; ++i) *reinterpret_cast<float4*>(state + 64 * i) = S[i];

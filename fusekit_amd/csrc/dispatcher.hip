@@ -1568,6 +1568,7 @@ const Family kFamilies[] = {
     {"fusekit_gqa_rows", plan_gqa_rows_d},
     {"fusekit_delta_prep", plan_delta_prep_d},
     {"fusekit_delta_scan", plan_delta_scan_d},
+    {"fusekit_delta_chunk", plan_delta_chunk_d},
     {"fusekit_lru_scan", plan_lru_scan_d},
     {"fusekit_latent_prefill", plan_latent_prefill_d},
     {"fusekit_ssm_chunk", plan_ssm_chunk_d},

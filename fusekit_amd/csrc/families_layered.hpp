@@ -244,6 +244,26 @@ fk_status plan_delta_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     return plan_delta_scan(a, act, l);
 }
 
+// qk, decay, beta, v, state, o, work   (parameters of fusekit_delta_scan, bf16)
+fk_status plan_delta_chunk_d(const Dispatch& d, Launch* l, SlotRW* rw) {
+    DeltaChunkArgs a;
+    memset(&a, 0, sizeof(a));
+    a.rows = d.u("rows", 1); a.heads = d.u("heads"); a.kv_heads = d.u("kv_heads"); a.dim_ld = d.u("dim_ld"); a.vdim_ld = d.u("vdim_ld"); a.state_ld = d.u("state_ld");
+    a.ldx = d.u("ldx"); a.ldb = d.u("ldb", a.heads);
+    const uint64_t nk = (uint64_t)a.kv_heads * a.dim_ld, nd = (uint64_t)a.heads * a.dim_ld, nv = (uint64_t)a.heads * a.vdim_ld;
+    if (!a.rows || !nk || !nv || !a.state_ld || a.ldx < nv) return set_error(FK_ERR_INVALID, d.kernel + ": shape parameters missing");
+    SlotCursor s{d, rw};
+    a.qk = s.in<float>(a.rows * nk * 8);
+    a.decay = s.in<float>(a.rows * nd * 4);
+    a.beta = s.in<float>(rows_bytes(a.rows, a.ldb, a.heads, 4));
+    a.v = s.in<uint16_t>(rows_bytes(a.rows, a.ldx, nv, 2));
+    a.state = s.inout<float>(nv * a.state_ld * 4);
+    a.o = s.out<float>(a.rows * nv * 4);
+    a.work = s.inout(delta_chunk_work_bytes(a.rows, a.heads, a.dim_ld, a.vdim_ld));
+    FK_TRY(s.end());
+    return plan_delta_chunk(a, l);
+}
+
 // u, gates, r bias, i bias, lam, state, y, carry   {rows, width, block, ldx, ldy, act}; carry holds 2 * width words per 32 rows
 fk_status plan_lru_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     LruScanArgs a;

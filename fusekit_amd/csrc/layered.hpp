@@ -313,6 +313,22 @@ struct DeltaScanArgs {
 };
 fk_status plan_delta_scan(const DeltaScanArgs& a, uint32_t act, Launch* out);
 
+// The same in chunks of 64 tokens on the matrix cores (bf16); `work`: delta_chunk_work_bytes.
+struct DeltaChunkArgs {
+    const float* qk;
+    const float* decay;
+    const float* beta;
+    const uint16_t* v;
+    float* state;
+    float* o;
+    void* work;
+    uint32_t rows, heads, kv_heads, dim_ld, vdim_ld, state_ld, ldx, ldb;
+};
+constexpr uint32_t kDeltaChunk = 64;
+bool delta_chunk_supported(uint32_t dim_ld, uint32_t vdim_ld);
+uint64_t delta_chunk_work_bytes(uint32_t rows, uint32_t heads, uint32_t dim_ld, uint32_t vdim_ld);
+fk_status plan_delta_chunk(const DeltaChunkArgs& a, Launch* out);
+
 // ---- real-gated linear recurrent unit ----
 // S <- a S + sqrt(1 - a^2) i u, log a = -8 r softplus(lam), r and i sigmoids of block-diagonal products; the output is
 // S times the gate branch, in its place.  `width` counts padded channels.

@@ -23,6 +23,7 @@ from .runtime import Dispatch, arg
 
 FN_RELU2, FN_GELU = 1, 2     # column functions of a product
 LRU_CHUNK = 32
+DELTA_ROWS = 16              # the recurrence goes in chunks from this many rows
 
 
 def pad(n: int, to: int = 64) -> int:
@@ -327,6 +328,8 @@ def scratch(m, f, R: int, act: int, capacity: int, want: Callable[[str, int], No
         want("qk", R * 2 * m.kv_heads * m.dim_ld * 4)
         want("o", R * m.heads * m.vdim_ld * 4)
         want("gate", R * m.heads * m.vdim_ld * e)
+        if act == 16 and native.delta_chunk_supported(m.dim_ld, m.vdim_ld):
+            want("work", native.delta_chunk_work_bytes(R, m.heads, m.dim_ld, m.vdim_ld))
     else:
         want("xbc", R * m.inner * e)
         want("gates", R * 2 * m.inner * 4)
@@ -401,8 +404,9 @@ class JointTasks:
         shape = dict(rows=rows, heads=m.heads, kv_heads=m.kv_heads, dim_ld=m.dim_ld, ldx=X, ldb=m.heads, act=c.act)
         t.append(Dispatch(self._name("delta_prep"),
                           [arg(b["xbc"]), arg(w.vecs[q + "dt_bias"]), arg(w.vecs[q + "A_log"]), arg(b["decays"]), arg(b["beta"]), arg(b["qk"])], dict(shape, dim=m.dim)))
-        t.append(Dispatch(self._name("delta_scan"),
-                          [arg(b["qk"]), arg(b["decays"]), arg(b["beta"]), arg(b["xbc"], None, 2 * nk * e), arg(st["state"]), arg(b["o"])],
+        long = c.act == 16 and c.tiled and rows >= DELTA_ROWS and native.delta_chunk_supported(m.dim_ld, m.vdim_ld)
+        t.append(Dispatch(self._name("delta_chunk" if long else "delta_scan"),
+                          [arg(b["qk"]), arg(b["decays"]), arg(b["beta"]), arg(b["xbc"], None, 2 * nk * e), arg(st["state"]), arg(b["o"])] + ([arg(b["work"])] if long else []),
                           dict(shape, vdim_ld=m.vdim_ld, state_ld=m.state_ld)))
         t.append(Dispatch(self._name("head_norm"), [arg(b["o"]), arg(b["gate"]), arg(w.vecs[q + "norm"]), u("v")],
                           dict(rows=rows, heads=m.heads, dim=m.vdim, ld=m.vdim_ld, ldx=nv, ldz=nv, ldy=col.width, eps=c.eps, act=c.act)))

@@ -1,12 +1,15 @@
-"""Prefill and decode throughput of the layer-list decoder (Pusavik) at sizes that resemble a real model's layers, beside
-the mixture-of-experts decoder with low-rank keys at equal size (`python bench.py --workload pusavik`).
+"""Prefill and decode throughput of the layer-list decoder at sizes that resemble a real model's layers, beside the closest
+other model at equal size: Pusavik beside the mixture-of-experts decoder with low-rank keys (`python bench.py --workload
+pusavik`), Fumotar beside Pusavik with one expert, which is a dense feed-forward (`--workload fumotar`).
 
-Both models have the same number of layers, width, heads, experts, active experts and vocabulary; the layer-list model
+Pusavik and the mixture-of-experts decoder have the same number of layers, width, heads, experts, active experts and vocabulary; the layer-list model
 alternates latent attention and Mamba-2 mixers and keeps bf16 matrices, the other one has attention in every layer and
-int4 matrices.  Random weights, generated in HBM.  Per launch shape: algorithmic bytes or flops over the average launch
+int4 matrices.  Fumotar and its Pusavik have the same layers, width, vocabulary and number of feed-forward weights, and bf16
+matrices both.  Random weights, generated in HBM.  Per launch shape: algorithmic bytes or flops over the average launch
 time in a chain of dependent launches with distinct weights (HIP events), as a fraction of the published peaks."""
 from __future__ import annotations
 
+import math
 import time
 from typing import Dict, List
 
@@ -21,6 +24,36 @@ SIZES = {
     "4k": dict(width=4096, heads=32, kv_rank=512, q_rank=1536, window=1024, ssm_heads=128, groups=8, experts=64, identity=8, top=8, ff=2048, vocab=102400),
 }
 LAYERS = 8
+
+# width, ff, attention heads / kv heads, delta heads, block and number of the linear recurrence, vocab; heads are 128 wide
+JOINT_SIZES = {
+    "1k": dict(width=1024, ff=4096, heads=8, kv_heads=2, delta_heads=8, blocks=8, rank=64, vocab=32768),
+    "2k": dict(width=2048, ff=8192, heads=16, kv_heads=4, delta_heads=16, blocks=8, rank=128, vocab=102400),
+    "4k": dict(width=4096, ff=16384, heads=32, kv_heads=8, delta_heads=32, blocks=16, rank=128, vocab=102400),
+}
+
+
+def joint_config(s: dict, rows_per_pass: int = 2048, capacity: int = 4096):
+    from .joint_layers import CausalAttention, ChannelDelta, DenseMlp, RgLru, RotaryScaling
+    from .layer_decoder import Layer, LayerConfig, PairTable
+    att = CausalAttention(heads=s["heads"], kv_heads=s["kv_heads"], dim=128, scale=128 ** -0.5, rot_base=1e5, rot_dims=128,
+                          rot_scaling=RotaryScaling(factor=4.0, original=4096, fast=32.0, slow=1.0))
+    dlt = ChannelDelta(heads=s["delta_heads"], kv_heads=s["delta_heads"], dim=128, vdim=128, conv=4, decay_rank=s["rank"], gate_rank=s["rank"])
+    lru = RgLru(width=s["width"], blocks=s["blocks"], conv=4)
+    mlp = DenseMlp(s["ff"])
+    return LayerConfig(width=s["width"], vocab=s["vocab"], layers=[Layer((dlt, lru, att)[i % 3], mlp) for i in range(LAYERS)], rows_per_pass=rows_per_pass,
+                       capacity=capacity, design="Fumotar", layer_norm=True, tied=True, join=True, loop_start=0, loop_stop=LAYERS, loop_times=1,
+                       pairs=PairTable(buckets=65535, mul_prev=31, mul_cur=17))
+
+
+def like_joint_config(s: dict, rows_per_pass: int = 2048):
+    """The layer-list model of the other design with the same width, layers and feed-forward weights."""
+    from .layer_decoder import Experts, LatentAttention, Layer, LayerConfig, Mamba2
+    w = s["width"]
+    lat = LatentAttention(heads=s["heads"], dim=128, rot_dim=64, vdim=128, kv_rank=min(512, w // 4), q_rank=w // 2, window=1024, scale=192 ** -0.5, rot_base=1e5, rot_dims=64)
+    ssm = Mamba2(heads=w // 32, vdim=64, state=128, groups=max(4, w // 512), conv=4, norm_groups=max(4, w // 512))
+    moe = Experts(experts=1, identity=0, top=1, ff=s["ff"] * 2 // 3 // 64 * 64)
+    return LayerConfig(width=w, vocab=s["vocab"], layers=[Layer(lat if i % 3 == 2 else ssm, moe) for i in range(LAYERS)], rows_per_pass=rows_per_pass)
 
 
 def layer_config(s: dict, rows_per_pass: int = 2048):
@@ -50,10 +83,11 @@ def label(t) -> str:
     f = _family(t.kernel)
     if f == "layer_jobs":
         parts = [f"{int(p[f'g{i}_n'])}x{int(p[f'g{i}_k'])}" for i in (0, 1) if f"g{i}_n" in p]
-        parts += [n for n, k in (("gate/up", "pair_n"), ("choice", "route_outputs"), ("cache row", "store_rank"), ("state step", "scan_heads")) if p.get(k)]
+        parts += [n for n, k in (("gate/up", "pair_n"), ("choice", "route_outputs"), ("cache row", "store_rank"), ("state step", "scan_heads"),
+                                 ("delta step", "delta_heads"), ("lru step", "lru_width")) if p.get(k)]
         return "jobs: " + " | ".join(parts)
     if f == "layer_out":
-        return "layer out" + (" (o + down)" if p.get("ko") else " (down)")
+        return "layer out" + (" %dx%d" % (p["n"], p["ko"]) if not p.get("top") else " (o + down)" if p.get("ko") else " (down)")
     if f in ("dense", "experts"):
         extra = " x%d heads" % p["batch"] if p.get("batch", 1) > 1 else ""
         return f"{f} {int(p['n'])}x{int(p['k'])}{extra}" + (" pair" if p.get("pair") else "")
@@ -83,8 +117,58 @@ def measure(rt, tasks, work, reps: int = 64) -> List[dict]:
     return sorted(out, key=lambda e: -e["avg_us"] * e["count"])
 
 
+def joint_work(c, rows: int, ctx: int):
+    """Algorithmic bytes and flops of a task of a model of joint layers."""
+    def work(t):
+        p, f = t.params, _family(t.kernel)
+        m = lambda *names: math.prod(p[n] for n in names)
+        if rows == 1:
+            w = {"layer_out": lambda: p["n"] * p["ko"] * 2,
+                 "layer_jobs": lambda: (p["g0_n"] * p["g0_k"] * 2 if "g0_n" in p else 0)
+                 + (m("delta_heads", "delta_vdim_ld", "delta_state_ld") * 8 + m("delta_heads", "delta_dim_ld", "delta_rank_ld") * 2 if p.get("delta_heads") else 0)
+                 + (m("lru_width", "lru_block") * 4 + p["lru_width"] * 8 if p.get("lru_width") else 0),
+                 "sdpa_decode": lambda: ctx * m("n_kv", "head_dim") * 4, "qk_store": lambda: (p["heads"] + 3 * p["kv_heads"]) * p["dim_ld"] * 4,
+                 "embed_rows": lambda: p["width"] * 8}.get(f)
+            return (w() if w else 0), 0
+        fl = {"dense": lambda: 2.0 * m("rows", "n", "k") * p.get("batch", 1),
+              "sdpa_prefill": lambda: 2.0 * rows * (rows + 1.0) * m("n_heads", "head_dim"),
+              # per token and head: keys against keys and queries of the chunk, its triangular solve, three products with the state
+              "delta_scan": lambda: 2.0 * rows * p["heads"] * 3 * m("dim_ld", "vdim_ld"),
+              "delta_chunk": lambda: 2.0 * rows * p["heads"] * (3 * m("dim_ld", "vdim_ld") + 64 * (1.5 * p["dim_ld"] + p["vdim_ld"]))}.get(f)
+        b = {"residual_norm": lambda: rows * c.width * (4 * 3 + 2), "ssm_conv": lambda: rows * p["channels"] * 4,
+             "embed_rows": lambda: rows * c.width * (2 * 2 + 4 + 2), "qk_store": lambda: rows * (p["heads"] + 1.5 * p["kv_heads"]) * p["dim_ld"] * 4,
+             "delta_prep": lambda: rows * (p["kv_heads"] * p["dim_ld"] * 12 + p["heads"] * p["dim_ld"] * 8),
+             "head_norm": lambda: rows * m("heads", "ld") * 8, "lru_scan": lambda: rows * p["width"] * 14,
+             "delta_scan": lambda: rows * (p["kv_heads"] * p["dim_ld"] * 8 + p["heads"] * (p["dim_ld"] * 4 + p["vdim_ld"] * 6)),
+             "delta_chunk": lambda: rows * (p["kv_heads"] * p["dim_ld"] * 8 + p["heads"] * (p["dim_ld"] * 4 + p["vdim_ld"] * 6))}.get(f)
+        return (b() if b else 0), (fl() if fl else 0)
+
+    return work
+
+
+def joint_token_bytes(c, ctx: int) -> int:
+    """Algorithmic HBM bytes of one decoded token of a model of joint layers."""
+    from .joint_layers import Columns
+    n, state = c.vocab * c.width + (2 * c.width * c.width * c.loop_times if c.looped and c.join else 0), 0
+    for i, _ in c.runs():
+        m = c.layers[i].mixer
+        col = Columns(m, c.layers[i].mlp)
+        n += (col.rows + col.ko) * c.width
+        if m.kind == "attention":
+            state += ctx * m.kv_heads * m.dim_ld * 4
+        elif m.kind == "channel_delta":
+            n += m.heads * (m.dim_ld * m.decay_rank + m.vdim_ld * m.gate_rank)
+            state += 2 * m.heads * m.vdim_ld * m.state_ld * 4
+        else:
+            n += 2 * m.inner * m.block_ld
+            state += 2 * m.inner * 4
+    return int(n * 2 + state)
+
+
 def layer_work(c, rows: int, ctx: int):
     """Algorithmic bytes (decode) or flops (portions) of a task of the layer-list model."""
+    if any(l.joint for l in c.layers):
+        return joint_work(c, rows, ctx)
     lat = next(l.mixer for l in c.layers if l.mixer.kind == "latent_attention")
     ssm = next(l.mixer for l in c.layers if l.mixer.kind == "mamba2")
     moe = c.layers[0].mlp
@@ -118,6 +202,8 @@ def layer_work(c, rows: int, ctx: int):
 
 def token_bytes(c, ctx: int) -> int:
     """Algorithmic HBM bytes of one decoded token: the matrices it touches, the window's latents, the states."""
+    if any(l.joint for l in c.layers):
+        return joint_token_bytes(c, ctx)
     n = c.vocab * c.width
     state = 0
     for i, _ in c.runs():
@@ -133,20 +219,20 @@ def token_bytes(c, ctx: int) -> int:
     return int(n * 2 + state)
 
 
-def bench_layer(size: str, ctx: int = 1024, steps: int = 128, kernels: bool = True) -> dict:
+def bench_layer(size: str, ctx: int = 1024, steps: int = 128, kernels: bool = True, config=None) -> dict:
     from . import native as fk
     from .layer_decoder import LayerRuntime, LayerWeights
-    s = SIZES[size]
-    c = layer_config(s)
+    c = config or layer_config(SIZES[size])
     w = LayerWeights.random_init(c, seed=1)
     rt = LayerRuntime(c, w)
     rng = np.random.Generator(np.random.PCG64(0))
-    out: dict = dict(model="Pusavik %s: %d layers, width %d, %.2f GB of bf16 weights" % (size, LAYERS, c.width, w.nbytes() / 1e9))
+    out: dict = dict(model="%s %s: %d layers, width %d, %.2f GB of bf16 weights" % (c.design, size, LAYERS, c.width, w.nbytes() / 1e9))
     for rows in (512, 2048):
         toks = rng.integers(0, c.vocab, rows).astype(np.uint32)
         rt.reset()
         rt.tokens.upload(toks)
         rt.row_offset.upload(np.zeros(1, np.uint32))
+        rt.row_kv.upload(np.array([rows], np.uint32))
         tasks = rt.rows_tasks(rows)
         g = rt.d.build_decode_graph(tasks, False)
         rt.d.execute_graph(g)
@@ -236,6 +322,11 @@ def bench_moe(size: str, ctx: int = 1024, steps: int = 128) -> dict:
     rt2.kv_len.upload(np.array([ctx], np.uint32))
     out["decode"]["by_launch"] = measure(rt2, rt2.tasks, work)
     return out
+
+
+def run_joint(sizes: List[str], kernels: bool = True) -> dict:
+    return {s: dict(fumotar=bench_layer(s, kernels=kernels, config=joint_config(JOINT_SIZES[s])),
+                    pusavik=bench_layer(s, kernels=kernels, config=like_joint_config(JOINT_SIZES[s]))) for s in sizes}
 
 
 def run(sizes: List[str], kernels: bool = True) -> dict:

@@ -185,6 +185,11 @@ class LayerConfig:
         return self.capacity if any(l.mixer.kind == "attention" for l in self.layers) else None
 
     @property
+    def padded_lookup(self) -> bool:
+        """Whether token rows come from tables in padded rows (those of a tied head, pairs, copies for a join)."""
+        return bool(self.pairs or self.tied or (self.looped and self.join))
+
+    @property
     def looped(self) -> bool:
         return self.loop_stop > self.loop_start
 
@@ -357,7 +362,10 @@ class LayerWeights:
             self._matrix("head", get("embed"))
             self.mats["embed"] = self.mats["head"]
         else:
-            self._dense("embed", DeviceBuffer.from_numpy(get("embed")), c.vocab, c.width)
+            if c.padded_lookup:
+                self._matrix("embed", get("embed"))
+            else:
+                self._dense("embed", DeviceBuffer.from_numpy(get("embed")), c.vocab, c.width)
             self._matrix("head", get("head"))
         if c.pairs:
             self._matrix("bigram", get("bigram"))
@@ -917,7 +925,7 @@ class LayerRuntime(JointTasks):
     def _embed_task(self, tokens, off, rows: int) -> Dispatch:
         """Embedding rows; with a join their copies beside the place of the stream."""
         c, b, W, D = self.cfg, self.buf, self.w.mats["embed"], pad(self.cfg.width)
-        if not c.pairs and not c.tied and not (c.looped and c.join):
+        if not c.padded_lookup:
             return Dispatch(self._name("embed_lookup_decode"), [tokens, arg(W.w), arg(b["x"])],
                             dict(bits=16, hidden=c.width, vocab=c.vocab, output_scale=c.embed_scale, rows=rows, out_bits=32, x_row_stride=D))
         a, p = [tokens, arg(W.w)], dict(rows=rows, width=c.width, vocab=c.vocab, ldw=W.k, ld=D, scale=c.embed_scale, act=c.act)

@@ -650,6 +650,17 @@ def latent_split_supported(rank_ld: int, ldc: int) -> bool:
     return bool(lib.fk_latent_split_supported(C.c_uint32(rank_ld), C.c_uint32(ldc)))
 
 
+def delta_chunk_supported(dim_ld: int, vdim_ld: int) -> bool:
+    """Is there a chunked matrix-core form of the gated delta rule of these padded head widths?"""
+    return bool(lib.fk_delta_chunk_supported(C.c_uint32(dim_ld), C.c_uint32(vdim_ld)))
+
+
+def delta_chunk_work_bytes(rows: int, heads: int, dim_ld: int, vdim_ld: int) -> int:
+    f = lib.fk_delta_chunk_work_bytes
+    f.restype = C.c_uint64
+    return f(C.c_uint32(rows), C.c_uint32(heads), C.c_uint32(dim_ld), C.c_uint32(vdim_ld))
+
+
 def ssm_chunk_supported(heads: int, vdim: int, state: int) -> bool:
     """Whether a state-space mixer's widths have the chunked matrix-core form."""
     return bool(lib.fk_ssm_chunk_supported(C.c_uint32(heads), C.c_uint32(vdim), C.c_uint32(state)))

@@ -661,6 +661,11 @@ fk_status fk_xcd_check(void *workspace, fk_stream s);
 int fk_latent_split_supported(uint32_t rank_ld, uint32_t ldc);
 int fk_latent_prefill_supported(uint32_t dim_ld, uint32_t rot_ld, uint32_t vdim_ld);
 int fk_ssm_chunk_supported(uint32_t heads, uint32_t p, uint32_t n);
+/* Joint layers (mixer and dense feed-forward read one norm): families fusekit_embed_rows, _head_norm, _qk_store, _gqa_rows,
+ * _delta_prep, _delta_scan, _lru_scan (any widths, bf16 or fp32), fusekit_delta_chunk (bf16 portions on the matrix cores;
+ * padded key and value width, and the bytes of its workspace), and column functions of fusekit_dense. */
+int fk_delta_chunk_supported(uint32_t dim_ld, uint32_t vdim_ld);
+uint64_t fk_delta_chunk_work_bytes(uint32_t rows, uint32_t heads, uint32_t dim_ld, uint32_t vdim_ld);
 
 /* ---- dispatcher: replaces `_fusekit_runtime_native` ------------------------
  *
