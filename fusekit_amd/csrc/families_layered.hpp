@@ -244,7 +244,7 @@ fk_status plan_delta_scan_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     return plan_delta_scan(a, act, l);
 }
 
-// qk, decay, beta, v, state, o, work   (parameters of fusekit_delta_scan, bf16)
+// qk, decay, beta, v, state, o (rows in whole 64s), work   (parameters of fusekit_delta_scan, bf16)
 fk_status plan_delta_chunk_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     DeltaChunkArgs a;
     memset(&a, 0, sizeof(a));
@@ -258,7 +258,7 @@ fk_status plan_delta_chunk_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     a.beta = s.in<float>(rows_bytes(a.rows, a.ldb, a.heads, 4));
     a.v = s.in<uint16_t>(rows_bytes(a.rows, a.ldx, nv, 2));
     a.state = s.inout<float>(nv * a.state_ld * 4);
-    a.o = s.out<float>(a.rows * nv * 4);
+    a.o = s.out<float>((a.rows + kDeltaChunk - 1) / kDeltaChunk * kDeltaChunk * nv * 4);
     a.work = s.inout(delta_chunk_work_bytes(a.rows, a.heads, a.dim_ld, a.vdim_ld));
     FK_TRY(s.end());
     return plan_delta_chunk(a, l);

@@ -313,7 +313,7 @@ struct DeltaScanArgs {
 };
 fk_status plan_delta_scan(const DeltaScanArgs& a, uint32_t act, Launch* out);
 
-// The same in chunks of 64 tokens on the matrix cores (bf16); `work`: delta_chunk_work_bytes.
+// The same in chunks of 64 tokens on the matrix cores (bf16); `work`: delta_chunk_work_bytes; o has whole chunks of rows.
 struct DeltaChunkArgs {
     const float* qk;
     const float* decay;

@@ -326,7 +326,7 @@ def scratch(m, f, R: int, act: int, capacity: int, want: Callable[[str, int], No
         want("xbc", R * pad(m.channels) * e)
         want("decays", R * m.heads * m.dim_ld * 4)
         want("qk", R * 2 * m.kv_heads * m.dim_ld * 4)
-        want("o", R * m.heads * m.vdim_ld * 4)
+        want("o", pad(R) * m.heads * m.vdim_ld * 4)
         want("gate", R * m.heads * m.vdim_ld * e)
         if act == 16 and native.delta_chunk_supported(m.dim_ld, m.vdim_ld):
             want("work", native.delta_chunk_work_bytes(R, m.heads, m.dim_ld, m.vdim_ld))
