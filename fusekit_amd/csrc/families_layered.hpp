@@ -45,7 +45,7 @@ uint64_t rows_bytes(uint64_t rows, uint64_t ld, uint64_t width, uint64_t elem) {
 
 // x, [mix: has_mix], [routes, weight, index, prev: top > 0], [step: has_step], [copy: ldcopy > 0], [w1, [b1: layer_norm], h1:
 // has_h1], [w2, h2: has_h2]
-//   {rows, width, ld, ldcopy, act, eps, top, experts}
+//   {rows, width, ld, ldcopy, act, eps, top, experts, mix_parts=1}
 fk_status plan_residual_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     ResidualNormArgs a;
     memset(&a, 0, sizeof(a));
@@ -56,7 +56,8 @@ fk_status plan_residual_norm_d(const Dispatch& d, Launch* l, SlotRW* rw) {
     const uint64_t x4 = (uint64_t)a.rows * a.ldx * 4, xa = (uint64_t)a.rows * a.ldx * act_bytes(act);
     SlotCursor s{d, rw};
     a.x = s.inout<float>(x4);
-    if (d.u("has_mix")) a.mix = s.in<float>(x4);
+    a.parts = d.u("mix_parts", 1);
+    if (d.u("has_mix")) a.mix = s.in<float>(x4 * a.parts);
     if (a.top) {
         a.routes = s.in(xa * a.top);
         a.weight = s.in<float>((uint64_t)a.rows * a.top * 4);

@@ -381,12 +381,27 @@ __device__ __forceinline__ float conv_token(const uint16_t* u, const uint16_t* w
     const uint16_t raw = u[ch];
     const uint16_t* k = w + (size_t)ch * taps;
     float v = b ? bf16_bits_to_f32(b[ch]) : 0.f;
-    for (uint32_t i = 0; i + 1u < taps; ++i) {
-        const uint32_t back = taps - 1u - i;
-        if (back <= pos) v = fmaf(bf16_bits_to_f32(k[i]), bf16_bits_to_f32(hist[(size_t)((pos - back) % taps) * ldh + ch]), v);
+    const uint32_t slot = pos % taps;
+    if (taps <= 4u) {   // every request ahead of the first use; rows before the start are multiplied away
+        uint16_t past[3], w3[3];
+#pragma unroll
+        for (uint32_t i = 0; i < 3; ++i) {
+            const uint32_t back = i + 1u, at = slot >= back ? slot - back : slot + taps - back;
+            const bool in = back < taps;
+            past[i] = hist[(size_t)(in ? at : 0u) * ldh + ch];
+            w3[i] = k[in ? taps - 1u - back : 0u];
+        }
+#pragma unroll
+        for (uint32_t i = 3; i-- > 0;)
+            if (i + 1u < taps && i + 1u <= pos) v = fmaf(bf16_bits_to_f32(w3[i]), bf16_bits_to_f32(past[i]), v);
+    } else {
+        for (uint32_t i = 0; i + 1u < taps; ++i) {
+            const uint32_t back = taps - 1u - i;
+            if (back <= pos) v = fmaf(bf16_bits_to_f32(k[i]), bf16_bits_to_f32(hist[(size_t)((pos - back) % taps) * ldh + ch]), v);
+        }
     }
     v = fmaf(bf16_bits_to_f32(k[taps - 1u]), bf16_bits_to_f32(raw), v);
-    if (write) hist[(size_t)(pos % taps) * ldh + ch] = raw;
+    if (write) hist[(size_t)slot * ldh + ch] = raw;
     return v;
 }
 
@@ -407,6 +422,7 @@ __device__ void delta_step(const DeltaJob& a, uint32_t h, uint32_t pt, float* sm
         float z = 0.f;
         if (d < a.dim_ld) {
             const uint16_t* row = a.a2 + ((size_t)h * a.dim_ld + d) * a.rank_ld;
+#pragma unroll 4
             for (uint32_t c = (tid & 3u) * 8u; c < a.rank_ld; c += 32u)
                 z = dot8(*reinterpret_cast<const ld_u32x4_t*>(row + c), *reinterpret_cast<const ld_u32x4_t*>(a.a1 + c), z);
         }
@@ -461,11 +477,12 @@ __device__ void delta_step(const DeltaJob& a, uint32_t h, uint32_t pt, float* sm
     if (nl == 0) a.o[(size_t)h * a.vdim_ld + p0 + pl] = fmaf(kq, u, sq);
 }
 
-// One token of some channels of one diagonal block: the convolution of the whole block, then per channel its two gates.
-__device__ void lru_token(const LruJob& a, uint32_t part, uint32_t sub, uint16_t* xs) {
+// One token of some channels of one diagonal block: the convolution of the whole block, their gates, then a thread per
+// channel, whose state and constants have been on their way since the start.
+__device__ void lru_token(const LruJob& a, uint32_t part, uint32_t sub, uint16_t* xs, float* gates) {
     const uint32_t tid = threadIdx.x, lane = tid & 63u, wave = tid >> 6, pos = *a.offset;
     const uint32_t c0 = sub * kLruRows, count = a.block - c0 < kLruRows ? a.block - c0 : kLruRows;
-    const uint32_t turns = wave < count ? (count - wave + 3u) / 4u : 0u;
+    const uint32_t turns = wave < count ? (count - wave + 3u) / 4u : 0u, mine = part * a.block + c0 + (tid < count ? tid : 0u);
     const uint16_t *wr = a.gates + (size_t)part * 2u * a.block * a.block, *wi = wr + (size_t)a.block * a.block;
     auto rows = [&](uint32_t t, const uint16_t*& w0, const uint16_t*& w1) __attribute__((always_inline)) {
         const uint32_t r = wave + t * 4u, rr = c0 + (r < count ? r : count - 1u);
@@ -474,20 +491,27 @@ __device__ void lru_token(const LruJob& a, uint32_t part, uint32_t sub, uint16_t
     };
     PairStream<decltype(rows)> st(rows, a.block, turns, lane);
     st.start();
+    const float rb = bf16_bits_to_f32(a.rb[mine]), ib = bf16_bits_to_f32(a.ib[mine]), y = act_load(a.y + mine);
+    const uint16_t lam = a.lam[mine];
+    float S = a.state[mine];
     for (uint32_t i = tid; i < a.block; i += kJobBlock)
         act_store(xs + i, conv_token(a.u, a.w, a.b, a.hist, part * a.block + i, a.taps, a.ldh, pos, i - c0 < count));
     __syncthreads();
-    if (!turns) return;
-    st.run(xs, [&](uint32_t t, float zr, float zi) __attribute__((always_inline)) {
-        const uint32_t r = wave + t * 4u;
-        if (lane != 0 || r >= count) return;
-        const uint32_t c = part * a.block + c0 + r;
-        float decay, add;
-        lru_step(zr + bf16_bits_to_f32(a.rb[c]), zi + bf16_bits_to_f32(a.ib[c]), lru_rate(a.lam[c]), act_load(xs + c0 + r), decay, add);
-        const float S = fmaf(decay, a.state[c], add);
-        a.state[c] = S;
-        act_store(a.y + c, S * act_load(a.y + c));
-    });
+    if (turns)
+        st.run(xs, [&](uint32_t t, float zr, float zi) __attribute__((always_inline)) {
+            const uint32_t r = wave + t * 4u;
+            if (lane == 0 && r < count) {
+                gates[r] = zr;
+                gates[kLruRows + r] = zi;
+            }
+        });
+    __syncthreads();
+    if (tid >= count) return;
+    float decay, add;
+    lru_step_fast(gates[tid] + rb, gates[kLruRows + tid] + ib, lru_rate(lam), act_load(xs + c0 + tid), decay, add);
+    S = fmaf(decay, S, add);
+    a.state[mine] = S;
+    act_store(a.y + mine, S * y);
 }
 
 __global__ __launch_bounds__(kJobBlock) void layer_jobs_kernel(const LayerJobsArgs a) {
@@ -577,7 +601,7 @@ __global__ __launch_bounds__(kJobBlock) void layer_jobs_kernel(const LayerJobsAr
     }
     if (b - a.lru.first < a.lru.blocks) {
         const uint32_t local = b - a.lru.first;
-        lru_token(a.lru, local / a.lru.blocks_per_part, local % a.lru.blocks_per_part, lds);
+        lru_token(a.lru, local / a.lru.blocks_per_part, local % a.lru.blocks_per_part, lds, red);
     }
 }
 

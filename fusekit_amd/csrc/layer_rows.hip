@@ -23,7 +23,13 @@ __global__ __launch_bounds__(kRowBlock) void residual_norm_kernel(const Residual
     for (uint32_t c = threadIdx.x * 4u; c < a.ldx; c += kRowBlock * 4u) {
         float4 v = *reinterpret_cast<const float4*>(x + c);
         float4 add = make_float4(0.f, 0.f, 0.f, 0.f);
-        if (mix) add = *reinterpret_cast<const float4*>(mix + c);
+        if (mix) {
+            add = *reinterpret_cast<const float4*>(mix + c);
+            for (uint32_t p = 1; p < a.parts; ++p) {
+                const float4 m = *reinterpret_cast<const float4*>(mix + (size_t)p * a.rows * a.ldx + c);
+                add.x += m.x; add.y += m.y; add.z += m.z; add.w += m.w;
+            }
+        }
         if (routes) {
             float4 f = make_float4(0.f, 0.f, 0.f, 0.f);
             for (uint32_t s = 0; s < a.top; ++s) {

@@ -18,7 +18,7 @@ constexpr uint32_t kRowPad = 64;
 // norms where a bias is given.
 struct ResidualNormArgs {
     float* x;               // [rows, ldx]
-    const float* mix;       // [rows, ldx] or null
+    const float* mix;       // [parts][rows, ldx] (a product in parts of its sum) or null
     const void* routes;     // [rows * top, ldx] expert outputs (act) or null
     const float* weight;    // [rows, top] route weights
     const uint32_t* index;  // [rows, top] chosen experts; >= experts: the identity, whose output is prev
@@ -30,7 +30,7 @@ struct ResidualNormArgs {
     void* h1;               // [rows, ldx] (act)
     void* h2;
     void* copy;             // [rows, ldcopy] (act): the new x itself, or null
-    uint32_t rows, width, ldx, top, experts, ldcopy;
+    uint32_t rows, width, ldx, top, experts, ldcopy, parts;
     float eps;
 };
 fk_status plan_residual_norm(const ResidualNormArgs& a, uint32_t act, Launch* out);

@@ -39,7 +39,8 @@ struct LruColumn {
             for (uint32_t e = 0; e < kLruAhead; ++e) {
                 if (r + e < r1) {
                     float decay, add;
-                    lru_step(rv[e] + rb, iv[e] + ib, rate, uv[e], decay, add);
+                    if (sizeof(T) == 2) lru_step_fast(rv[e] + rb, iv[e] + ib, rate, uv[e], decay, add);
+                    else lru_step(rv[e] + rb, iv[e] + ib, rate, uv[e], decay, add);
                     f(r + e, decay, add);
                 }
                 fetch(e, r + e + kLruAhead);

@@ -180,6 +180,16 @@ class Columns:
                 self.fns = dict(fn=FN_GELU, fn_begin=self.out, fn_end=self.up, fn2=FN_RELU2, fn2_begin=self.up)
 
 
+def out_parts(rows: int, n: int, k: int) -> int:
+    """Parts of the sum that the product [rows, k] . [n, k] is formed in, side by side: a long sum over few output tiles would
+    leave most compute units without work.  The rows form (8 rows or fewer) has a wave per column and needs none."""
+    if rows <= 8:
+        return 1
+    tiles = -(-n // 64) * (1 if rows <= 32 else -(-rows // 64))
+    want = 8 if rows <= 32 or tiles <= 64 else 4 if tiles <= 128 else 2 if tiles <= 256 else max(1, 2048 // tiles)
+    return next(p for p in (8, 4, 2, 1) if p <= want and (p == 1 or (k % (64 * p) == 0 and k >= 512 * p)))
+
+
 # ---------------------------------------------------------------- checkpoint
 
 def mixer_shapes(m, p: str, D: int) -> Dict[str, Tuple[int, ...]]:
@@ -366,7 +376,14 @@ class JointTasks:
         self._dense(t, arg(b["h1"]), w.mats[q + "in"], arg(b["u"]), rows, D, col.width, base=base, tail=tail, **more)
         u = lambda name: arg(b["u"], None, col.at[name] * e)
         {"attention": self._attention_tasks, "channel_delta": self._delta_tasks, "rglru": self._lru_tasks}[m.kind](t, m, q, col, run, rows, off, kv_len, u)
-        self._dense(t, arg(b["u"], None, col.out * e), w.mats[p + "out"], arg(b["mix"]), rows, col.width, D, y32=True)
+        W, parts = w.mats[p + "out"], self._out_parts(i, rows)
+        k = W.k // parts
+        self._dense(t, arg(b["u"], None, col.out * e), W, arg(b["mix"]), rows, col.width, D, y32=True, **(dict(batch=parts, k=k, xb=k, wb=k, yb=rows * D) if parts > 1 else {}))
+
+    def _out_parts(self, layer: int, rows: int) -> int:
+        c = self.cfg
+        l = c.layers[layer]
+        return out_parts(rows, c.width, Columns(l.mixer, l.mlp).ko) if l.joint and c.act == 16 and c.tiled else 1
 
     def _qk_store(self, m, q: str, col: Columns, run: int, rows: int, off) -> Dispatch:
         c, w, b, st = self.cfg, self.w, self.buf, self.state.entries[run]

@@ -134,13 +134,16 @@ def joint_work(c, rows: int, ctx: int):
               "sdpa_prefill": lambda: 2.0 * rows * (rows + 1.0) * m("n_heads", "head_dim"),
               # per token and head: keys against keys and queries of the chunk, its triangular solve, three products with the state
               "delta_scan": lambda: 2.0 * rows * p["heads"] * 3 * m("dim_ld", "vdim_ld"),
-              "delta_chunk": lambda: 2.0 * rows * p["heads"] * (3 * m("dim_ld", "vdim_ld") + 64 * (1.5 * p["dim_ld"] + p["vdim_ld"]))}.get(f)
+              "delta_chunk": lambda: 2.0 * rows * p["heads"] * (3 * m("dim_ld", "vdim_ld") + 64 * (3 * p["dim_ld"] + 2 * p["vdim_ld"]) / 2)}.get(f)
         b = {"residual_norm": lambda: rows * c.width * (4 * 3 + 2), "ssm_conv": lambda: rows * p["channels"] * 4,
              "embed_rows": lambda: rows * c.width * (2 * 2 + 4 + 2), "qk_store": lambda: rows * (p["heads"] + 1.5 * p["kv_heads"]) * p["dim_ld"] * 4,
              "delta_prep": lambda: rows * (p["kv_heads"] * p["dim_ld"] * 12 + p["heads"] * p["dim_ld"] * 8),
              "head_norm": lambda: rows * m("heads", "ld") * 8, "lru_scan": lambda: rows * p["width"] * 14,
              "delta_scan": lambda: rows * (p["kv_heads"] * p["dim_ld"] * 8 + p["heads"] * (p["dim_ld"] * 4 + p["vdim_ld"] * 6)),
-             "delta_chunk": lambda: rows * (p["kv_heads"] * p["dim_ld"] * 8 + p["heads"] * (p["dim_ld"] * 4 + p["vdim_ld"] * 6))}.get(f)
+             # besides: per chunk the operands of its sequential part, written and read once
+             "delta_chunk": lambda: rows * (p["kv_heads"] * p["dim_ld"] * 8 + p["heads"] * (p["dim_ld"] * 4 + p["vdim_ld"] * 6))
+             + 2 * rows * p["heads"] * (p["dim_ld"] * 12 + p["vdim_ld"] * 4 + 64 * 4),
+             "dense": lambda: rows * p["n"] * p["batch"] * 4 + m("n", "k", "batch") * 2 + m("rows", "k", "batch") * 2 if p.get("batch", 1) > 1 and p["n"] == 2 * p["k"] else 0}.get(f)
         return (b() if b else 0), (fl() if fl else 0)
 
     return work

@@ -582,8 +582,10 @@ class LayerRuntime(JointTasks):
             need[name] = max(need.get(name, 0), nbytes + 256)   # slack: padded walks may read past the last row
 
         D = pad(c.width)
-        for n, b in (("x", 4), ("mix", 4), ("h1", e), ("h2", e)):
+        for n, b in (("x", 4), ("h1", e), ("h2", e)):
             want(n, R * D * b)
+        most = {rows: max(self._out_parts(i, rows) for i in range(c.n_layers)) for rows in {R, *range(1, min(R, 2048) + 1)}}
+        want("mix", max(rows * p for rows, p in most.items()) * D * 4)
         if c.looped and c.join:
             want("cat", R * 2 * D * e)
             want("x2", D * 4)
@@ -665,8 +667,9 @@ class LayerRuntime(JointTasks):
                y32: bool = False, **more) -> None:
         """y = x . W[n0 : n0 + n]^T."""
         n = W.n - n0 if n is None else n
+        k = more.pop("k", W.k)      # a part of the sum
         t.append(Dispatch(self._name("dense"), [x, arg(W.w, (W.w.nbytes // (2 * W.k) - n0) * W.k * 2, n0 * W.k * 2)] + more.pop("base", []) + [y] + more.pop("tail", []),
-                          dict(rows=rows, n=n, k=W.k, ldx=ldx, ldw=W.k, ldy=ldy, y32=int(y32), act=self.cfg.act, **more)))
+                          dict(rows=rows, n=n, k=k, ldx=ldx, ldw=W.k, ldy=ldy, y32=int(y32), act=self.cfg.act, **more)))
 
     def _norm_tasks(self, t, run: int, rows: int, first: bool) -> None:
         """The residual sum behind run - 1 (nothing yet when `first`), the vector ahead of a loop pass and the norms
@@ -686,7 +689,7 @@ class LayerRuntime(JointTasks):
 
         if not first:
             a.append(arg(b["mix"]))
-            p["has_mix"] = 1
+            p.update(has_mix=1, mix_parts=self._out_parts(self.runs[run - 1][0], rows))
             f = c.layers[self.runs[run - 1][0]].experts
             if f:
                 a += [arg(b["eo"]), arg(b["rwt"]), arg(b["ridx"]), arg(b["h2"])]
