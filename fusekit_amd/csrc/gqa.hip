@@ -13,7 +13,8 @@ namespace {
 constexpr int kGqaBlock = 256;
 constexpr uint32_t kGqaWaves = kGqaBlock / kWave, kGqaTile = 64, kMaxRotPairs = 512;
 
-// One block per row: the two mean squares, then every head by a wave.
+// A block forms the two mean squares of its row, then its waves take heads in turn; a row's heads are dealt to gridDim.y
+// blocks (one for a portion, one wave per head for a single row).
 template <typename T>
 __global__ __launch_bounds__(kGqaBlock) void qk_store_kernel(const QkStoreArgs a) {
     __shared__ float red[kGqaWaves + 1], red2[kGqaWaves + 1];
@@ -39,7 +40,7 @@ __global__ __launch_bounds__(kGqaBlock) void qk_store_kernel(const QkStoreArgs a
     }
     const float rq = 1.0f / sqrtf(block_sum<kGqaBlock>(sq, red) / (float)(a.heads * a.dim) + a.eps);
     const float rk = 1.0f / sqrtf(block_sum<kGqaBlock>(sk, red2) / (float)(a.kv_heads * a.dim) + a.eps);
-    for (uint32_t h = wave; h < a.heads + a.kv_heads; h += kGqaWaves) {
+    for (uint32_t h = blockIdx.y * kGqaWaves + wave; h < a.heads + a.kv_heads; h += kGqaWaves * gridDim.y) {
         const bool key = h >= a.heads;
         const uint32_t n = key ? h - a.heads : h;
         const T* src = row + (key ? a.k0 : a.q0) + (size_t)n * a.dim_ld;
@@ -131,7 +132,7 @@ fk_status plan_qk_store(const QkStoreArgs& a, uint32_t act, Launch* out) {
         return set_error(FK_ERR_INVALID, "qk store: bad shape");
     if (a.rot_dims > 2 * kMaxRotPairs) return set_error(FK_ERR_UNSUPPORTED, "qk store: at most 1024 rotated dimensions");
     out->func = act == 16 ? (const void*)&qk_store_kernel<uint16_t> : (const void*)&qk_store_kernel<float>;
-    out->grid = dim3(a.rows, 1, 1);
+    out->grid = dim3(a.rows, a.rows >= 64 ? 1 : (a.heads + a.kv_heads + kGqaWaves - 1) / kGqaWaves, 1);
     out->block = dim3(kGqaBlock, 1, 1);
     out->shmem = 0;
     out->set_args(a);

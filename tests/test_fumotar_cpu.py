@@ -61,6 +61,15 @@ def test_columns_of_a_joint_row(name):
         assert c.rows - c.width == (m.heads if m.kind == "channel_delta" else 0)
 
 
+def test_parts_of_a_long_sum():
+    from fusekit_amd.joint_layers import out_parts
+    for n, k in ((72, 192), (2048, 10240), (4096, 20480), (1024, 64 * 7)):
+        for rows in (1, 8, 9, 32, 33, 64, 500, 2048):
+            p = out_parts(rows, n, k)
+            assert k % (64 * p) == 0 and (p == 1 or k // p >= 512) and (rows > 8 or p == 1)
+    assert out_parts(16, 2048, 10240) == 8 and out_parts(2048, 4096, 20480) == 1
+
+
 def test_spread_rows():
     a = np.arange(12).reshape(6, 2)
     s = spread(a, 2, 4)

@@ -125,6 +125,18 @@ def test_single_far_keys_decide(fk, dim, heads, kv):
         assert_close_bf16(b.run(t, cuts), ref, 0.15)
 
 
+@pytest.mark.parametrize("heads,kv,dim,capacity", [(5, 1, 40, 256), (8, 1, 64, 256), (12, 4, 32, 300), (4, 1, 96, 2500), (3, 3, 128, 2500), (1, 1, 8, 64 * 3), (2, 1, 160, 256)])
+def test_head_groups_and_capacities(fk, heads, kv, dim, capacity):
+    c = model([(att(heads=heads, kv_heads=kv, dim=dim, rot_dims=dim // 2 // 2 * 2, scale=2.0 * dim ** -0.5), mlp()), (att(heads=heads, kv_heads=kv, dim=dim, rot_dims=dim), None)],
+              width=64, capacity=capacity)
+    a, b = Model(c, seed=1), Model(c, seed=1, act=16)
+    t = tokens(c, 190)
+    ref = a.plain(t)
+    for cuts in (None, [1], [130, 1], [17, 2, 70, 9]):
+        assert_close_f32(a.run(t, cuts), ref)
+        assert_close_bf16(b.run(t, cuts), ref)
+
+
 @pytest.mark.parametrize("act", [32, 16])
 def test_state_that_is_kept_for_long(fk, act):
     """Almost no decay: the first tokens still decide after hundreds; a state lost at a portion's edge would show."""
@@ -223,15 +235,23 @@ def test_command_line_artifact_and_trace(fk, tmp_path, capsys, monkeypatch):
     assert len(a) == len(f) == 12
     run("patch", "--model", d)
     art = [json.loads(run("generate", "--model", d, "--artifact", d + "/.fusekit", "--ids", ids, "--max-tokens", "12"))["tokens"] for _ in range(2)]
-    assert art[0] == art[1] and len(art[0]) == 12
+    from fusekit_amd import registry
+    fam = registry.family_of(registry.read_config(d))
+    rt = fam.runtime(*fam.load(d, 64, 16))
+    rt.reset()
+    seq = [int(t) for t in ids.split(",")]
+    for t in seq:
+        logits = rt.step([t], [0])
+    want = []
+    for _ in range(12):                                     # the artifact feeds the prompt through the decode graph as well
+        want.append(int(np.argmax(logits)))
+        logits = rt.step([want[-1]], [0])
+    assert art[0] == art[1] == want
     out = run("bench", d, "--tokens", "8", "--ids", ids, "--dump-tokens", "--per-kernel")
     assert f"tokens={a[:8]}" in out
 
     # the trace runner: the same logits as the runtime's own steps
-    from fusekit_amd import registry
-    fam = registry.family_of(registry.read_config(d))
     rt = fam.runtime(*fam.load(d, 64, 32))
-    seq = [int(t) for t in ids.split(",")]
     steps = [{"step": 0, "entries": [{"id": "a", "tokens": seq[:4], "want": [1, 3]}], "end": []},
              {"step": 1, "entries": [{"id": "a", "tokens": seq[4:5], "want": []}], "end": []},
              {"step": 2, "entries": [{"id": "a", "tokens": seq[5:], "want": [0]}], "end": ["a"]},

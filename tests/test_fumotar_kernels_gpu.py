@@ -92,6 +92,23 @@ def test_product_with_column_functions(fk, act, rows, n, tail):
         assert np.abs(t.to_numpy(np.float32, (rows, tail)) - ref[:, n:]).max() <= 2e-6 * np.abs(ref).max()
 
 
+@pytest.mark.parametrize("rows,parts", [(9, 8), (33, 4), (130, 2)])
+def test_product_in_parts_of_its_sum(fk, rows, parts):
+    """One product as `parts` products over a share of k each, added where the residual takes them."""
+    g, r = Rig(16), rng(rows)
+    n, k = 100, 1024
+    ld, kp = pad(n), k // parts
+    (bx, x), (bw, w) = g.up(r.standard_normal((rows, k))), g.w16(r.standard_normal((n, k)))
+    mix, h = g.zeros(parts * rows * ld, 4), g.zeros(rows * ld)
+    g.run("dense", [bx, bw, mix], rows=rows, n=n, k=kp, ldx=k, ldw=k, ldy=ld, batch=parts, xb=kp, wb=kp, yb=rows * ld, y32=1)
+    res = padded(r.standard_normal((rows, n)).astype(np.float32), ld)
+    (bn, nw), (bb, nb), bres = g.w16(padded(r.standard_normal(n), ld)), g.w16(padded(r.standard_normal(n), ld)), g.raw(res)
+    g.run("residual_norm", [bres, mix, bn, bb, h], rows=rows, width=n, ld=ld, eps=1e-3, has_mix=1, mix_parts=parts, has_h1=1, layer_norm=1)
+    ref = res[:, :n] + x @ w.T
+    assert np.abs(bres.to_numpy(np.float32, (rows, ld))[:, :n] - ref).max() <= 2e-6 * np.abs(ref).max()
+    g.close(g.down(h, (rows, ld))[:, :n], plain.layer_norm(ref, nw[:n], nb[:n], 1e-3))
+
+
 # ---- attention ----
 
 def qk_case(g, r, rows, heads, kv, dim, dim_ld):
