@@ -230,9 +230,15 @@ __global__ __launch_bounds__(kTileThreads) void dense_tile_kernel(const TileArgs
                 if (mr >= live || n >= a.n) continue;
                 const size_t row = GROUPED ? (size_t)a.perm[m0 + mr] : (size_t)(m0 + mr);
                 if (PLAIN_OUT) {
+                    if (a.out.bias) {   // rows of whole fours: the planner has checked
+                        const float4 b = act_load4(a.out.bias + n);
+                        v[0] += b.x; v[1] += b.y; v[2] += b.z; v[3] += b.w;
+                    }
+                    const uint32_t fn = column_fn(a.out, n);   // one for the four columns
+                    if (fn != kFnNone) {
 #pragma unroll
-                    for (int r = 0; r < 4; ++r)
-                        if (n + (uint32_t)r < a.n) v[r] = column_value(a.out, n + (uint32_t)r, v[r]);
+                        for (int r = 0; r < 4; ++r) v[r] = apply_fn(fn, v[r]);
+                    }
                     if (a.out.tail && n >= a.out.tail_begin) {
                         for (uint32_t r = 0; r < 4; ++r)
                             if (n + r < a.n) a.out.tail[row * a.out.ldt + n + r - a.out.tail_begin] = v[r];
@@ -356,6 +362,7 @@ fk_status plan_dense(const DenseArgs& a, uint32_t act, Launch* out) {
         if (a.transposed || a.batch != 1) return set_error(FK_ERR_UNSUPPORTED, "dense: column functions go with one row-major product");
         if (o.fn > kFnMax || o.fn2 > kFnMax || o.begin % 4 || o.end % 4 || o.begin2 % 4 || (o.tail && (o.tail_begin % 4 || o.tail_begin > a.n || o.ldt < a.n - o.tail_begin)))
             return set_error(FK_ERR_INVALID, "dense: column functions start at multiples of four columns");
+        if (o.bias && act == 16 && (a.n % 4 || ((uintptr_t)o.bias & 7u))) return set_error(FK_ERR_INVALID, "dense: biases come in fours");
     }
     out->shmem = 0;
     out->block = dim3(256, 1, 1);

@@ -3,6 +3,8 @@
 //
 // bf16 attention itself is sdpa_decode (one row) and sdpa_prefill (portions); heads are padded with zeros to the widths
 // they take, which changes no score and no output.
+#include <algorithm>
+
 #include "act_device.hpp"
 #include "layered.hpp"
 
@@ -132,7 +134,7 @@ fk_status plan_qk_store(const QkStoreArgs& a, uint32_t act, Launch* out) {
         return set_error(FK_ERR_INVALID, "qk store: bad shape");
     if (a.rot_dims > 2 * kMaxRotPairs) return set_error(FK_ERR_UNSUPPORTED, "qk store: at most 1024 rotated dimensions");
     out->func = act == 16 ? (const void*)&qk_store_kernel<uint16_t> : (const void*)&qk_store_kernel<float>;
-    out->grid = dim3(a.rows, a.rows >= 64 ? 1 : (a.heads + a.kv_heads + kGqaWaves - 1) / kGqaWaves, 1);
+    out->grid = dim3(a.rows, std::min((a.heads + a.kv_heads + kGqaWaves - 1) / kGqaWaves, std::max(1u, 2048u / a.rows)), 1);   // enough blocks to fill the device
     out->block = dim3(kGqaBlock, 1, 1);
     out->shmem = 0;
     out->set_args(a);

@@ -340,7 +340,7 @@ struct LruScanArgs {
     const uint16_t* lam;
     float* state;             // [width]
     void* y;                  // [rows, ldy] (act): the gate branch in, the output out
-    float* carry;             // [chunks][2][width]: product of decays and end of every chunk
+    float* carry;             // [chunks][2][width]: product of decays and end of every chunk but the last, a copy of the state
     uint32_t rows, width, block, ldx, ldy;
 };
 constexpr uint32_t kLruChunk = 32;

@@ -9,10 +9,13 @@ namespace fk {
 
 namespace {
 
-constexpr uint32_t kLruAhead = 8;
-
+// One channel's constants, and its inputs for half a chunk.
 template <typename T>
 struct LruColumn {
+    static constexpr uint32_t kHalf = kLruChunk / 2;
+    struct Rows {
+        float u[kHalf], r[kHalf], i[kHalf], y[kHalf];
+    };
     const LruScanArgs& a;
     const T* u;
     const float* gr;
@@ -22,72 +25,89 @@ struct LruColumn {
         : a(args), u(reinterpret_cast<const T*>(args.u) + c), gr(args.gates + (size_t)(c / args.block) * 2u * args.block + c % args.block),
           rb(bf16_bits_to_f32(args.rb[c])), ib(bf16_bits_to_f32(args.ib[c])), rate(lru_rate(args.lam[c])) {}
 
-    // f(row, decay, addend) for rows r0 .. r1 - 1 in order, the inputs a few rows ahead
-    template <typename F>
-    __device__ __forceinline__ void walk(uint32_t r0, uint32_t r1, const F& f) const {
-        float uv[kLruAhead], rv[kLruAhead], iv[kLruAhead];
-        auto fetch = [&](uint32_t e, uint32_t r) __attribute__((always_inline)) {
-            r = r < r1 ? r : r1 - 1u;
-            uv[e] = act_load(u + (size_t)r * a.ldx);
-            rv[e] = gr[(size_t)r * 2u * a.width];
-            iv[e] = gr[(size_t)r * 2u * a.width + a.block];
-        };
+    // Requests only, all of them in flight together; rows past the pass repeat its last one.
+    template <bool GATE>
+    __device__ __forceinline__ void fetch(Rows& x, uint32_t r0, const T* y) const {
 #pragma unroll
-        for (uint32_t e = 0; e < kLruAhead; ++e) fetch(e, r0 + e);
-        for (uint32_t r = r0; r < r1; r += kLruAhead) {
-#pragma unroll
-            for (uint32_t e = 0; e < kLruAhead; ++e) {
-                if (r + e < r1) {
-                    float decay, add;
-                    if (sizeof(T) == 2) lru_step_fast(rv[e] + rb, iv[e] + ib, rate, uv[e], decay, add);
-                    else lru_step(rv[e] + rb, iv[e] + ib, rate, uv[e], decay, add);
-                    f(r + e, decay, add);
-                }
-                fetch(e, r + e + kLruAhead);
-            }
+        for (uint32_t e = 0; e < kHalf; ++e) {
+            const uint32_t r = r0 + e < a.rows ? r0 + e : a.rows - 1u;
+            x.u[e] = act_load(u + (size_t)r * a.ldx);
+            x.r[e] = gr[(size_t)r * 2u * a.width];
+            x.i[e] = gr[(size_t)r * 2u * a.width + a.block];
+            if (GATE) x.y[e] = act_load(y + (size_t)r * a.ldy);
         }
+    }
+    __device__ __forceinline__ void step(const Rows& x, uint32_t e, float& decay, float& add) const {
+        if (sizeof(T) == 2) lru_step_fast(x.r[e] + rb, x.i[e] + ib, rate, x.u[e], decay, add);
+        else lru_step(x.r[e] + rb, x.i[e] + ib, rate, x.u[e], decay, add);
     }
 };
 
+// Chunks with a successor, which are whole.
 template <typename T>
 __global__ __launch_bounds__(64) void lru_ends_kernel(const LruScanArgs a) {
+    using Column = LruColumn<T>;
     const uint32_t c = blockIdx.x * 64u + threadIdx.x, r0 = blockIdx.y * kLruChunk;
     if (c >= a.width) return;
-    const LruColumn<T> col(a, c);
+    const Column col(a, c);
+    typename Column::Rows x[2];
+    col.template fetch<false>(x[0], r0, nullptr);
+    col.template fetch<false>(x[1], r0 + Column::kHalf, nullptr);
     float prod = 1.f, end = 0.f;
-    col.walk(r0, r0 + kLruChunk, [&](uint32_t, float decay, float add) __attribute__((always_inline)) {   // the last chunk has no successor: whole chunks only
-        prod *= decay;
-        end = fmaf(decay, end, add);
-    });
+#pragma unroll
+    for (uint32_t h = 0; h < 2; ++h)
+#pragma unroll
+        for (uint32_t e = 0; e < Column::kHalf; ++e) {
+            float decay, add;
+            col.step(x[h], e, decay, add);
+            prod *= decay;
+            end = fmaf(decay, end, add);
+        }
     float* o = a.carry + (size_t)blockIdx.y * 2u * a.width + c;
     o[0] = prod;
     o[a.width] = end;
+    // the last chunk of the next launch replaces the state while others still start from it: they read this copy
+    if (blockIdx.y == 0) a.carry[(size_t)gridDim.y * 2u * a.width + c] = a.state[c];
 }
 
 template <typename T>
 __global__ __launch_bounds__(64) void lru_out_kernel(const LruScanArgs a) {
+    using Column = LruColumn<T>;
     const uint32_t c = blockIdx.x * 64u + threadIdx.x, chunk = blockIdx.y, r0 = chunk * kLruChunk;
     if (c >= a.width) return;
-    const uint32_t r1 = r0 + kLruChunk < a.rows ? r0 + kLruChunk : a.rows;
-    const LruColumn<T> col(a, c);
-    float S = a.state[c];
-    const float* e = a.carry + c;
-#pragma unroll 4
-    for (uint32_t k = 0; k < chunk; ++k) S = fmaf(e[(size_t)k * 2u * a.width], S, e[(size_t)k * 2u * a.width + a.width]);
+    const Column col(a, c);
     T* y = reinterpret_cast<T*>(a.y) + c;
-    col.walk(r0, r1, [&](uint32_t r, float decay, float add) __attribute__((always_inline)) {
-        S = fmaf(decay, S, add);
-        T* p = y + (size_t)r * a.ldy;
-        act_store(p, S * act_load(p));
-    });
-    if (r1 != a.rows) return;
-    if (gridDim.y == 1u) a.state[c] = S;
-    else a.carry[(size_t)chunk * 2u * a.width + c] = S;   // other chunks still read the state: a launch of its own replaces it
-}
-
-__global__ __launch_bounds__(256) void lru_state_kernel(const LruScanArgs a) {
-    const uint32_t c = blockIdx.x * 256u + threadIdx.x, chunk = (a.rows - 1u) / kLruChunk;
-    if (c < a.width) a.state[c] = a.carry[(size_t)chunk * 2u * a.width + c];
+    typename Column::Rows x[2];
+    col.template fetch<true>(x[0], r0, y);
+    col.template fetch<true>(x[1], r0 + Column::kHalf, y);
+    const float* e = a.carry + c;
+    float S = gridDim.y == 1u ? a.state[c] : e[(size_t)(gridDim.y - 1u) * 2u * a.width];
+    constexpr uint32_t kPrefix = 16;   // chunks whose ends are requested together
+    for (uint32_t k0 = 0; k0 < chunk; k0 += kPrefix) {
+        float d[kPrefix], b[kPrefix];
+#pragma unroll
+        for (uint32_t i = 0; i < kPrefix; ++i) {
+            const size_t k = k0 + i < chunk ? k0 + i : chunk - 1u;
+            d[i] = e[k * 2u * a.width];
+            b[i] = e[k * 2u * a.width + a.width];
+        }
+#pragma unroll
+        for (uint32_t i = 0; i < kPrefix; ++i)
+            if (k0 + i < chunk) S = fmaf(d[i], S, b[i]);
+    }
+#pragma unroll
+    for (uint32_t h = 0; h < 2; ++h)
+#pragma unroll
+        for (uint32_t i = 0; i < Column::kHalf; ++i) {
+            const uint32_t r = r0 + h * Column::kHalf + i;
+            if (r < a.rows) {
+                float decay, add;
+                col.step(x[h], i, decay, add);
+                S = fmaf(decay, S, add);
+                act_store(y + (size_t)r * a.ldy, S * x[h].y[i]);
+            }
+        }
+    if (r0 + kLruChunk >= a.rows) a.state[c] = S;
 }
 
 }  // namespace
@@ -112,13 +132,7 @@ fk_status plan_lru_scan(const LruScanArgs& a, uint32_t act, Launch* out) {
     out->block = dim3(64, 1, 1);
     out->shmem = 0;
     out->set_args(a);
-    Launch st;
-    st.func = (const void*)&lru_state_kernel;
-    st.grid = dim3((a.width + 255) / 256, 1, 1);
-    st.block = dim3(256, 1, 1);
-    st.set_args(a);
     out->then.push_back(fin);
-    out->then.push_back(st);
     return FK_OK;
 }
 

@@ -81,9 +81,9 @@ def test_product_with_column_functions(fk, act, rows, n, tail):
     k, N = 128, n + tail
     (bx, x), (bw, w), (bb, b) = g.up(r.standard_normal((rows, k))), g.w16(r.standard_normal((N, k)) * 0.2), g.w16(r.standard_normal(N))
     y, t = g.zeros(rows * n), g.zeros(rows * max(tail, 1), 4)
-    more = dict(tail_begin=n, ldt=tail) if tail else {}
-    g.run("dense", [bx, bw, bb, y] + ([t] if tail else []), rows=rows, n=N, k=k, ldx=k, ldw=k, ldy=n, has_bias=1, fn=2, fn_begin=64, fn_end=n - 64, fn2=1, fn2_begin=n - 64 if not tail else N + 3 & ~3, **more)
-    ref = x @ w.T + b
+    more = dict(tail_begin=n, ldt=tail, fn2_begin=pad(N, 4)) if tail else dict(has_bias=1, fn2_begin=n - 64)
+    g.run("dense", [bx, bw] + ([y, t] if tail else [bb, y]), rows=rows, n=N, k=k, ldx=k, ldw=k, ldy=n, fn=2, fn_begin=64, fn_end=n - 64, fn2=1, **more)
+    ref = x @ w.T + (0.0 if tail else b)
     got = g.down(y, (rows, n))
     g.close(got[:, :64], ref[:, :64])
     g.close(got[:, 64:n - 64], plain.gelu_tanh(ref[:, 64:n - 64]))
