@@ -174,7 +174,7 @@ def _graph_dict(rt: DecoderRuntime, task_list: List[Dispatch], graph_id: int, sy
         decode_pipeline=[t["id"] for t in tasks],
         decode_capabilities=dict(dispatchable=True, reasons=[]),
         uniforms=uniforms,
-        model_config=dict(dataclasses.asdict(c), config_class=type(c).__name__))
+        model_config=dict(dataclasses.asdict(c), config_class=type(c).__name__, **({"max_positions": c.max_positions} if hasattr(c, "max_positions") else {})))
 
 
 def write_artifact(rt: DecoderRuntime, out_dir: str, model_name: str = "synthetic", prefill_variants=()) -> None:
@@ -311,6 +311,9 @@ class ArtifactRuntime:
         return nxt
 
     def generate(self, prompt, max_tokens: int) -> List[int]:
+        limit = self.model_config.get("max_positions")
+        if limit is not None and len(prompt) + max_tokens - 1 > limit:
+            raise ValueError(f"the sequence would exceed the cache's {limit} positions")
         for name, buf in self.scratch.items():   # recurrent states of a new sequence start at zero
             if name.startswith("state."):
                 native.fill_u32(buf, 0, buf.nbytes // 4)

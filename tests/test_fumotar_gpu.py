@@ -247,6 +247,8 @@ def test_command_line_artifact_and_trace(fk, tmp_path, capsys, monkeypatch):
         want.append(int(np.argmax(logits)))
         logits = rt.step([want[-1]], [0])
     assert art[0] == art[1] == want
+    with pytest.raises(ValueError, match="1024 positions"):
+        run("generate", "--model", d, "--artifact", d + "/.fusekit", "--ids", ids, "--max-tokens", "1030")
     out = run("bench", d, "--tokens", "8", "--ids", ids, "--dump-tokens", "--per-kernel")
     assert f"tokens={a[:8]}" in out
 
