@@ -37,13 +37,13 @@ def joint_config(s: dict, rows_per_pass: int = 2048, capacity: int = 4096):
     from .joint_layers import CausalAttention, ChannelDelta, DenseMlp, RgLru, RotaryScaling
     from .layer_decoder import Layer, LayerConfig, PairTable
     att = CausalAttention(heads=s["heads"], kv_heads=s["kv_heads"], dim=128, scale=128 ** -0.5, rot_base=1e5, rot_dims=128,
-                          rot_scaling=RotaryScaling(factor=4.0, original=4096, fast=32.0, slow=1.0))
+                          rot_scaling=RotaryScaling(factor=4.0, original=4096, fast=24.0, slow=1.5))
     dlt = ChannelDelta(heads=s["delta_heads"], kv_heads=s["delta_heads"], dim=128, vdim=128, conv=4, decay_rank=s["rank"], gate_rank=s["rank"])
     lru = RgLru(width=s["width"], blocks=s["blocks"], conv=4)
     mlp = DenseMlp(s["ff"])
     return LayerConfig(width=s["width"], vocab=s["vocab"], layers=[Layer((dlt, lru, att)[i % 3], mlp) for i in range(LAYERS)], rows_per_pass=rows_per_pass,
                        capacity=capacity, design="Fumotar", layer_norm=True, tied=True, join=True, loop_start=0, loop_stop=LAYERS, loop_times=1,
-                       pairs=PairTable(buckets=65535, mul_prev=31, mul_cur=17))
+                       pairs=PairTable(buckets=65535, mul_prev=8191, mul_cur=127))
 
 
 def like_joint_config(s: dict, rows_per_pass: int = 2048):
